@@ -181,13 +181,16 @@ def rotary_table(n_pos: int, rot: dict, device) -> torch.Tensor:
     """fp32 [n_pos, dims]: cos | sin of position * frequency (rotate-half pairing, ``dims / 2`` frequencies
     base^(-2i/dims)). With ``rot["scaling"]`` (YaRN: factor, original, fast, slow) frequency i is blended between
     f_i (fast-turning dimensions) and f_i / factor (slow ones) by a linear ramp between the dimensions that make
-    ``fast`` and ``slow`` turns over the original context, and cos / sin are scaled by 0.1 ln(factor) + 1."""
+    ``fast`` and ``slow`` turns over the original context, and cos / sin are scaled by 0.1 ln(factor) + 1. A scaling
+    entry with nothing but a factor is linear: every frequency is divided by it."""
     dims, base = int(rot["dims"]), float(rot["base"])
     half = dims // 2
     f = torch.tensor([base ** (-2.0 * i / dims) for i in range(half)], dtype=torch.float64)
     mag = 1.0
     sc = rot.get("scaling")
-    if sc:
+    if sc and set(sc) == {"factor"}:
+        f = f / float(sc["factor"])
+    elif sc:
         factor, orig = float(sc["factor"]), float(sc["original"])
 
         def turns_dim(t: float) -> float:

@@ -223,6 +223,39 @@ MAGEDRA_PRESETS: dict[str, dict] = {
 }
 
 
+def _rogosun(width: int, heads: int, kv_heads: int, n_layers: int, vocab: int, ff: int, experts: int = 8, top: int = 2,
+             expert_ff: int | None = None, head_dim: int = 128) -> dict:
+    """A Rogosun config dict at transformer-like sizes: layers alternate gated linear attention (``width / 256`` heads of
+    128 x 256) and parallel (grouped-query attention beside a delta rule of ``width / 128`` heads of 128 x 128); two
+    layers of four with the dense feed-forward of ``ff`` rows, two with ``experts`` routed experts in 4 groups (2 kept)
+    of ``expert_ff`` rows and a shared one of the same size."""
+    e = expert_ff or ff // 4
+    moe = {"kind": "moe", "expert": {"ff": e}, "shared": {"ff": e},
+           "router": {"experts": experts, "top": top, "scale": 2.5,
+                      "groups": {"count": 4 if experts % 4 == 0 else 1, "keep": 2 if experts % 4 == 0 else 1}}}
+    layers = []
+    for i in range(n_layers):
+        mlp = moe if i % 4 in (1, 2) else {"kind": "dense", "ff": ff}
+        if i % 2 == 0:
+            layers.append({"type": "gla", "mixer": {"heads": max(1, width // 256), "dim": 128, "vdim": 256,
+                                                    "tau": 16.0}, "mlp": mlp})
+        else:
+            left = {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim,
+                    "rot": {"base": 100000.0, "dims": head_dim, "scaling": {"factor": 4.0}}, "scale": head_dim ** -0.5}
+            n = max(1, width // 128)
+            right = {"heads": n, "kv_heads": n, "dim": 128, "vdim": 128, "conv": 4}
+            layers.append({"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.7,
+                                                         "right_scale": 0.7}, "mlp": mlp})
+    return {"architecture": "Rogosun", "vocab": vocab, "width": width, "layers": layers, "norm": {"eps": 1e-6}}
+
+
+ROGOSUN_PRESETS: dict[str, dict] = {
+    # widths, heads and vocabularies of the Llama presets above; 8 experts of ff / 4 rows, top 2 (random init)
+    "rogosun-small": _rogosun(1024, 8, 2, 8, 128256, 3584, expert_ff=768),
+    "rogosun-tiny": _rogosun(512, 8, 2, 4, 32000, 1024, experts=4, expert_ff=256, head_dim=64),
+}
+
+
 def _budurax_config(c: dict, name: str):
     from kafka_llm_service_amd.models.budurax import BuduraxConfig
 
@@ -247,17 +280,23 @@ def _magedra_config(c: dict, name: str):
     return MagedraConfig.from_dict(c, name=name)
 
 
+def _rogosun_config(c: dict, name: str):
+    from kafka_llm_service_amd.models.rogosun import RogosunConfig
+
+    return RogosunConfig.from_dict(c, name=name)
+
+
 # config.json "architecture" (lower case) -> config class of a model family that names itself there
 ARCH_CONFIGS = {"budurax": _budurax_config, "lisorax": _lisorax_config, "mozidra": _mozidra_config,
-                "magedra": _magedra_config}
+                "magedra": _magedra_config, "rogosun": _rogosun_config}
 # model families whose kernels are built for float32 as well as bfloat16 (EngineConfig.dtype)
-FP32_ARCHS = ("budurax", "lisorax", "mozidra", "magedra")
+FP32_ARCHS = ("budurax", "lisorax", "mozidra", "magedra", "rogosun")
 
 
 def _from_json(path: Path):
     """A config.json names its model class: ``"architecture": "Budurax"`` (models/budurax.py), ``"Lisorax"``
-    (models/lisorax.py), ``"Mozidra"`` (models/mozidra.py), ``"Magedra"`` (models/magedra.py), else HF Llama /
-    Mixtral."""
+    (models/lisorax.py), ``"Mozidra"`` (models/mozidra.py), ``"Magedra"`` (models/magedra.py), ``"Rogosun"``
+    (models/rogosun.py), else HF Llama / Mixtral."""
     c = json.loads(path.read_text())
     make = ARCH_CONFIGS.get(str(c.get("architecture", "")).lower())
     if make is not None:
@@ -276,9 +315,11 @@ def get_config(name: str):
         return _mozidra_config(MOZIDRA_PRESETS[name], name)
     if name in MAGEDRA_PRESETS:
         return _magedra_config(MAGEDRA_PRESETS[name], name)
+    if name in ROGOSUN_PRESETS:
+        return _rogosun_config(ROGOSUN_PRESETS[name], name)
     p = Path(name)
     if p.is_dir() and (p / "config.json").exists():
         return _from_json(p / "config.json")
     if p.suffix == ".json" and p.exists():
         return _from_json(p)
-    raise KeyError(f"unknown model {name!r}; presets: {sorted(PRESETS) + sorted(BUDURAX_PRESETS) + sorted(LISORAX_PRESETS) + sorted(MOZIDRA_PRESETS) + sorted(MAGEDRA_PRESETS)}")
+    raise KeyError(f"unknown model {name!r}; presets: {sorted(PRESETS) + sorted(BUDURAX_PRESETS) + sorted(LISORAX_PRESETS) + sorted(MOZIDRA_PRESETS) + sorted(MAGEDRA_PRESETS) + sorted(ROGOSUN_PRESETS)}")

@@ -1,4 +1,4 @@
-// Python bindings of the hybrid-family kernels (hybrid.hip). Shapes, dtypes, strides and index ranges that the
+// Python bindings of the hybrid-family kernels (hybrid*.hip). Shapes, dtypes, strides and index ranges that the
 // kernels assume are checked here, so a malformed call raises instead of launching.
 #include <torch/extension.h>
 #include <c10/hip/HIPStream.h>
@@ -80,7 +80,7 @@ hipError_t kafka_hy_mlstm_scan(int f32, const void* qkv, int64_t qs, const float
                                int64_t os, hipStream_t st);
 hipError_t kafka_hy_head_norm_gate(int f32, const float* o, int64_t os_, const void* w, const void* g, int64_t gs,
                                    int g_off, int H, int Dv, float eps, void* out, int64_t outs, int64_t T,
-                                   float scale, hipStream_t st);
+                                   float scale, int silu, hipStream_t st);
 int kafka_hy_router_max_e();
 int kafka_hy_router_max_k();
 hipError_t kafka_hy_moe_topk(const float* logits, int64_t ls, int E, int k, float* tw, int* te, int64_t T,
@@ -111,18 +111,19 @@ int kafka_hy_window_attn_max_dv();
 hipError_t kafka_hy_window_attn(int f32, const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                 int bt_stride, const int* tok_seg, const int64_t* positions, int H, int G, int D,
                                 int Dv, float scale, int window, const float* sink, void* out, int64_t os, int64_t T,
-                                int shared_keys, hipStream_t st);
+                                int shared_keys, float out_scale, hipStream_t st);
 int kafka_hy_window_attn_mfma_ok(int page, int D, int Dv, int rep);
 hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                      int bt_stride, const int* items, int n_items, const int64_t* positions, int H,
                                      int G, int D, int Dv, float scale, int window, const float* sink, void* out,
                                      int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
-                                     hipStream_t st);
+                                     float out_scale, hipStream_t st);
 int kafka_hy_grouped_router_max_e();
 int kafka_hy_grouped_router_max_k();
 int kafka_hy_grouped_router_max_g();
 hipError_t kafka_hy_moe_topk_grouped(const float* logits, int64_t ls, int E, int k, const float* corr, int groups,
-                                     int keep, float eps, float* tw, int* te, float* gate, int64_t T, hipStream_t st);
+                                     int keep, float eps, float* tw, int* te, float* gate, int64_t T, int sigmoid,
+                                     int top2, int norm, float scale, hipStream_t st);
 
 // gated recurrences beside attention, rotation + head mix + paged store (hybrid_parallel.hip)
 hipError_t kafka_hy_act_norm(int f32, const void* x, int64_t xs, int c0, int n, const float* w, float eps, void* out,
@@ -146,8 +147,28 @@ hipError_t kafka_hy_hgrn2_combine(const int* cs, int R, const float* F, int HD, 
 int kafka_hy_rope_store_max_q();
 hipError_t kafka_hy_rope_kv_store(int f32, const void* qkv, int64_t qs, int H, int G, int D, int Dv,
                                   const int64_t* positions, const float* cos_sin, int dims, int pairs,
-                                  const float* talk, void* kc, void* vt, const int64_t* slots, void* q_out, int64_t qos,
-                                  int64_t T, hipStream_t st);
+                                  const float* talk, const float* qn, const float* kn, float eps, int v_off, void* kc,
+                                  void* vt, const int64_t* slots, void* q_out, int64_t qos, int64_t T, hipStream_t st);
+
+// post-normed residual, linear-attention recurrences (hybrid_linear.hip)
+int kafka_hy_norm_add_max_slabs();
+hipError_t kafka_hy_norm_add(int f32, float* x, int64_t xs, const void* y1, int64_t y1s, int y1_f32, int S, int64_t slab,
+                             const void* y2, int64_t y2s, const float* w, float eps, void* out, int64_t os, int64_t T,
+                             int d, hipStream_t st);
+hipError_t kafka_hy_ff_act(int f32, const void* u, int64_t us, void* out, int64_t os, int64_t T, int F, int glu,
+                           hipStream_t st);
+int kafka_hy_lin_max_d();
+int kafka_hy_lin_chunk();
+hipError_t kafka_hy_lin_scan(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
+                             const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
+                             int64_t beta_s, int H, int G, int D, int Dv, float qscale, float inv_tau, const int* seg,
+                             int R, int max_n, float* S, float* out, int64_t os, hipStream_t st);
+int64_t kafka_hy_lin_chunk_scratch(int D, int Dv, int delta);
+hipError_t kafka_hy_lin_chunked(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
+                                const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
+                                int64_t beta_s, int H, int G, int D, int Dv, float qscale, float inv_tau,
+                                const int* vseg, int n_chunks, const int* cs, int R, float* scratch, float* S,
+                                float* out, int64_t os, hipStream_t st);
 }
 
 namespace {
@@ -667,7 +688,7 @@ void mlstm_scan(at::Tensor qkv, at::Tensor gates, int64_t H, int64_t D, int64_t 
 }
 
 void head_norm_gate(at::Tensor o, at::Tensor w, OptT g, int64_t g_off, int64_t H, double eps, at::Tensor out,
-                    double scale) {
+                    double scale, bool silu) {
   rows2d(o, "o"); rows2d(out, "out"); f32t(o, "o");
   const int f32 = act_f32(out);
   same_act(f32, {&w});
@@ -681,7 +702,8 @@ void head_norm_gate(at::Tensor o, at::Tensor w, OptT g, int64_t g_off, int64_t H
     gp = g->data_ptr(); gs = g->stride(0);
   }
   HY_HIP(kafka_hy_head_norm_gate(f32, o.data_ptr<float>(), o.stride(0), w.data_ptr(), gp, gs, (int)g_off, (int)H,
-                                 (int)(n / H), (float)eps, out.data_ptr(), out.stride(0), T, (float)scale, stream()));
+                                 (int)(n / H), (float)eps, out.data_ptr(), out.stride(0), T, (float)scale, silu ? 1 : 0,
+                                 stream()));
 }
 
 void moe_topk(at::Tensor logits, at::Tensor tw, at::Tensor te) {
@@ -847,7 +869,8 @@ void qk_norm_rope_store(at::Tensor qkv, int64_t H, int64_t G, int64_t D, int64_t
 }
 
 void window_attn(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::Tensor tok_seg, at::Tensor positions,
-                 int64_t H, int64_t G, double scale, int64_t window, OptT sink, at::Tensor out, bool shared_keys) {
+                 int64_t H, int64_t G, double scale, int64_t window, OptT sink, at::Tensor out, bool shared_keys,
+                 double out_scale) {
   rows2d(q, "q"); rows2d(out, "out");
   const int f32 = act_f32(q);
   same_act(f32, {&kc, &vt, &out});
@@ -867,14 +890,14 @@ void window_attn(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::
   HY_HIP(kafka_hy_window_attn(f32, q.data_ptr(), q.stride(0), kc.data_ptr(), vt.data_ptr(), bt.data_ptr<int>(),
                               (int)bt.stride(0), tok_seg.data_ptr<int>(), positions.data_ptr<int64_t>(), (int)H, (int)G,
                               (int)D, (int)Dv, (float)scale, (int)window, sink_ptr(sink, H), out.data_ptr(),
-                              out.stride(0), T, shared_keys ? 1 : 0, stream()));
+                              out.stride(0), T, shared_keys ? 1 : 0, (float)out_scale, stream()));
 }
 
 // the matrix-core kernel: items int32 [n, 4] = (first row, tokens, segment, 0), each at most 32 (token, query head of
 // one key/value head) rows of one segment
 void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::Tensor items, int64_t tile_tokens,
                       at::Tensor positions, int64_t H, int64_t G, double scale, int64_t window, OptT sink,
-                      at::Tensor out, int64_t nsplit, OptT po, OptT pml, bool shared_keys) {
+                      at::Tensor out, int64_t nsplit, OptT po, OptT pml, bool shared_keys, double out_scale) {
   for (const at::Tensor* t : {&q, &kc, &vt, &out})
     TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16, "window_attn_mfma: bf16 GPU tensors");
   rows2d(q, "q"); rows2d(out, "out");
@@ -907,11 +930,11 @@ void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt,
                                    (int)bt.stride(0), items.data_ptr<int>(), (int)items.size(0),
                                    positions.data_ptr<int64_t>(), (int)H, (int)G, (int)D, (int)Dv, (float)scale,
                                    (int)window, sink_ptr(sink, H), out.data_ptr(), out.stride(0), (int)nsplit, pop,
-                                   pmlp, T, shared_keys ? 1 : 0, stream()));
+                                   pmlp, T, shared_keys ? 1 : 0, (float)out_scale, stream()));
 }
 
-void moe_topk_grouped(at::Tensor logits, int64_t E, at::Tensor corr, int64_t groups, int64_t keep, double eps,
-                      at::Tensor tw, at::Tensor te, OptT gate) {
+void moe_topk_grouped(at::Tensor logits, int64_t E, OptT corr, int64_t groups, int64_t keep, double eps,
+                      at::Tensor tw, at::Tensor te, OptT gate, bool sigmoid, bool top2, bool norm, double scale) {
   rows2d(logits, "logits"); f32t(logits, "logits"); f32t(tw, "weights");
   const int64_t T = logits.size(0);
   TORCH_CHECK(tw.is_contiguous() && tw.dim() == 2 && tw.size(0) == T && te.is_cuda() && te.is_contiguous() &&
@@ -927,7 +950,8 @@ void moe_topk_grouped(at::Tensor logits, int64_t E, at::Tensor corr, int64_t gro
   HY_HIP(kafka_hy_moe_topk_grouped(logits.data_ptr<float>(), logits.stride(0), (int)E, (int)k,
                                    f32vec(corr, E, "correction"), (int)groups, (int)keep, (float)eps,
                                    tw.data_ptr<float>(), te.data_ptr<int>(),
-                                   const_cast<float*>(f32vec(gate, T, "gate")), T, stream()));
+                                   const_cast<float*>(f32vec(gate, T, "gate")), T, sigmoid ? 1 : 0, top2 ? 1 : 0,
+                                   norm ? 1 : 0, (float)scale, stream()));
 }
 
 void act_norm(at::Tensor x, int64_t c0, int64_t n, at::Tensor w, double eps, at::Tensor out, bool center) {
@@ -1000,12 +1024,13 @@ void hgrn2_scan(at::Tensor proj, int64_t q_off, int64_t f_off, int64_t v_off, at
 
 void rope_kv_store(at::Tensor qkv, int64_t H, int64_t G, int64_t D, int64_t Dv, at::Tensor positions, OptT cos_sin,
                    int64_t dims, bool pairs, OptT talk, at::Tensor kc, at::Tensor vt, at::Tensor slots,
-                   at::Tensor q_out) {
+                   at::Tensor q_out, OptT q_norm, OptT k_norm, double eps, int64_t v_off) {
   rows2d(qkv, "qkv"); rows2d(q_out, "q_out");
   const int f32 = act_f32(qkv);
   same_act(f32, {&kc, &vt, &q_out});
   const int64_t T = qkv.size(0);
-  TORCH_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0 && qkv.size(1) >= H * D + G * D + G * Dv &&
+  TORCH_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && Dv > 0 && qkv.size(1) >= H * D + G * D && v_off >= 0 &&
+                  v_off + G * Dv <= qkv.size(1) && q_norm.has_value() == k_norm.has_value() &&
                   q_out.size(0) == T && q_out.size(1) == (talk.has_value() ? H * G * D : H * D),
               "rope_kv_store: head sizes (q_out [T, H D], or [T, H G D] with a head mix)");
   TORCH_CHECK(dims >= 0 && dims % 2 == 0 && dims <= D && cos_sin.has_value() == (dims > 0),
@@ -1023,7 +1048,8 @@ void rope_kv_store(at::Tensor qkv, int64_t H, int64_t G, int64_t D, int64_t Dv, 
   // positions index the table's rows and slots the cache on the device: the step plan keeps both in range
   HY_HIP(kafka_hy_rope_kv_store(f32, qkv.data_ptr(), qkv.stride(0), (int)H, (int)G, (int)D, (int)Dv,
                                 positions.data_ptr<int64_t>(), dims > 0 ? cos_sin->data_ptr<float>() : nullptr,
-                                (int)dims, pairs ? 1 : 0, f32vec(talk, H * H, "head mix"), kc.data_ptr(), vt.data_ptr(),
+                                (int)dims, pairs ? 1 : 0, f32vec(talk, H * H, "head mix"), f32vec(q_norm, D, "q norm"),
+                                f32vec(k_norm, D, "k norm"), (float)eps, (int)v_off, kc.data_ptr(), vt.data_ptr(),
                                 slots.data_ptr<int64_t>(), q_out.data_ptr(), q_out.stride(0), T, stream()));
 }
 
@@ -1050,6 +1076,96 @@ void hgrn2_chunk_combine(at::Tensor cs, at::Tensor F, at::Tensor tmp, at::Tensor
   HY_HIP(kafka_hy_hgrn2_combine(cs.data_ptr<int>(), (int)cs.size(0), F.data_ptr<float>(),
                                 (int)(tmp.size(1) * tmp.size(2)), (int)tmp.size(3), tmp.data_ptr<float>(),
                                 state.data_ptr<float>(), stream()));
+}
+
+void norm_add(at::Tensor x, at::Tensor y1, OptT y2, at::Tensor w, double eps, OptT out) {
+  rows2d(x, "x"); f32t(x, "x"); f32t(w, "w");
+  const int64_t T = x.size(0), d = x.size(1);
+  vec(w, d, "w");
+  TORCH_CHECK(x.stride(0) >= d && y1.is_cuda(), "norm_add: rows");
+  const int y1f = act_f32(y1);
+  int64_t S = 1, slab = 0, y1s;
+  if (y1.dim() == 3) {   // split-K slabs
+    TORCH_CHECK(y1f && y1.stride(2) == 1 && y1.size(1) == T && y1.size(2) == d && y1.size(0) >= 1 &&
+                    y1.size(0) <= kafka_hy_norm_add_max_slabs(), "norm_add: slabs fp32 [splits, T, d]");
+    S = y1.size(0); slab = y1.stride(0); y1s = y1.stride(1);
+  } else {
+    rows2d(y1, "y1");
+    TORCH_CHECK(y1.size(0) == T && y1.size(1) == d, "norm_add: y1 shape");
+    y1s = y1.stride(0);
+  }
+  int f32 = y1f;   // the activation dtype is the output's, else y2's, else y1's
+  const void* p2 = nullptr; int64_t s2 = 0; void* op = nullptr; int64_t os = 0;
+  if (out.has_value()) f32 = act_f32(*out);
+  else if (y2.has_value()) f32 = act_f32(*y2);
+  TORCH_CHECK(y1f || !f32, "norm_add: y1 is fp32 or of the activation dtype");
+  if (y2.has_value()) {
+    rows2d(*y2, "y2"); same_act(f32, {&*y2});
+    TORCH_CHECK(y2->size(0) == T && y2->size(1) == d, "norm_add: y2 shape");
+    p2 = y2->data_ptr(); s2 = y2->stride(0);
+  }
+  if (out.has_value()) {
+    rows2d(*out, "out"); same_act(f32, {&*out});
+    TORCH_CHECK(out->size(0) == T && out->size(1) == d, "norm_add: out shape");
+    op = out->data_ptr(); os = out->stride(0);
+  }
+  HY_HIP(kafka_hy_norm_add(f32, x.data_ptr<float>(), x.stride(0), y1.data_ptr(), y1s, y1f, (int)S, slab, p2, s2,
+                           w.data_ptr<float>(), (float)eps, op, os, T, (int)d, stream()));
+}
+
+void ff_act(at::Tensor u, at::Tensor out, bool glu) {
+  rows2d(u, "u"); rows2d(out, "out");
+  const int f32 = act_f32(u);
+  same_act(f32, {&out});
+  const int64_t T = out.size(0), F = out.size(1);
+  TORCH_CHECK(u.size(0) == T && u.size(1) == (glu ? 2 * F : F), "ff_act: shapes");
+  HY_HIP(kafka_hy_ff_act(f32, u.data_ptr(), u.stride(0), out.data_ptr(), out.stride(0), T, (int)F, glu ? 1 : 0,
+                         stream()));
+}
+
+// The linear-attention recurrence. rate / beta given: gated delta rule. vseg / cs given: the segments of cs in chunks
+// (the tables come from ops.hybrid.lin_chunk_tables, which keeps chunks inside their segments and numbers them
+// 0 .. n - 1); else seg's segments of up to max_n rows token by token.
+void lin_scan(at::Tensor qk, int64_t q_off, int64_t k_off, at::Tensor v, at::Tensor z, at::Tensor z_bias, OptT rate,
+              OptT beta, int64_t H, int64_t G, int64_t D, int64_t Dv, double qscale, double inv_tau, at::Tensor seg,
+              int64_t max_n, OptT cs, at::Tensor S, at::Tensor out) {
+  rows2d(qk, "qk"); rows2d(v, "v"); rows2d(z, "z"); rows2d(out, "out");
+  f32t(z_bias, "z_bias"); f32t(S, "S"); f32t(out, "out");
+  const int f32 = act_f32(qk);
+  same_act(f32, {&v, &z});
+  const int64_t T = qk.size(0);
+  seg_only(seg);
+  TORCH_CHECK(H >= 1 && G >= 1 && H % G == 0 && D >= 1 && Dv >= 1 && D <= kafka_hy_lin_max_d(),
+              "lin_scan: head sizes (dim up to ", kafka_hy_lin_max_d(), ")");
+  TORCH_CHECK(q_off >= 0 && q_off + G * D <= qk.size(1) && k_off >= 0 && k_off + G * D <= qk.size(1) &&
+                  v.size(0) == T && v.size(1) == H * Dv && z.size(0) == T && z.size(1) == H * D && out.size(0) == T &&
+                  out.size(1) == H * Dv, "lin_scan: shapes");
+  vec(z_bias, H * D, "z_bias");
+  TORCH_CHECK(rate.has_value() == beta.has_value(), "lin_scan: the delta rule needs rate and beta");
+  const void* bp = nullptr; int64_t bst = 0;
+  if (beta.has_value()) {
+    rows2d(*beta, "beta"); same_act(f32, {&*beta});
+    TORCH_CHECK(beta->size(0) == T && beta->size(1) == H, "lin_scan: beta [T, H]");
+    bp = beta->data_ptr(); bst = beta->stride(0);
+  }
+  const float* rp = f32vec(rate, H, "rate");
+  TORCH_CHECK(S.is_contiguous() && S.dim() == 4 && S.size(1) == H && S.size(2) == D && S.size(3) == Dv,
+              "lin_scan: state fp32 [slots, H, D, Dv]");
+  if (cs.has_value()) {
+    seg_only(*cs);
+    const int64_t n = seg.size(0);
+    auto scratch = at::empty({n * H * kafka_hy_lin_chunk_scratch((int)D, (int)Dv, rp != nullptr)}, S.options());
+    HY_HIP(kafka_hy_lin_chunked(f32, qk.data_ptr(), qk.stride(0), (int)q_off, (int)k_off, v.data_ptr(), v.stride(0),
+                                z.data_ptr(), z.stride(0), z_bias.data_ptr<float>(), rp, bp, bst, (int)H, (int)G,
+                                (int)D, (int)Dv, (float)qscale, (float)inv_tau, seg.data_ptr<int>(), (int)n,
+                                cs->data_ptr<int>(), (int)cs->size(0), scratch.data_ptr<float>(), S.data_ptr<float>(),
+                                out.data_ptr<float>(), out.stride(0), stream()));
+    return;
+  }
+  HY_HIP(kafka_hy_lin_scan(f32, qk.data_ptr(), qk.stride(0), (int)q_off, (int)k_off, v.data_ptr(), v.stride(0),
+                           z.data_ptr(), z.stride(0), z_bias.data_ptr<float>(), rp, bp, bst, (int)H, (int)G, (int)D,
+                           (int)Dv, (float)qscale, (float)inv_tau, seg.data_ptr<int>(), (int)seg.size(0), (int)max_n,
+                           S.data_ptr<float>(), out.data_ptr<float>(), out.stride(0), stream()));
 }
 
 }  // namespace
@@ -1090,7 +1206,7 @@ void kafka_bind_hybrid(pybind11::module_& m) {
         py::arg("state"), py::arg("out"), py::arg("max_rows") = 0);
   m.def("hy_mlstm_scan", &mlstm_scan);
   m.def("hy_head_norm_gate", &head_norm_gate, py::arg("o"), py::arg("w"), py::arg("g"), py::arg("g_off"), py::arg("H"),
-        py::arg("eps"), py::arg("out"), py::arg("scale") = 1.0);
+        py::arg("eps"), py::arg("out"), py::arg("scale") = 1.0, py::arg("silu") = false);
   m.def("hy_moe_topk", &moe_topk);
   m.def("hy_moe_rows", &moe_rows, py::arg("h"), py::arg("wgu"), py::arg("wd"), py::arg("tw"), py::arg("te"),
         py::arg("a"), py::arg("out"), py::arg("limit") = 0.0, py::arg("alpha") = 1.0);
@@ -1104,13 +1220,13 @@ void kafka_bind_hybrid(pybind11::module_& m) {
   m.def("hy_qk_norm_rope_store", &qk_norm_rope_store);
   m.def("hy_window_attn", &window_attn, py::arg("q"), py::arg("kc"), py::arg("vt"), py::arg("bt"), py::arg("tok_seg"),
         py::arg("positions"), py::arg("H"), py::arg("G"), py::arg("scale"), py::arg("window"), py::arg("sink"),
-        py::arg("out"), py::arg("shared_keys") = false);
+        py::arg("out"), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0);
   m.def("hy_window_attn_mfma_ok",
         [](int page, int D, int Dv, int rep) { return kafka_hy_window_attn_mfma_ok(page, D, Dv, rep) != 0; });
   m.def("hy_window_attn_mfma", &window_attn_mfma, py::arg("q"), py::arg("kc"), py::arg("vt"), py::arg("bt"),
         py::arg("items"), py::arg("tile_tokens"), py::arg("positions"), py::arg("H"), py::arg("G"), py::arg("scale"),
         py::arg("window"), py::arg("sink"), py::arg("out"), py::arg("nsplit") = 1, py::arg("po") = py::none(),
-        py::arg("pml") = py::none(), py::arg("shared_keys") = false);
+        py::arg("pml") = py::none(), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0);
   m.def("hy_moe_topk_grouped", &moe_topk_grouped);
   m.def("hy_act_norm", &act_norm);
   m.def("hy_gate_mul", &gate_mul);
@@ -1120,6 +1236,10 @@ void kafka_bind_hybrid(pybind11::module_& m) {
   m.def("hy_hgrn2_chunk_decay", &hgrn2_chunk_decay);
   m.def("hy_hgrn2_chunk_combine", &hgrn2_chunk_combine);
   m.def("hy_rope_kv_store", &rope_kv_store);
+  m.def("hy_norm_add", &norm_add);
+  m.def("hy_ff_act", &ff_act);
+  m.def("hy_lin_scan", &lin_scan);
+  m.def("hy_lin_chunk", []() { return kafka_hy_lin_chunk(); });
   m.def("hy_sigmoid_attn_mfma_ok",
         [](int page, int D, int Dv, int rep) { return kafka_hy_sigmoid_attn_mfma_ok(page, D, Dv, rep) != 0; });
   m.def("hy_sigmoid_attn_mfma", &sigmoid_attn_mfma, py::arg("q"), py::arg("q_off"), py::arg("kc"), py::arg("vt"),

@@ -20,7 +20,7 @@
 //   mlstm_scan      one workgroup per (segment, head, 63 value columns + the normaliser as a 64th): thread (dg, v) keeps
 //                   a quarter of the rows of column v of the matrix memory in registers; q, k, v and gates of 8
 //                   tokens are staged in LDS (double buffered), the four partial read-outs per column summed through LDS
-//   head_norm_gate  unit RMS per head * weight * sigmoid(gate)
+//   head_norm_gate  unit RMS per head * weight * sigmoid(gate) or silu(gate)
 //   moe_topk        top-k of fp32 router logits by k wave-wide arg-max passes (ties: the lower index), softmax over
 //                   the chosen
 //   moe_gate_up / moe_down   experts evaluated per (row, chosen expert) pair: any sizes, both dtypes; the pairs of a
@@ -617,7 +617,7 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restr
                                                             const AT* __restrict__ w, const AT* __restrict__ g,
                                                             int64_t gs, int g_off, int H, int Dv, float eps,
                                                             AT* __restrict__ out, int64_t outs, int64_t pairs,
-                                                            float scale) {
+                                                            float scale, bool silu) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int64_t pair = (int64_t)blockIdx.x * (NT / 64) + wave;
   if (pair >= pairs) return;
@@ -630,7 +630,10 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restr
   for (int i = lane; i < Dv; i += 64) {
     const int c = h * Dv + i;
     float v = r[i] * rs * ldf(w + c) * scale;
-    if (g != nullptr) v *= sigmoidf(ldf(g + t * gs + g_off + c));
+    if (g != nullptr) {
+      const float z = ldf(g + t * gs + g_off + c);
+      v *= silu ? z * sigmoidf(z) : sigmoidf(z);
+    }
     stf(out + t * outs + c, v);
   }
 }
@@ -934,13 +937,13 @@ hipError_t kafka_hy_mlstm_scan(int f32, const void* qkv, int64_t qs, const float
 
 hipError_t kafka_hy_head_norm_gate(int f32, const float* o, int64_t os_, const void* w, const void* g, int64_t gs,
                                    int g_off, int H, int Dv, float eps, void* out, int64_t outs, int64_t T,
-                                   float scale, hipStream_t st) {
+                                   float scale, int silu, hipStream_t st) {
   if (T <= 0) return hipSuccess;
   const int64_t pairs = T * H;
   const int grid = (int)((pairs + NT / 64 - 1) / (NT / 64));
   DISPATCH_AT(f32, {
     head_norm_gate_kernel<AT><<<grid, NT, 0, st>>>(o, os_, (const AT*)w, (const AT*)g, gs, g_off, H, Dv, eps, (AT*)out,
-                                                   outs, pairs, scale);
+                                                   outs, pairs, scale, silu != 0);
   });
   return hipGetLastError();
 }

@@ -12,9 +12,9 @@
 //   hgrn2_scan      per head S <- diag(f) S + (1 - f) v^T, out = S^T silu(q), f = l + (1 - l) sigmoid(.): a workgroup per
 //                   (segment, head, 64 value columns), a thread keeps a quarter of the rows of one column in registers,
 //                   8 tokens' inputs staged in LDS (double buffered, the next block's loads in flight)
-//   rope_kv_store   rotation of q and k heads (halves or neighbour pairs), optional mix of the queries over the heads
-//                   (so that one product with the whole key row gives the head-mixed score), paged key / transposed
-//                   value store
+//   rope_kv_store   optional RMS norm of every q and k head, rotation of q and k heads (halves or neighbour pairs),
+//                   optional mix of the queries over the heads (so that one product with the whole key row gives the
+//                   head-mixed score), paged key / transposed value store; the values may be the raw key columns
 #include "common.h"
 
 namespace kafka {
@@ -369,7 +369,9 @@ __global__ void hgrn2_combine_kernel(const int* __restrict__ cs, const float* __
 // ---- attention inputs: rotation, head mix, paged store -------------------------------------------------------------------
 // One workgroup per row of the fused projection [q (H D) | k (G D) | v (G Dv) | ...]. The row's q and k parts, the
 // position's cos | sin row and the mix matrix are staged in LDS as fp32 in one batch of independent loads (a step of few
-// rows pays one memory latency per row); pairs are rotated in place (a thread owns both members); keys leave for
+// rows pays one memory latency per row); with qn / kn (one weight vector each for all q / all k heads) every head is
+// RMS-normed first; the values are the columns from v_off on (the key columns themselves when keys double as values:
+// they are read as projected); pairs are rotated in place (a thread owns both members); keys leave for
 // their page; the queries leave as they are, or with `talk` as q'[h][c D + i] = sum_r talk[h][c rep + r] q[c rep + r][i]
 // (rep = H / G).
 constexpr int MIX_REP = 32;   // query heads per key head whose values a lane keeps in registers for the head mix
@@ -377,7 +379,8 @@ constexpr int MIX_REP = 32;   // query heads per key head whose values a lane ke
 template <typename AT>
 __global__ __launch_bounds__(NT) void rope_kv_store_kernel(
     const AT* __restrict__ qkv, int64_t qs, int H, int G, int D, int Dv, const int64_t* __restrict__ positions,
-    const float* __restrict__ cos_sin, int dims, bool pairs, const float* __restrict__ talk, AT* __restrict__ kc,
+    const float* __restrict__ cos_sin, int dims, bool pairs, const float* __restrict__ talk,
+    const float* __restrict__ qn, const float* __restrict__ kn, float eps, int v_off, AT* __restrict__ kc,
     AT* __restrict__ vt, const int64_t* __restrict__ slots, AT* __restrict__ q_out, int64_t qos) {
   extern __shared__ float lds[];   // [H D + G D] q | k, [dims] cos | sin, [H H] mix weights
   const int64_t t = blockIdx.x;
@@ -411,9 +414,20 @@ __global__ __launch_bounds__(NT) void rope_kv_store_kernel(
   if (slot >= 0) {
     AT* vd = vt + (slot / PAGE) * (int64_t)Cv * PAGE + (slot % PAGE);
 #pragma unroll 4
-    for (int i = threadIdx.x; i < Cv; i += NT) vd[(int64_t)i * PAGE] = row[Cq + Ck + i];
+    for (int i = threadIdx.x; i < Cv; i += NT) vd[(int64_t)i * PAGE] = row[v_off + i];
   }
   __syncthreads();
+  if (qn != nullptr) {   // a wave per head: its mean square, then its elements scaled in place
+    for (int hd = wave; hd < H + G; hd += NT / 64) {
+      float* x = qk + hd * D;
+      const float* nw = hd < H ? qn : kn;
+      float s = 0.f;
+      for (int i = lane; i < D; i += 64) s += x[i] * x[i];
+      const float rs = 1.0f / sqrtf(wave_sum(s) / (float)D + eps);
+      for (int i = lane; i < D; i += 64) x[i] = x[i] * rs * nw[i];
+    }
+    __syncthreads();
+  }
   // a wave per head (query heads, then key heads), lanes over its frequencies
   for (int hd = wave; hd < H + G; hd += NT / 64) {
     float* x = qk + hd * D;
@@ -598,16 +612,19 @@ int kafka_hy_rope_store_max_q() { return 15360; }   // floats of LDS: H D + G D 
 
 hipError_t kafka_hy_rope_kv_store(int f32, const void* qkv, int64_t qs, int H, int G, int D, int Dv,
                                   const int64_t* positions, const float* cos_sin, int dims, int pairs,
-                                  const float* talk, void* kc, void* vt, const int64_t* slots, void* q_out, int64_t qos,
-                                  int64_t T, hipStream_t st) {
+                                  const float* talk, const float* qn, const float* kn, float eps, int v_off, void* kc,
+                                  void* vt, const int64_t* slots, void* q_out, int64_t qos, int64_t T, hipStream_t st) {
   if (T <= 0) return hipSuccess;
-  if (dims < 0 || dims % 2 || dims > D || (dims > 0 && cos_sin == nullptr) || G < 1 || H % G) return hipErrorInvalidValue;
+  if (dims < 0 || dims % 2 || dims > D || (dims > 0 && cos_sin == nullptr) || G < 1 || H % G ||
+      (qn != nullptr) != (kn != nullptr))
+    return hipErrorInvalidValue;
   const int64_t fl = (int64_t)(H + G) * D + dims + (talk != nullptr ? H * H : 0);
   if (fl > kafka_hy_rope_store_max_q()) return hipErrorInvalidValue;
   const size_t lds = (size_t)fl * sizeof(float);
   DISPATCH_AT(f32, {
     rope_kv_store_kernel<AT><<<(unsigned)T, NT, lds, st>>>((const AT*)qkv, qs, H, G, D, Dv, positions, cos_sin, dims,
-                                                           pairs != 0, talk, (AT*)kc, (AT*)vt, slots, (AT*)q_out, qos);
+                                                           pairs != 0, talk, qn, kn, eps, v_off, (AT*)kc, (AT*)vt, slots,
+                                                           (AT*)q_out, qos);
   });
   return hipGetLastError();
 }

@@ -19,7 +19,8 @@
 //                       row's keys are visited in order, whatever the batch
 //   window_attn_mfma    the same attention on the matrix cores (bf16): 32 (token, head) rows of one key/value head per
 //                       workgroup, 128-key blocks, online softmax, key-range splits with a merge pass
-//   moe_topk_grouped    softmax over all experts, choice among the best groups by corrected score, normalised weights
+//   moe_topk_grouped    softmax or sigmoid scores, choice among the best groups (by their largest score or the sum of
+//                       their two largest) by corrected score, weights normalised or as they are, times a scale
 #include "common.h"
 
 namespace kafka {
@@ -283,7 +284,7 @@ __global__ __launch_bounds__(NT) void window_attn_kernel(const AT* __restrict__ 
                                                          const int64_t* __restrict__ positions, int H, int G, int D,
                                                          int Dv, int Ck, int kstep, float scale_log2e, int window,
                                                          const float* __restrict__ sink, AT* __restrict__ out,
-                                                         int64_t os, int64_t pairs) {
+                                                         int64_t os, int64_t pairs, float out_scale) {
   // D: size of a query row and of the key it meets; key/value head g's key starts at column g * kstep of a key row of
   // Ck columns (kstep = D: one key head per key/value head; kstep = 0, D = Ck: every query row meets the whole key row)
   __shared__ float qsh[NT / 64][WA_MAXD];
@@ -348,7 +349,7 @@ __global__ __launch_bounds__(NT) void window_attn_kernel(const AT* __restrict__ 
       }
     }
   }
-  const float inv = 1.0f / l;
+  const float inv = out_scale / l;
 #pragma unroll
   for (int i = 0; i < WA_NV; ++i) {
     const int v = lane + 64 * i;
@@ -379,7 +380,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
     const bf16* __restrict__ q, int64_t qs, const bf16* __restrict__ kc, const bf16* __restrict__ vt,
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ items, const int64_t* __restrict__ positions,
     int H, int G, int D, int Dv, int Ck, int kstep, float scale_log2e, int window, const float* __restrict__ sink,
-    bf16* __restrict__ out, int64_t os, float* __restrict__ po, float* __restrict__ pml, int64_t T) {
+    bf16* __restrict__ out, int64_t os, float* __restrict__ po, float* __restrict__ pml, int64_t T, float out_scale) {
   // (D, Ck, kstep as in window_attn_kernel: kstep = 0 and D = Ck when every query row meets the whole key row)
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int nks = D >> 4, qstride = D + 8;
@@ -523,7 +524,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
     const int h = g * rep + r % rep;
     if (nsplit == 1) {
       if (sink != nullptr) l += fast_exp2(sink[h] * LOG2E - m[i]);
-      const float inv = 1.0f / l;
+      const float inv = out_scale / l;
 #pragma unroll
       for (int tw = 0; tw < TW; ++tw) {
         const int col = (w * TW + tw) * 32 + lr;
@@ -546,7 +547,8 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
 
 // out[t][h] = sum_z 2^(m_z - m) O_z / (sum_z 2^(m_z - m) l_z + 2^(sink_h - m)) over the key-range splits
 __global__ void window_merge_kernel(const float* __restrict__ po, const float* __restrict__ pml, int nsplit, int64_t T,
-                                    int H, int Dv, const float* __restrict__ sink, bf16* __restrict__ out, int64_t os) {
+                                    int H, int Dv, const float* __restrict__ sink, bf16* __restrict__ out, int64_t os,
+                                    float out_scale) {
   const int64_t th = blockIdx.x;  // t * H + h
   const int64_t t = th / H;
   const int h = (int)(th - t * H);
@@ -559,7 +561,7 @@ __global__ void window_merge_kernel(const float* __restrict__ po, const float* _
     if (mz != -INFINITY) den += fast_exp2(mz - mx) * pml[2 * (z * zs + th) + 1];
   }
   if (sink != nullptr) den += fast_exp2(sink[h] * LOG2E - mx);
-  const float inv = 1.0f / den;
+  const float inv = out_scale / den;
   for (int d = threadIdx.x; d < Dv; d += blockDim.x) {
     float a = 0.f;
     for (int z = 0; z < nsplit; ++z) {
@@ -575,15 +577,22 @@ constexpr int GR_MAXE = 512;  // experts (8 per lane)
 constexpr int GR_MAXK = 16;
 constexpr int GR_MAXG = 64;   // groups (one per lane)
 
-// one wave per row of fp32 logits [T, >= E]: s = softmax over the E experts; c = s + correction; the `keep` groups
-// (of `groups` equal runs of neighbouring experts) with the largest max c stay, the others' c count as -inf; the k
-// largest c are chosen (ties: the lower index); weights = s of the chosen / (their sum + eps). With `gate` the
-// logit in column E goes through a sigmoid.
+struct RouteForm {
+  bool sigmoid;   // scores: sigmoid of each logit, else softmax over all experts
+  bool top2;      // a group's score: the sum of its two largest c (groups of one: that one), else its largest c
+  bool norm;      // weights: divided by (their sum + eps), else as they are
+  float scale;    // factor on the weights
+};
+
+// one wave per row of fp32 logits [T, >= E]: s = softmax over the E experts or sigmoid; c = s + correction (when given);
+// the `keep` groups (of `groups` equal runs of neighbouring experts) with the largest group score stay, the others' c
+// count as -inf; the k largest c are chosen (ties: the lower index); weights from s of the chosen (RouteForm). With
+// `gate` the logit in column E goes through a sigmoid.
 __global__ __launch_bounds__(NT) void moe_topk_grouped_kernel(const float* __restrict__ logits, int64_t ls, int E,
                                                               int k, const float* __restrict__ corr, int groups,
                                                               int keep, float eps, float* __restrict__ tw,
                                                               int* __restrict__ te, float* __restrict__ gate,
-                                                              int64_t T) {
+                                                              int64_t T, RouteForm form) {
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int64_t t = (int64_t)blockIdx.x * (NT / 64) + wave;
   if (t >= T) return;
@@ -596,20 +605,26 @@ __global__ __launch_bounds__(NT) void moe_topk_grouped_kernel(const float* __res
     sc[i] = e < E ? logits[t * ls + e] : -INFINITY;
     mx = fmaxf(mx, sc[i]);
   }
-  mx = wave_max(mx);
-  float sum = 0.f;
+  if (form.sigmoid) {
 #pragma unroll
-  for (int i = 0; i < PL; ++i) {
-    sc[i] = lane + 64 * i < E ? expf(sc[i] - mx) : 0.f;
-    sum += sc[i];
+    for (int i = 0; i < PL; ++i) sc[i] = 1.0f / (1.0f + expf(-sc[i]));   // (0 past E)
+  } else {
+    mx = wave_max(mx);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PL; ++i) {
+      sc[i] = lane + 64 * i < E ? expf(sc[i] - mx) : 0.f;
+      sum += sc[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < PL; ++i) sc[i] = sc[i] / sum;
   }
-  sum = wave_sum(sum);
   const int gsz = E / groups;
 #pragma unroll
   for (int i = 0; i < PL; ++i) {
     const int e = lane + 64 * i;
-    sc[i] = sc[i] / sum;
-    c[i] = e < E ? sc[i] + corr[e] : -INFINITY;
+    c[i] = e < E ? (corr != nullptr ? sc[i] + corr[e] : sc[i]) : -INFINITY;
   }
   if (keep < groups) {
     // lane g holds group g's score
@@ -622,6 +637,23 @@ __global__ __launch_bounds__(NT) void moe_topk_grouped_kernel(const float* __res
         if (e < E && e / gsz == g) v = fmaxf(v, c[i]);
       }
       v = wave_max(v);
+      if (form.top2 && gsz > 1) {   // the second largest: one holder of the largest (the lowest index) left out
+        int hold = 0x7fffffff;
+#pragma unroll
+        for (int i = 0; i < PL; ++i) {
+          const int e = lane + 64 * i;
+          if (e < E && e / gsz == g && c[i] == v) hold = min(hold, e);
+        }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) hold = min(hold, __shfl_xor(hold, o, 64));
+        float v2 = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < PL; ++i) {
+          const int e = lane + 64 * i;
+          if (e < E && e / gsz == g && e != hold) v2 = fmaxf(v2, c[i]);
+        }
+        v += wave_max(v2);
+      }
       if (lane == g) gs = v;
     }
     unsigned long long kept = 0ull;
@@ -673,7 +705,7 @@ __global__ __launch_bounds__(NT) void moe_topk_grouped_kernel(const float* __res
     if (lane == 0) te[t * k + j] = bi;
   }
   if (lane == 0) {
-    const float inv = 1.0f / (wsum + eps);
+    const float inv = (form.norm ? 1.0f / (wsum + eps) : 1.0f) * form.scale;
     for (int j = 0; j < k; ++j) tw[t * k + j] = val[j] * inv;
     if (gate != nullptr) gate[t] = 1.0f / (1.0f + expf(-logits[t * ls + E]));
   }
@@ -767,7 +799,7 @@ int kafka_hy_window_attn_max_dv() { return 64 * WA_NV; }
 hipError_t kafka_hy_window_attn(int f32, const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                 int bt_stride, const int* tok_seg, const int64_t* positions, int H, int G, int D,
                                 int Dv, float scale, int window, const float* sink, void* out, int64_t os, int64_t T,
-                                int shared_keys, hipStream_t st) {
+                                int shared_keys, float out_scale, hipStream_t st) {
   // shared_keys: D is the whole key row's size and every query row meets all G key heads of a token at once
   if (T <= 0) return hipSuccess;
   if (D > WA_MAXD || Dv > 64 * WA_NV || G < 1 || H % G || window < 0) return hipErrorInvalidValue;
@@ -777,7 +809,7 @@ hipError_t kafka_hy_window_attn(int f32, const void* q, int64_t qs, const void* 
   DISPATCH_AT(f32, {
     window_attn_kernel<AT><<<grid, NT, 0, st>>>((const AT*)q, qs, (const AT*)kc, (const AT*)vt, bt, bt_stride, tok_seg,
                                                 positions, H, G, D, Dv, Ck, kstep, scale * LOG2E, window, sink,
-                                                (AT*)out, os, pairs);
+                                                (AT*)out, os, pairs, out_scale);
   });
   return hipGetLastError();
 }
@@ -791,7 +823,7 @@ hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, 
                                      int bt_stride, const int* items, int n_items, const int64_t* positions, int H,
                                      int G, int D, int Dv, float scale, int window, const float* sink, void* out,
                                      int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
-                                     hipStream_t st) {
+                                     float out_scale, hipStream_t st) {
   if (n_items <= 0) return hipSuccess;
   const int Ck = shared_keys ? D : G * D, kstep = shared_keys ? 0 : D;
   if (G < 1 || H % G || window < 0 || !kafka_hy_window_attn_mfma_ok(PAGE, D, Dv, H / G)) return hipErrorInvalidValue;
@@ -800,7 +832,8 @@ hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, 
   const dim3 grid((unsigned)n_items, (unsigned)G, (unsigned)nsplit);
   auto a = [&](auto k) {
     k<<<grid, 256, lds, st>>>((const bf16*)q, qs, (const bf16*)kc, (const bf16*)vt, bt, bt_stride, items, positions, H,
-                              G, D, Dv, Ck, kstep, scale * LOG2E, window, sink, (bf16*)out, os, po, pml, T);
+                              G, D, Dv, Ck, kstep, scale * LOG2E, window, sink, (bf16*)out, os, po, pml, T,
+                              out_scale);
   };
   const int nks = D / 16, tw = ((Dv + 31) / 32 + 3) / 4;
   if (tw == 1 && nks <= 4) a(window_attn_mfma_kernel<1, 4>);
@@ -809,7 +842,8 @@ hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, 
   else if (nks <= 8) a(window_attn_mfma_kernel<2, 8>);
   else a(window_attn_mfma_kernel<2, 16>);
   if (nsplit > 1)
-    window_merge_kernel<<<(unsigned)(T * H), 64, 0, st>>>(po, pml, nsplit, T, H, Dv, sink, (bf16*)out, os);
+    window_merge_kernel<<<(unsigned)(T * H), 64, 0, st>>>(po, pml, nsplit, T, H, Dv, sink, (bf16*)out, os,
+                                                             out_scale);
   return hipGetLastError();
 }
 
@@ -818,13 +852,15 @@ int kafka_hy_grouped_router_max_k() { return GR_MAXK; }
 int kafka_hy_grouped_router_max_g() { return GR_MAXG; }
 
 hipError_t kafka_hy_moe_topk_grouped(const float* logits, int64_t ls, int E, int k, const float* corr, int groups,
-                                     int keep, float eps, float* tw, int* te, float* gate, int64_t T, hipStream_t st) {
+                                     int keep, float eps, float* tw, int* te, float* gate, int64_t T, int sigmoid,
+                                     int top2, int norm, float scale, hipStream_t st) {
   if (T <= 0) return hipSuccess;
   if (E > GR_MAXE || k > GR_MAXK || k < 1 || groups < 1 || groups > GR_MAXG || E % groups || keep < 1 ||
       keep > groups || k > keep * (E / groups))
     return hipErrorInvalidValue;
   const int grid = (int)((T + NT / 64 - 1) / (NT / 64));
-  moe_topk_grouped_kernel<<<grid, NT, 0, st>>>(logits, ls, E, k, corr, groups, keep, eps, tw, te, gate, T);
+  moe_topk_grouped_kernel<<<grid, NT, 0, st>>>(logits, ls, E, k, corr, groups, keep, eps, tw, te, gate, T,
+                                              RouteForm{sigmoid != 0, top2 != 0, norm != 0, scale});
   return hipGetLastError();
 }
 

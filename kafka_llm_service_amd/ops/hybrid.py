@@ -1,7 +1,7 @@
 """Ops of the segment-planned decoder families (layer norm, token shift, latent attention, Mamba-2, depth average;
-gated mixers and routed experts; residual streams, windowed attention with sinks, group-limited routing): GPU tensors
-run the HIP kernels of ``csrc/hybrid.hip``, ``hybrid_gated.hip`` and ``hybrid_streams.hip``, CPU tensors the fp32
-references of ``hybrid_reference.py``.
+gated mixers and routed experts; residual streams, windowed attention with sinks, group-limited routing; post-normed
+residual, linear attention with per-channel decays and the gated delta rule): GPU tensors run the HIP kernels of
+``csrc/hybrid.hip`` and ``csrc/hybrid_*.hip``, CPU tensors the fp32 references of ``hybrid_reference.py``.
 
 Activations are bf16 or fp32 (the model's dtype, the kernels are built for both); the residual stream, recurrent
 state, norms, softmax and every gate of a recurrence are fp32 in both. A step's rows are described by ``seg`` int32
@@ -342,13 +342,15 @@ def mlstm_scan(qkv, gates, H: int, D: int, Dv: int, cap: float, tok_seg, seg, S,
         ref.mlstm_scan(qkv, gates, H, D, Dv, cap, tok_seg, seg, S, nrm, mx, out)
 
 
-def head_norm_gate(o, w, g, g_off: int, H: int, eps, out, scale: float = 1.0) -> None:
-    """out = o / rms_per_head(o) * w * sigmoid(g[:, g_off : g_off + H Dv]) * scale for o fp32 [T, H Dv]; ``g`` None:
-    no gate. ``out`` may be a column slice of a wider buffer."""
+def head_norm_gate(o, w, g, g_off: int, H: int, eps, out, scale: float = 1.0, act: str = "sigmoid") -> None:
+    """out = o / rms_per_head(o) * w * act(g[:, g_off : g_off + H Dv]) * scale for o fp32 [T, H Dv]; ``act`` is
+    "sigmoid" or "silu", ``g`` None: no gate. ``out`` may be a column slice of a wider buffer."""
+    if act not in ("sigmoid", "silu"):
+        raise ValueError(f"head_norm_gate: unknown gate {act!r}")
     if _gpu(o):
-        ext().hy_head_norm_gate(o, w, g, int(g_off), int(H), float(eps), out, float(scale))
+        ext().hy_head_norm_gate(o, w, g, int(g_off), int(H), float(eps), out, float(scale), act == "silu")
     else:
-        ref.head_norm_gate(o, w, g, g_off, H, eps, out, scale)
+        ref.head_norm_gate(o, w, g, g_off, H, eps, out, scale, act)
 
 
 def moe_router(h, w, b, k: int):
@@ -524,7 +526,7 @@ def window_attn_mfma_ok(q, k_cache, v_cache_t, H: int, G: int, shared_keys: bool
 
 
 def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int, G: int, scale: float, window: int,
-                sink, out, tiles=None, max_keys: int = 0, shared_keys: bool = False) -> None:
+                sink, out, tiles=None, max_keys: int = 0, shared_keys: bool = False, out_scale: float = 1.0) -> None:
     """Causal softmax attention over paged keys [pages, page, G D] and page-wise transposed values [pages, G Dv, page]:
     row t at position p, head h (key/value head h // (H / G)) sees the keys p - window < j <= p (window 0: all j <= p);
         out = sum_j e^(s_j) v_j / (sum_j e^(s_j) + e^(sink[h])),  s_j = (q . k_j) scale
@@ -535,7 +537,7 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
     over more workgroups (``sig_splits``); a merge pass combines them.
     ``shared_keys``: q is [T, H G D] - every query head is a row of the whole key row's size and its score is the
     product with ALL G key heads of a token (queries that hold a mix over the heads, see ``rope_kv_store``); values
-    stay per key/value head."""
+    stay per key/value head. The result is multiplied by ``out_scale``; ``out`` may be a column slice."""
     if window < 0:
         raise ValueError("window_attn: window must be positive (0 = every earlier position)")
     if _gpu(q):
@@ -551,28 +553,33 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
                 po = torch.empty(ns, q.shape[0], out.shape[1], dtype=torch.float32, device=q.device)
                 pml = torch.empty(ns, q.shape[0], H, 2, dtype=torch.float32, device=q.device)
             ext().hy_window_attn_mfma(q, k_cache, v_cache_t, block_tables, tiles, tt, positions, int(H), int(G),
-                                      float(scale), int(window), sink, out, ns, po, pml, bool(shared_keys))
+                                      float(scale), int(window), sink, out, ns, po, pml, bool(shared_keys),
+                                      float(out_scale))
         else:
             ext().hy_window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, int(H), int(G), float(scale),
-                                 int(window), sink, out, bool(shared_keys))
+                                 int(window), sink, out, bool(shared_keys), float(out_scale))
     else:
         ref.window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H, G, scale, window, sink, out,
-                        shared_keys)
+                        shared_keys, out_scale)
 
 
-def moe_router_grouped(h, w, correction, k: int, groups: int, keep: int, eps: float = 0.0, extra_gate: bool = False):
+def moe_router_grouped(h, w, correction, k: int, groups: int, keep: int, eps: float = 0.0, extra_gate: bool = False,
+                       score: str = "softmax", group_score: str = "max", norm: bool = True, scale: float = 1.0):
     """Group-limited router: fp32 logits h W^T over the first E rows of ``w`` (fp32 [E (+ 1), d]); s = softmax over
-    all E; the choice looks at s + correction, only within the ``keep`` groups (of ``groups`` equal groups of
-    neighbouring experts) whose largest corrected score is largest, and takes the k largest there (ties: the lower
-    index); the weights are s of the chosen divided by (their sum + eps). With ``extra_gate`` the last row of ``w`` is
-    a gate vector and sigmoid of its product is returned per row. Returns (weights fp32 [T, k], experts int32
-    [T, k], gate fp32 [T] or None)."""
+    all E or (``score`` "sigmoid") sigmoid of each; the choice looks at s + correction (None: at s), only within the
+    ``keep`` groups (of ``groups`` equal groups of neighbouring experts) with the largest group score - the largest
+    value of a group, or (``group_score`` "top2") the sum of its two largest - and takes the k largest there (ties:
+    the lower index); the weights are s of the chosen, divided by (their sum + eps) unless ``norm`` is off, times
+    ``scale``. With ``extra_gate`` the last row of ``w`` is a gate vector and sigmoid of its product is returned per
+    row. Returns (weights fp32 [T, k], experts int32 [T, k], gate fp32 [T] or None)."""
     T = h.shape[0]
     E = w.shape[0] - (1 if extra_gate else 0)
     if E < 1 or groups < 1 or E % groups or not 1 <= keep <= groups or not 1 <= k <= keep * (E // groups):
         raise ValueError("router: experts, groups and choices do not fit")
-    if correction.shape[0] != E:
+    if correction is not None and correction.shape[0] != E:
         raise ValueError("router: one correction per expert")
+    if score not in ("softmax", "sigmoid") or group_score not in ("max", "top2"):
+        raise ValueError("router: unknown score")
     tw = torch.empty(T, k, dtype=torch.float32, device=h.device)
     te = torch.empty(T, k, dtype=torch.int32, device=h.device)
     gate = torch.empty(T, dtype=torch.float32, device=h.device) if extra_gate else None
@@ -580,9 +587,9 @@ def moe_router_grouped(h, w, correction, k: int, groups: int, keep: int, eps: fl
         # logits as one full-precision fp32 matrix product (the engine switches reduced-precision matrix modes off),
         # then the choice kernel
         ext().hy_moe_topk_grouped(torch.mm(h.float(), w.t()), int(E), correction, int(groups), int(keep), float(eps),
-                                  tw, te, gate)
+                                  tw, te, gate, score == "sigmoid", group_score == "top2", bool(norm), float(scale))
     else:
-        ref.moe_router_grouped(h, w, E, correction, k, groups, keep, eps, tw, te, gate)
+        ref.moe_router_grouped(h, w, E, correction, k, groups, keep, eps, tw, te, gate, score, group_score, norm, scale)
     return tw, te, gate
 
 
@@ -653,24 +660,103 @@ def hgrn2_scan_chunked(proj, q_off: int, f_off: int, v_off: int, f_bias, lower, 
     e.hy_hgrn2_scan(proj, int(q_off), int(f_off), int(v_off), f_bias, lower, int(H), int(D), int(Dv), cont, tmp, out)
 
 
-def rope_kv_store(qkv, H: int, G: int, D: int, Dv: int, positions, cos_sin, rot_dims: int, pairs: bool, talk,
-                  k_cache, v_cache_t, slot_mapping, q_out) -> None:
+def rope_kv_store(qkv, H: int, G: int, D: int, Dv: int, positions, cos_sin, rot_dims, pairs: bool, talk,
+                  k_cache, v_cache_t, slot_mapping, q_out, q_norm=None, k_norm=None, eps: float = 0.0,
+                  v_off: int | None = None) -> None:
     """Attention inputs from the fused projection row [q (H D) | k (G D) | v (G Dv)] (further columns are ignored):
+      * with ``q_norm`` / ``k_norm`` (fp32 [D], shared by all heads) an RMS norm of every q and k head;
       * rotation of the first ``rot_dims`` dimensions of every q and k head by the row's position (``cos_sin`` fp32
         [positions, rot_dims] = cos | sin per frequency): dimension i with i + rot_dims / 2, or with ``pairs``
         dimension 2i with 2i + 1; rot_dims = 0 and no table: no rotation;
-      * k -> k_cache [pages, page, G D] at the row's slot; v -> v_cache_t [pages, G Dv, page];
+      * k -> k_cache [pages, page, G D] at the row's slot; v -> v_cache_t [pages, G Dv, page]; the values are the
+        columns from ``v_off`` on (default: after the keys; H D: the keys as projected double as values);
       * q -> q_out [T, H D]; or with ``talk`` fp32 [H, H] (scores mixed over the heads before the softmax,
         s'_h = sum_g talk[h, g] s_g) -> q_out [T, H G D]: q'[h] = for every key head c the sum over its query heads g
         of talk[h, g] q[g], so that q'[h] . (the whole key row) = s'_h (``window_attn`` with ``shared_keys``).
-    Rotation and the mix are fp32."""
+    Norm, rotation and the mix are fp32."""
     if rot_dims % 2 or rot_dims > D or (rot_dims > 0) != (cos_sin is not None):
         raise ValueError("rope_kv_store: rot_dims even, at most the head size, with its table")
     if G < 1 or H % G:
         raise ValueError("rope_kv_store: query heads must split evenly over the key heads")
+    if (q_norm is None) != (k_norm is None):
+        raise ValueError("rope_kv_store: q_norm and k_norm come together")
+    v_off = H * D + G * D if v_off is None else int(v_off)
     if _gpu(qkv):
         ext().hy_rope_kv_store(qkv, int(H), int(G), int(D), int(Dv), positions, cos_sin, int(rot_dims), bool(pairs),
-                               talk, k_cache, v_cache_t, slot_mapping, q_out)
+                               talk, k_cache, v_cache_t, slot_mapping, q_out, q_norm, k_norm, float(eps), v_off)
     else:
         ref.rope_kv_store(qkv, H, G, D, Dv, positions, cos_sin, rot_dims, pairs, talk, k_cache, v_cache_t,
-                          slot_mapping, q_out)
+                          slot_mapping, q_out, q_norm, k_norm, eps, v_off)
+
+
+# ---- post-normed residual, linear attention with per-channel decays, gated delta rule -------------------------------
+def norm_add(x, y1, y2, w, eps, out=None) -> None:
+    """x += rms_norm(y1 + y2) * w on the fp32 stream (y2 may be None); with ``out`` the new x also in out's dtype.
+    y1 [T, d] in the activation dtype or fp32, or the fp32 split-K slabs [S, T, d] of a projection (summed here)."""
+    if _gpu(x):
+        ext().hy_norm_add(x, y1, y2, w, float(eps), out)
+    else:
+        ref.norm_add(x, y1, y2, w, eps, out)
+
+
+def relu2(u, out) -> None:
+    """out = relu(u)^2."""
+    if _gpu(u):
+        ext().hy_ff_act(u, out, False)
+    else:
+        ref.relu2(u, out)
+
+
+def silu_mul(gu, out) -> None:
+    """out = silu(gu[:, :F]) * gu[:, F:]."""
+    if _gpu(gu):
+        ext().hy_ff_act(gu, out, True)
+    else:
+        ref.silu_mul(gu, out)
+
+
+LIN_CHUNK = 32        # tokens of a chunk (the kernels' constant)
+LIN_CHUNK_MIN = 64    # segments of at least this many rows are scanned in chunks
+
+
+def lin_chunk_tables(seg_host):
+    """Chunk tables of a step for ``lin_scan``: (vseg, cs) as numpy int32, or None when no segment is long enough -
+    every segment of at least LIN_CHUNK_MIN rows cut into chunks of LIN_CHUNK: vseg[c] = (first row, rows, 0, 0),
+    cs[r] = (first chunk, chunks, first position, state slot). Shorter segments stay with the token-by-token kernel."""
+    import numpy as np
+
+    if seg_host is None:
+        return None
+    vs, cs = [], []
+    for q0, n, p0, slot in seg_host.tolist():
+        if n >= LIN_CHUNK_MIN:
+            cs.append((len(vs), -(-n // LIN_CHUNK), p0, slot))
+            vs += [(q0 + a, min(LIN_CHUNK, n - a), 0, 0) for a in range(0, n, LIN_CHUNK)]
+    if not cs:
+        return None
+    return np.asarray(vs, dtype=np.int32), np.asarray(cs, dtype=np.int32)
+
+
+def lin_scan(qk, q_off: int, k_off: int, v, z, z_bias, H: int, G: int, D: int, Dv: int, tok_seg, seg, S, out,
+             tau: float = 1.0, rate=None, beta=None, chunks=None, any_short: bool = True) -> None:
+    """Linear attention with a decay per head and key channel over a step's segments. q / k: G heads of D columns of
+    ``qk`` at q_off / k_off, head h uses q/k head h // (H / G); v [T, H Dv]; z [T, H D] raw decays, z_bias fp32 [H D].
+    Per head, with q' = q D^(-1/2):
+      rate None    gated linear attention:  a = sigmoid(z + z_bias)^(1 / tau),  S <- diag(a) S + k v^T,  out = S^T q'
+      rate fp32 [H], beta [T, H] raw    gated delta rule: q and k are made unit vectors first (x / sqrt(sum(x^2) +
+                   1e-6)), a = exp(rate softplus(z + z_bias)), S <- diag(a) S;  u = sigmoid(beta) (v - S^T k);
+                   S <- S + k u^T;  out = S^T q'
+    S fp32 [slots, H, D, Dv], zero before a sequence's first token; out fp32 [T, H Dv]. ``chunks``: device tensors of
+    ``lin_chunk_tables`` - their segments run in chunks of LIN_CHUNK tokens (the same recurrence as matrix products,
+    re-associated: fp32 rounding only), the others token by token; ``any_short`` False: there are no others."""
+    if D > 256:
+        raise ValueError("lin_scan: head sizes up to 256")
+    if _gpu(qk):
+        args = (qk, int(q_off), int(k_off), v, z, z_bias, rate, beta, int(H), int(G), int(D), int(Dv), D ** -0.5,
+                1.0 / float(tau))
+        if chunks is not None:
+            ext().hy_lin_scan(*args, chunks[0], 0, chunks[1], S, out)
+        if chunks is None or any_short:
+            ext().hy_lin_scan(*args, seg, LIN_CHUNK_MIN - 1 if chunks is not None else 1 << 30, None, S, out)
+    else:
+        ref.lin_scan(qk, q_off, k_off, v, z, z_bias, H, G, D, Dv, tok_seg, seg, S, out, tau, rate, beta)

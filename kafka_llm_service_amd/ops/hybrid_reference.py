@@ -266,15 +266,16 @@ def mlstm_scan(qkv, gates, H, D, Dv, cap, tok_seg, seg, S, nrm, mx, out):
         S[slot], nrm[slot], mx[slot] = Ss, ns, ms
 
 
-def head_norm_gate(o, w, g, g_off, H, eps, out, scale=1.0):
-    """out = unit_rms_per_head(o) * w * sigmoid(g[:, g_off : g_off + H Dv]) * scale (o fp32 [T, H Dv]; no gate
+def head_norm_gate(o, w, g, g_off, H, eps, out, scale=1.0, act="sigmoid"):
+    """out = unit_rms_per_head(o) * w * act(g[:, g_off : g_off + H Dv]) * scale (o fp32 [T, H Dv]; no gate
     when ``g`` is None)."""
     T, n = o.shape
     v = o.float().view(T, H, n // H)
     v = v * torch.rsqrt((v * v).mean(-1, keepdim=True) + eps)
     v = v.reshape(T, n) * w.float()
     if g is not None:
-        v = v * torch.sigmoid(g[:, g_off:g_off + n].float())
+        z = g[:, g_off:g_off + n].float()
+        v = v * (F.silu(z) if act == "silu" else torch.sigmoid(z))
     out.copy_((v * scale).to(out.dtype))
 
 
@@ -360,7 +361,7 @@ def qk_norm_rope_store(qkv, H, G, D, Dv, q_w, k_w, eps, positions, cos_sin, rot_
 
 
 def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H, G, scale, window, sink, out,
-                shared_keys=False):
+                shared_keys=False, out_scale=1.0):
     """``shared_keys``: every query head is a row of the whole key row's size and meets all G key heads at once
     (queries that already hold a mix over the heads); values stay per key/value head."""
     T = q.shape[0]
@@ -380,16 +381,19 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H, G, s
         if sink is not None:
             s = torch.cat([s, sink.float()[:, None]], 1)
         pw = torch.softmax(s, -1)[:, :n - lo]
-        out[t] = torch.einsum("hj,jhv->hv", pw, v.repeat_interleave(rep, 1)).reshape(H * Dv).to(out.dtype)
+        o = torch.einsum("hj,jhv->hv", pw, v.repeat_interleave(rep, 1)) * out_scale
+        out[t] = o.reshape(H * Dv).to(out.dtype)
 
 
-def moe_router_grouped(h, w, E, correction, k, groups, keep, eps, topk_w, topk_e, gate):
+def moe_router_grouped(h, w, E, correction, k, groups, keep, eps, topk_w, topk_e, gate, score="softmax",
+                       group_score="max", norm=True, scale=1.0):
     z = h.float() @ w.float().T
-    s = torch.softmax(z[:, :E], -1)
-    choice = s + correction.float()
+    s = torch.sigmoid(z[:, :E]) if score == "sigmoid" else torch.softmax(z[:, :E], -1)
+    choice = s if correction is None else s + correction.float()
     T = h.shape[0]
     gsz = E // groups
-    gs = choice.view(T, groups, gsz).max(-1).values
+    gs = choice.view(T, groups, gsz)
+    gs = gs.topk(min(2, gsz), -1).values.sum(-1) if group_score == "top2" else gs.max(-1).values
     gi = torch.sort(gs, dim=-1, descending=True, stable=True).indices[:, :keep]
     ok = torch.zeros(T, groups, dtype=torch.bool)
     ok.scatter_(1, gi, True)
@@ -397,7 +401,7 @@ def moe_router_grouped(h, w, E, correction, k, groups, keep, eps, topk_w, topk_e
     idx = torch.sort(choice, dim=-1, descending=True, stable=True).indices[:, :k]
     wv = s.gather(1, idx)
     topk_e.copy_(idx)
-    topk_w.copy_(wv / (wv.sum(-1, keepdim=True) + eps))
+    topk_w.copy_((wv / (wv.sum(-1, keepdim=True) + eps) if norm else wv) * scale)
     if gate is not None:
         gate.copy_(torch.sigmoid(z[:, E]))
 
@@ -453,15 +457,20 @@ def hgrn2_scan(proj, q_off, f_off, v_off, f_bias, lower, H, D, Dv, tok_seg, seg,
 
 
 def rope_kv_store(qkv, H, G, D, Dv, positions, cos_sin, rot_dims, pairs, talk, k_cache, v_cache_t, slot_mapping,
-                  q_out):
-    """Fused projection row [q (H D) | k (G D) | v (G Dv)]: rotation of the first rot_dims dimensions of every q and
+                  q_out, q_norm=None, k_norm=None, eps=0.0, v_off=None):
+    """Fused projection row [q (H D) | k (G D) | v (G Dv)] (values from column v_off on): optional RMS norm of every q
+    and k head (weights [D]), rotation of the first rot_dims dimensions of every q and
     k head (partners i, i + rot_dims / 2, or with ``pairs`` 2i, 2i + 1), keys and values into their pages. With
     ``talk`` fp32 [H, H] the queries leave as q'[h] = [sum over the heads g of key head c of talk[h, g] q[g]] for
     c = 0 .. G - 1 (row size G D): q'[h] . (whole key row) is the head-mixed score."""
     T = qkv.shape[0]
     Cq, Ck, Cv = H * D, G * D, G * Dv
-    q, k, v = (t.float() for t in qkv[:, :Cq + Ck + Cv].split([Cq, Ck, Cv], 1))
-    q, k = q.view(T, H, D).clone(), k.view(T, G, D).clone()
+    v_off = Cq + Ck if v_off is None else v_off
+    q, k, v = qkv[:, :Cq].float(), qkv[:, Cq:Cq + Ck].float(), qkv[:, v_off:v_off + Cv].float()
+    q, k = q.reshape(T, H, D).clone(), k.reshape(T, G, D).clone()
+    if q_norm is not None:
+        q = q * torch.rsqrt((q * q).mean(-1, keepdim=True) + eps) * q_norm.float()
+        k = k * torch.rsqrt((k * k).mean(-1, keepdim=True) + eps) * k_norm.float()
     if rot_dims:
         half = rot_dims // 2
         cs = cos_sin[positions.long()]
@@ -480,3 +489,49 @@ def rope_kv_store(qkv, H, G, D, Dv, positions, cos_sin, rot_dims, pairs, talk, k
         q = torch.einsum("hcr,tcrd->thcd", talk.float().view(H, G, rep), q.view(T, G, rep, D)).reshape(T, H * Ck)
     q_out.copy_(q.reshape(T, -1).to(q_out.dtype))
     kv_store(torch.cat([k.reshape(T, Ck), v], 1).to(k_cache.dtype), 0, Ck, k_cache, v_cache_t, slot_mapping)
+
+
+# ---- post-normed residual, linear attention with per-channel decays, gated delta rule -------------------------------
+def norm_add(x, y1, y2, w, eps, out=None):
+    """x += rms_norm(y1 + y2) * w (y1 may be split-K slabs [S, T, d]); ``out`` the new x in its dtype."""
+    y = y1.float().sum(0) if y1.dim() == 3 else y1.float()
+    if y2 is not None:
+        y = y + y2.float()
+    x += y * torch.rsqrt((y * y).mean(-1, keepdim=True) + eps) * w.float()
+    if out is not None:
+        out.copy_(x)
+
+
+def relu2(u, out):
+    out.copy_(torch.relu(u.float()).square())
+
+
+def silu_mul(gu, out):
+    n = out.shape[1]
+    out.copy_(F.silu(gu[:, :n].float()) * gu[:, n:].float())
+
+
+def lin_scan(qk, q_off, k_off, v, z, z_bias, H, G, D, Dv, tok_seg, seg, S, out, tau=1.0, rate=None, beta=None):
+    """Per head: S <- diag(a) S + k u^T, out = S^T q D^(-1/2) with a = sigmoid(z)^(1 / tau) and u = v, or (``rate``)
+    unit q and k, a = exp(rate softplus(z)) and u = sigmoid(beta) (v - (diag(a) S)^T k)."""
+    T, rep = qk.shape[0], H // G
+    q = qk[:, q_off:q_off + G * D].float().reshape(T, G, D)
+    k = qk[:, k_off:k_off + G * D].float().reshape(T, G, D)
+    zz = (z.float() + z_bias.float()).view(T, H, D)
+    if rate is None:
+        a = torch.exp(F.logsigmoid(zz) / tau)
+    else:
+        q = q * torch.rsqrt((q * q).sum(-1, keepdim=True) + 1e-6)
+        k = k * torch.rsqrt((k * k).sum(-1, keepdim=True) + 1e-6)
+        a = torch.exp(rate.float()[:, None] * F.softplus(zz))
+        bt = torch.sigmoid(beta.float())
+    q, k = (q * D ** -0.5).repeat_interleave(rep, 1), k.repeat_interleave(rep, 1)
+    vv = v.float().reshape(T, H, Dv)
+    for q0, n, p0, slot in seg.tolist():
+        St = S[slot].clone() if p0 > 0 else torch.zeros(H, D, Dv)
+        for t in range(q0, q0 + n):
+            St = a[t][:, :, None] * St
+            u = vv[t] if rate is None else bt[t][:, None] * (vv[t] - torch.einsum("hdv,hd->hv", St, k[t]))
+            St = St + k[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", St, q[t]).reshape(-1)
+        S[slot] = St
