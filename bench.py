@@ -109,7 +109,8 @@ def parse(argv=None):
                          "(windowed latent and grouped-query attention over 4 residual streams; 8 group-routed "
                          "experts, 2 per token, and a shared one, of a third of the dense feed-forward each), magedra "
                          "(latent attention, minGRU and parallel head-mixed attention + HGRN2 layers over 4 residual "
-                         "streams, the dense clamped feed-forward)")
+                         "streams, the dense clamped feed-forward), rogosun (gated linear attention and parallel "
+                         "attention + gated delta rule layers; dense squared-relu and routed feed-forwards in turn)")
     return ap.parse_args(argv)
 
 
@@ -120,11 +121,12 @@ def arch_compare(args) -> int:
     import torch
 
     from kafka_llm_service_amd.engine.engine import EngineConfig, LLMEngine
-    from kafka_llm_service_amd.models.config import ModelConfig, _budurax, _lisorax, _magedra, _mozidra
+    from kafka_llm_service_amd.models.config import ModelConfig, _budurax, _lisorax, _magedra, _mozidra, _rogosun
     from kafka_llm_service_amd.models.magedra import MagedraConfig
     from kafka_llm_service_amd.models.budurax import BuduraxConfig
     from kafka_llm_service_amd.models.lisorax import LisoraxConfig
     from kafka_llm_service_amd.models.mozidra import MozidraConfig
+    from kafka_llm_service_amd.models.rogosun import RogosunConfig
 
     dev = "cuda:0" if torch.cuda.is_available() else "cpu"
     w, L = args.arch_width, args.arch_layers
@@ -139,6 +141,8 @@ def arch_compare(args) -> int:
                                                name=f"mozidra-w{w}-l{L}"),
             # (two key heads of 128: the head-mixed queries meet a 256-wide key row, the matrix-core kernel's limit)
             "magedra": MagedraConfig.from_dict(_magedra(w, heads, 2, L, vocab, ff), name=f"magedra-w{w}-l{L}"),
+            "rogosun": RogosunConfig.from_dict(_rogosun(w, heads, 2, L, vocab, ff, expert_ff=ff // 3 // 256 * 256),
+                                               name=f"rogosun-w{w}-l{L}"),
             "llama": ModelConfig(name=f"llama-w{w}-l{L}", hidden_size=w, intermediate_size=ff, num_layers=L,
                                  num_heads=heads, num_kv_heads=max(1, heads // 4), vocab_size=vocab,
                                  max_position_embeddings=131072, bos_token_id=1, eos_token_ids=[2])}
