@@ -496,13 +496,17 @@ class RogosunLM:
         return self._lin(hf, self.head, getattr(self, "head_t", None)).float()[:, :cfg.vocab_size]
 
     def _chunks(self, m: SegMeta):
-        """(chunk tables on the device or None, whether any segment is scanned token by token), built once per step."""
+        """(chunk tables on the device or None, fewest and most rows of the segments that are scanned token by token or
+        None), built once per step."""
         if "lin" not in m.cache:
-            tabs, short = None, True
-            if self.device.type == "cuda" and m.seg_host is not None:
+            tabs, short = None, (1, 1 << 30)
+            if self.device.type == "cuda" and m.seg_host is not None and len(m.seg_host):
                 tabs = hops.lin_chunk_tables(m.seg_host)
+                rows = m.seg_host[:, 1]
                 if tabs is not None:
-                    short = bool((m.seg_host[:, 1] < hops.LIN_CHUNK_MIN).any())
+                    rows = rows[rows < hops.LIN_CHUNK_MIN]
+                short = (int(rows.min()), int(rows.max())) if len(rows) else None
+                if tabs is not None:
                     nv = tabs[0].size
                     up = torch.from_numpy(tabs[0]).view(-1)
                     up = torch.cat([up, torch.from_numpy(tabs[1]).view(-1)]).to(self.device)
@@ -518,7 +522,7 @@ class RogosunLM:
         o = torch.empty(T, H * Dv, dtype=torch.float32, device=dev)
         chunks, short = self._chunks(m)
         hops.lin_scan(proj, off["q"], off["k"], proj[:, off["v"]:off["v"] + H * Dv], z, lw.z_bias, H, H, D, Dv,
-                      m.tok_seg, m.seg, st["S"], o, tau=lw.tau, chunks=chunks, any_short=short)
+                      m.tok_seg, m.seg, st["S"], o, tau=lw.tau, chunks=chunks, rows=short)
         on = torch.empty(T, H * Dv, dtype=dt, device=dev)
         hops.head_norm_gate(o, lw.hnorm, proj, off["g"], H, self.cfg.norm_eps, on, act="silu")
         return self._lin(on, lw.o, getattr(lw, "o_t", None), slabs=True)
@@ -545,7 +549,7 @@ class RogosunLM:
         chunks, short = self._chunks(m)
         hops.lin_scan(qkv, 0, Gr * Dr, qkv[:, 2 * Gr * Dr:], low[:, :Hr * Dr], lw.z_bias, Hr, Gr, Dr, Dvr, m.tok_seg,
                       m.seg, st["S"], o, rate=lw.rate, beta=proj[:, off["b"]:off["b"] + Hr], chunks=chunks,
-                      any_short=short)
+                      rows=short)
         hops.head_norm_gate(o, lw.hnorm, low, Hr * Dr, Hr, eps, both[:, H * D:], lw.right_scale)
         return self._lin(both, lw.o, getattr(lw, "o_t", None), slabs=True)
 

@@ -777,6 +777,65 @@ __global__ void short_conv_kernel(const AT* __restrict__ proj, int64_t ps, int c
   }
 }
 
+// The same on bf16 rows whose sizes, offsets, strides and bases are multiples of 8 elements: a thread takes 8 channels of
+// TB consecutive rows and slides the window over them (a row is loaded once per thread; a row that starts a segment
+// takes its window from the slot's tail, or zeros).
+template <int TAPS, int TB>
+__global__ void short_conv_vec8_kernel(const bf16* __restrict__ proj, int64_t ps, int c0, const bf16* __restrict__ w,
+                                       const bf16* __restrict__ b, int C, const int* __restrict__ tok_seg,
+                                       const int* __restrict__ seg, const bf16* __restrict__ state,
+                                       bf16* __restrict__ out, int64_t T, int silu, int residual) {
+  const int C8 = C >> 3;
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  const int64_t blk = i / C8;
+  const int c = (int)(i - blk * C8) << 3;
+  const int64_t ta = blk * TB;
+  if (ta >= T) return;
+  float wt[TAPS][8], bias[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    bias[e] = b ? (float)b[c + e] : 0.f;
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) wt[k][e] = (float)w[(int64_t)(c + e) * TAPS + k];
+  }
+  bf16x8 win[TAPS];   // inputs of rows t - TAPS + 1 .. t
+  const bf16x8 zero = {0, 0, 0, 0, 0, 0, 0, 0};
+  for (int j = 0; j < TB; ++j) {
+    const int64_t t = ta + j;
+    if (t >= T) return;
+    const int sg = tok_seg[t];
+    const int q0 = seg[4 * sg];
+    if (j == 0 || t == q0) {
+      const int p0 = seg[4 * sg + 2], slot = seg[4 * sg + 3];
+#pragma unroll
+      for (int k = 0; k < TAPS - 1; ++k) {
+        const int64_t src = t - (TAPS - 1) + k;
+        if (src >= q0) {
+          win[k] = load_bf16x8(proj + src * ps + c0 + c);
+        } else {
+          const int si = TAPS - 1 + (int)(src - q0);
+          win[k] = (p0 > 0 && si >= 0) ? load_bf16x8(state + ((int64_t)slot * (TAPS - 1) + si) * C + c) : zero;
+        }
+      }
+    } else {
+#pragma unroll
+      for (int k = 0; k < TAPS - 1; ++k) win[k] = win[k + 1];
+    }
+    win[TAPS - 1] = load_bf16x8(proj + t * ps + c0 + c);
+    bf16x8 o;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float a = bias[e];
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) a += (float)win[k][e] * wt[k][e];
+      if (silu) a = a / (1.0f + expf(-a));
+      if (residual) a += (float)win[TAPS - 1][e];
+      o[e] = (bf16)a;
+    }
+    store_bf16x8(out + t * C + c, o);
+  }
+}
+
 // the slot's tail <- the last taps - 1 entries of (old tail ++ the segment's raw inputs); one thread per (segment,
 // channel) reads all it needs before it writes
 template <typename AT>
@@ -1265,6 +1324,21 @@ hipError_t kafka_hy_short_conv(int f32, const void* proj, int64_t ps, int c0, co
                                int taps, const int* tok_seg, const int* seg, int R, void* state, void* out, int64_t T,
                                int silu, int residual, hipStream_t st) {
   if (T <= 0 || C <= 0 || taps > 16 || taps < 1) return (taps > 16 || taps < 1) ? hipErrorInvalidValue : hipSuccess;
+  auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (!f32 && taps >= 2 && taps <= 4 && C % 8 == 0 && c0 % 8 == 0 && ps % 8 == 0 && al(proj) && al(state) && al(out)) {
+    const bool runs = T >= 2048;   // few rows: a thread per row, many: a thread per eight
+    const int64_t n = (runs ? (T + 7) / 8 : T) * (C / 8);
+    auto a = [&](auto k) {
+      k<<<(unsigned)((n + 255) / 256), 256, 0, st>>>((const bf16*)proj, ps, c0, (const bf16*)w, (const bf16*)b, C, tok_seg,
+                                                     seg, (const bf16*)state, (bf16*)out, T, silu, residual);
+    };
+    if (taps == 2) runs ? a(short_conv_vec8_kernel<2, 8>) : a(short_conv_vec8_kernel<2, 1>);
+    else if (taps == 3) runs ? a(short_conv_vec8_kernel<3, 8>) : a(short_conv_vec8_kernel<3, 1>);
+    else runs ? a(short_conv_vec8_kernel<4, 8>) : a(short_conv_vec8_kernel<4, 1>);
+    conv_state_kernel<bf16><<<(int)(((int64_t)R * C + 255) / 256), 256, 0, st>>>((const bf16*)proj, ps, c0, C, taps, seg,
+                                                                                 (bf16*)state, R);
+    return hipGetLastError();
+  }
   DISPATCH_AT(f32, {
     short_conv_kernel<AT><<<ew_grid(T * C), 256, 0, st>>>((const AT*)proj, ps, c0, (const AT*)w, (const AT*)b, C, taps,
                                                           tok_seg, seg, (const AT*)state, (AT*)out, T, silu, residual);

@@ -162,7 +162,7 @@ int kafka_hy_lin_chunk();
 hipError_t kafka_hy_lin_scan(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
                              const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
                              int64_t beta_s, int H, int G, int D, int Dv, float qscale, float inv_tau, const int* seg,
-                             int R, int max_n, float* S, float* out, int64_t os, hipStream_t st);
+                             int R, int min_n, int max_n, float* S, float* out, int64_t os, hipStream_t st);
 int64_t kafka_hy_lin_chunk_scratch(int D, int Dv, int delta);
 hipError_t kafka_hy_lin_chunked(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
                                 const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
@@ -1125,10 +1125,10 @@ void ff_act(at::Tensor u, at::Tensor out, bool glu) {
 
 // The linear-attention recurrence. rate / beta given: gated delta rule. vseg / cs given: the segments of cs in chunks
 // (the tables come from ops.hybrid.lin_chunk_tables, which keeps chunks inside their segments and numbers them
-// 0 .. n - 1); else seg's segments of up to max_n rows token by token.
+// 0 .. n - 1); else seg's segments of min_n .. max_n rows token by token.
 void lin_scan(at::Tensor qk, int64_t q_off, int64_t k_off, at::Tensor v, at::Tensor z, at::Tensor z_bias, OptT rate,
               OptT beta, int64_t H, int64_t G, int64_t D, int64_t Dv, double qscale, double inv_tau, at::Tensor seg,
-              int64_t max_n, OptT cs, at::Tensor S, at::Tensor out) {
+              int64_t min_n, int64_t max_n, OptT cs, at::Tensor S, at::Tensor out) {
   rows2d(qk, "qk"); rows2d(v, "v"); rows2d(z, "z"); rows2d(out, "out");
   f32t(z_bias, "z_bias"); f32t(S, "S"); f32t(out, "out");
   const int f32 = act_f32(qk);
@@ -1164,7 +1164,8 @@ void lin_scan(at::Tensor qk, int64_t q_off, int64_t k_off, at::Tensor v, at::Ten
   }
   HY_HIP(kafka_hy_lin_scan(f32, qk.data_ptr(), qk.stride(0), (int)q_off, (int)k_off, v.data_ptr(), v.stride(0),
                            z.data_ptr(), z.stride(0), z_bias.data_ptr<float>(), rp, bp, bst, (int)H, (int)G, (int)D,
-                           (int)Dv, (float)qscale, (float)inv_tau, seg.data_ptr<int>(), (int)seg.size(0), (int)max_n,
+                           (int)Dv, (float)qscale, (float)inv_tau, seg.data_ptr<int>(), (int)seg.size(0), (int)min_n,
+                           (int)max_n,
                            S.data_ptr<float>(), out.data_ptr<float>(), out.stride(0), stream()));
 }
 

@@ -638,6 +638,39 @@ __global__ __launch_bounds__(NT) void head_norm_gate_kernel(const float* __restr
   }
 }
 
+// the same for heads of 4 L columns (L = 4 .. 64 lanes, a power of two) and rows that can be moved four elements at a time
+template <typename AT, int L>
+__global__ __launch_bounds__(NT) void head_norm_gate_vec4_kernel(const float* __restrict__ o, int64_t os_,
+                                                                 const AT* __restrict__ w, const AT* __restrict__ g,
+                                                                 int64_t gs, int g_off, int H, float eps,
+                                                                 AT* __restrict__ out, int64_t outs, int64_t pairs,
+                                                                 float scale, bool silu) {
+  typedef AT at4 __attribute__((ext_vector_type(4)));
+  const int64_t pair = (int64_t)blockIdx.x * (NT / L) + threadIdx.x / L;
+  if (pair >= pairs) return;   // (whole groups of L lanes leave)
+  const int64_t t = pair / H;
+  const int c = (int)(pair - t * H) * 4 * L + 4 * (threadIdx.x % L);
+  f32x4 v = *reinterpret_cast<const f32x4*>(o + t * os_ + c);
+  const at4 wv = *reinterpret_cast<const at4*>(w + c);
+  at4 gv = {0, 0, 0, 0};
+  if (g != nullptr) gv = *reinterpret_cast<const at4*>(g + t * gs + g_off + c);
+  float s = (v[0] * v[0] + v[1] * v[1]) + (v[2] * v[2] + v[3] * v[3]);
+#pragma unroll
+  for (int x = L / 2; x > 0; x >>= 1) s += __shfl_xor(s, x, L);
+  const float rs = 1.0f / sqrtf(s / (float)(4 * L) + eps);
+  at4 r;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    float y = v[e] * rs * (float)wv[e] * scale;
+    if (g != nullptr) {
+      const float z = (float)gv[e];
+      y *= silu ? z * sigmoidf(z) : sigmoidf(z);
+    }
+    r[e] = (AT)y;
+  }
+  *reinterpret_cast<at4*>(out + t * outs + c) = r;
+}
+
 // ---- routed feed-forward ---------------------------------------------------------------------------------------------------
 constexpr int RT_MAXE = 512;  // experts (8 per lane)
 constexpr int RT_MAXK = 16;
@@ -941,6 +974,24 @@ hipError_t kafka_hy_head_norm_gate(int f32, const float* o, int64_t os_, const v
   if (T <= 0) return hipSuccess;
   const int64_t pairs = T * H;
   const int grid = (int)((pairs + NT / 64 - 1) / (NT / 64));
+  auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  const int L = Dv / 4;
+  if (Dv % 4 == 0 && L >= 4 && L <= 64 && (L & (L - 1)) == 0 && os_ % 4 == 0 && outs % 4 == 0 && gs % 4 == 0 &&
+      g_off % 4 == 0 && al(o) && al(w) && al(g) && (reinterpret_cast<uintptr_t>(out) & (f32 ? 15 : 7)) == 0) {
+    const unsigned blocks = (unsigned)((pairs * L + NT - 1) / NT);
+    DISPATCH_AT(f32, {
+      auto a = [&](auto k) {
+        k<<<blocks, NT, 0, st>>>(o, os_, (const AT*)w, (const AT*)g, gs, g_off, H, eps, (AT*)out, outs, pairs, scale,
+                                 silu != 0);
+      };
+      if (L == 4) a(head_norm_gate_vec4_kernel<AT, 4>);
+      else if (L == 8) a(head_norm_gate_vec4_kernel<AT, 8>);
+      else if (L == 16) a(head_norm_gate_vec4_kernel<AT, 16>);
+      else if (L == 32) a(head_norm_gate_vec4_kernel<AT, 32>);
+      else a(head_norm_gate_vec4_kernel<AT, 64>);
+    });
+    return hipGetLastError();
+  }
   DISPATCH_AT(f32, {
     head_norm_gate_kernel<AT><<<grid, NT, 0, st>>>(o, os_, (const AT*)w, (const AT*)g, gs, g_off, H, Dv, eps, (AT*)out,
                                                    outs, pairs, scale, silu != 0);

@@ -14,11 +14,12 @@
 //   lin_scan     token by token: one workgroup per (segment, head, 64 value columns), a wave owns 16 columns (a thread:
 //                a quarter of the rows of one column, in registers), so that the row sums stay inside the wave; 8
 //                tokens' inputs are staged in LDS, double buffered, one barrier per block
+//   lin_step     segments of one token (decode): the state moves through registers once in 16-byte pieces
 //   lin_chunk_prep / lin_chunk_scan   long segments in chunks of 32 tokens. With b_t the running sum of the chunk's log
 //                decays, the chunk's outputs and its new state are matrix products:
 //                  P[t][j] = q_t . (k_j e^(b_t - b_j)) (j <= t),  A[t][j] = beta_t k_t . (k_j e^(b_t - b_j)) (j < t)
 //                  U = V,  or for the delta rule  (I + A) U = diag(beta) (V - (K e^b) S), i.e. U = U0 - W S with
-//                  (I + A) [W | U0] = diag(beta) [K e^b | V] (forward substitution)
+//                  [W | U0] = (I + A)^(-1) diag(beta) [K e^b | V]
 //                  O = (Q e^b) S + P U,   S <- diag(e^(b_end)) S + (K e^(b_end - b))^T U
 //                prep computes everything that does not depend on S for all chunks in parallel; scan walks a
 //                sequence's chunks with 16 value columns of S in the accumulators of a workgroup, all products on
@@ -215,8 +216,8 @@ constexpr float UNIT_EPS = 1e-6f;
 constexpr int LS_TB = 8;   // tokens per staged block
 
 template <typename AT, int RD, bool DELTA>
-__global__ __launch_bounds__(NT) void lin_scan_kernel(LinIn<AT> in, const int* __restrict__ seg, int max_n,
-                                                      float* __restrict__ Sst, float* __restrict__ out, int64_t os) {
+__global__ __launch_bounds__(NT) void lin_scan_kernel(LinIn<AT> in, const int* __restrict__ seg, int min_n,
+                                                      int max_n, float* __restrict__ Sst, float* __restrict__ out, int64_t os) {
   constexpr int DMAX = 4 * RD;
   constexpr int LROW = DMAX + 16;            // a row group's rows are shifted by 4 floats: reads of the groups spread
   constexpr int NE = (DMAX + 63) / 64;       // elements of a staged row per lane
@@ -225,8 +226,8 @@ __global__ __launch_bounds__(NT) void lin_scan_kernel(LinIn<AT> in, const int* _
   __shared__ float bs[2][LS_TB];
   const int r = blockIdx.z, h = blockIdx.y, v0 = blockIdx.x * 64;
   const int q0 = seg[4 * r], n = seg[4 * r + 1], p0 = seg[4 * r + 2], slot = seg[4 * r + 3];
-  if (n > max_n) return;   // (uniform) a segment that the chunk kernels take
-  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63, rg = lane >> 4;
+  if (n > max_n || n < min_n) return;   // (uniform) a segment that the chunk or the step kernel takes
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, rg = lane >> 4;
   const int col = w * 16 + (lane & 15);
   const bool vok = v0 + col < in.Dv;
   const int D = in.D, g = h / (in.H / in.G);
@@ -363,15 +364,26 @@ constexpr float MIN_LOG2 = -43.f; // log2 decays of one token are cut off here (
 __device__ __forceinline__ f32x4 mfma16f(float a, float b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
+// The wait states a matrix product's result needs before another instruction reads it. The compiler inserts them within
+// straight-line code, but was seen to leave them out where a branch lies between the product and the reader: products
+// whose results are read behind a branch are kept out of conditional code and followed by this.
+__device__ __forceinline__ void mfma_settle() {
+  __builtin_amdgcn_sched_barrier(0);
+  asm volatile("s_nop 15");
+  __builtin_amdgcn_sched_barrier(0);
+}
 
-// Scratch of a chunk and head, index ch = chunk H + head (Dp = D rounded up to 16, NV = ceil(Dv / 16)):
+// Scratch of a chunk and head, index ch = chunk H + head (Dp = D rounded up to 16, NV = ceil(Dv / 16)). "Fragments": 16 x
+// 16 tiles in the operand layout of the scan's products, [64 lanes][4], lane l holding columns 4 (l / 16) .. + 3 of row
+// l % 16 (a lane's four values serve four steps; which of the tile's columns a step takes does not matter as long as
+// both operands agree).
 struct ChunkBuf {
-  float* Q;    // [32][Dp]     q_t e^(b_t)
-  float* W;    // [32][Dp]     delta rule: rows of W
-  float* K;    // [Dp][32]     k_t e^(b_end - b_t), channel-major
+  float* Q;    // [2][Dp / 16] fragments: rows t, columns d of q_t e^(b_t)
+  float* W;    // [2][Dp / 16] fragments: rows t, columns d of W (delta rule)
+  float* K;    // [Dp / 16][2] fragments: rows d, columns t of k_t e^(b_end - b_t)
   float* E;    // [Dp]         e^(b_end)
   float* P;    // [32][32]
-  float* U;    // [2][NV][64][4]  delta rule: U0 in the accumulator layout of the scan
+  float* U;    // [2][NV] tiles of U0 in the accumulator layout: lane l holds rows 4 (l / 16) .. + 3 of column l % 16
 };
 
 // out[row m of x][row n of y] over the DS channels of two LDS slices, 16 x 16, channel order permuted alike in both
@@ -387,237 +399,310 @@ __device__ __forceinline__ f32x4 block_dot(const float* x, const float* y, int l
   return acc;
 }
 
-// One workgroup per (chunk, head). Channels go by in slices of 64: wave w holds rows 8 w .. 8 w + 7, a lane one channel.
-// e^(b_t - b_j) is split at the start of row t's block (reference r): e^(b_t - r) <= 1 for row t, e^(r - b_j) for key j -
-// also <= 1 for keys of an earlier block; within a block it grows to e^(the block's decay), which is formed only while
-// that stays below 2^60. A slice with a faster decay takes its within-block products pair by pair.
-template <typename AT, bool DELTA>
+constexpr int LA = CH + 4;   // LDS row stride of the 32 x 32 matrices
+
+// One workgroup per (chunk, head). Channels go by in NS slices of 64: wave w holds rows 8 w .. 8 w + 7, a lane one
+// channel of every slice. e^(b_t - b_j) is split at the start of row t's block of 16 (reference r): e^(b_t - r) <= 1 for
+// row t, e^(r - b_j) for key j - also <= 1 for keys of the earlier block; within a block it grows to e^(the block's
+// decay), which is formed only while that stays below 2^60. A slice with a faster decay takes its within-block products
+// pair by pair. The delta rule's unit lower triangular I + A is inverted by blocks of 16 (forward substitution on the
+// diagonal, T21 = -T22 A21 T11); W and U0 are then products with T diag(beta).
+template <typename AT, int NS, bool DELTA>
 __global__ __launch_bounds__(NT) void lin_chunk_prep_kernel(LinIn<AT> in, const int* __restrict__ vseg, ChunkBuf cb) {
-  __shared__ __attribute__((aligned(16))) float qs[CH * LD], ks[CH * LD], kn[CH * LD], kc[16 * LD];
-  __shared__ __attribute__((aligned(16))) float As[CH * 36];
-  __shared__ float Ps[CH * 36];
+  __shared__ __attribute__((aligned(16))) float qs[CH * LD], kn[CH * LD], kc[16 * LD];
+  __shared__ __attribute__((aligned(16))) float ks[(DELTA ? NS : 1) * CH * LD];   // k_t e^(b_t - r), kept for W
+  __shared__ __attribute__((aligned(16))) float As[DELTA ? CH * LA : 4];
+  __shared__ float Ps[CH * LA];
   __shared__ float tot[4][DS];
-  __shared__ float rq[CH], rk[CH], bt[CH];
+  __shared__ __attribute__((aligned(16))) float e1s[NS * DS];   // e^(decay of the first block) per channel
+  __shared__ float bt[CH];
+  float* Tm = qs;   // the inverse, and the diagonal blocks of A by [key][row]: after the last slice
+  float* At = kn;
   const int c = blockIdx.x, h = blockIdx.y;
   const int t0 = vseg[4 * c], n = vseg[4 * c + 1];
-  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int D = in.D, Dp = (D + 15) & ~15, g = h / (in.H / in.G);
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63;
+  const int m = lane & 15, kq = lane >> 4;
+  const int D = in.D, Dp = (D + 15) & ~15, ndt = Dp >> 4, g = h / (in.H / in.G);
   const int64_t ch = (int64_t)c * in.H + h;
-  const AT* qp = in.qk + in.q_off + (int64_t)g * D;
-  const AT* kp = in.qk + in.k_off + (int64_t)g * D;
-  const AT* zp = in.z + (int64_t)h * D;
   const float rate = DELTA ? in.rate[h] : 0.f;
   float* Qo = cb.Q + ch * CH * Dp;
   float* Ko = cb.K + ch * CH * Dp;
-  float* Wo = DELTA ? cb.W + ch * CH * Dp : nullptr;
-  for (int i = threadIdx.x; i < CH * 36; i += NT) As[i] = Ps[i] = 0.f;
-  if (DELTA) {
+  // ---- this thread's inputs, all slices: 8 rows of one channel each
+  float qv[NS][8], kv[NS][8], b[NS][8], zb[NS];
+  {
+    const AT* qp = in.qk + in.q_off + (int64_t)g * D;
+    const AT* kp = in.qk + in.k_off + (int64_t)g * D;
+    const AT* zp = in.z + (int64_t)h * D;
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {   // unit norms of this wave's rows
+    for (int j = 0; j < 8; ++j) {
       const int t = 8 * w + j;
-      float sq = 0.f, sk = 0.f;
-      if (t < n)
-        for (int d = lane; d < D; d += 64) {
-          const float a = ldf(qp + (int64_t)(t0 + t) * in.qk_s + d), b = ldf(kp + (int64_t)(t0 + t) * in.qk_s + d);
-          sq += a * a;
-          sk += b * b;
-        }
-      sq = wave_sum(sq);
-      sk = wave_sum(sk);
-      if (lane == 0) {
-        rq[t] = in.qscale / sqrtf(sq + UNIT_EPS);
-        rk[t] = 1.0f / sqrtf(sk + UNIT_EPS);
-        bt[t] = t < n ? sigmoidf(ldf(in.beta + (int64_t)(t0 + t) * in.beta_s + h)) : 0.f;
+      const int64_t row = t0 + min(t, n - 1);
+      const AT* qr = qp + row * in.qk_s;
+      const AT* kr = kp + row * in.qk_s;
+      const AT* zr = zp + row * in.z_s;
+#pragma unroll
+      for (int s = 0; s < NS; ++s) {
+        const int d = min(DS * s + lane, D - 1);
+        qv[s][j] = ldf(qr + d);
+        kv[s][j] = ldf(kr + d);
+        b[s][j] = ldf(zr + d);
       }
+    }
+#pragma unroll
+    for (int s = 0; s < NS; ++s) zb[s] = in.z_bias[h * D + min(DS * s + lane, D - 1)];
+  }
+  if (DELTA && threadIdx.x < CH)
+    bt[threadIdx.x] =
+        (int)threadIdx.x < n ? sigmoidf(ldf(in.beta + (int64_t)(t0 + threadIdx.x) * in.beta_s + h)) : 0.f;
+  for (int i = threadIdx.x; i < CH * LA; i += NT) {
+    Ps[i] = 0.f;
+    if (DELTA) As[i] = 0.f;
+  }
+#pragma unroll
+  for (int j = 0; j < 8; ++j) {
+    const bool ok = 8 * w + j < n;
+    float sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+      if (!ok || DS * s + lane >= D) qv[s][j] = kv[s][j] = 0.f;
+      sq += qv[s][j] * qv[s][j];
+      sk += kv[s][j] * kv[s][j];
+    }
+    float fq = in.qscale, fk = 1.0f;
+    if (DELTA) {   // unit vectors
+      fq = in.qscale / sqrtf(wave_sum(sq) + UNIT_EPS);
+      fk = 1.0f / sqrtf(wave_sum(sk) + UNIT_EPS);
+    }
+#pragma unroll
+    for (int s = 0; s < NS; ++s) {
+      qv[s][j] *= fq;
+      kv[s][j] *= fk;
+      const float lg = ok && DS * s + lane < D ? log_decay<DELTA>(b[s][j] + zb[s], rate, in.inv_tau) * LOG2E : 0.f;
+      b[s][j] = fmaxf(lg, MIN_LOG2) + (j > 0 ? b[s][j > 0 ? j - 1 : 0] : 0.f);   // running sum over the wave's rows
     }
   }
-  __syncthreads();
-  const int b0 = w < 2 ? 0 : 1;      // block of this wave's rows
+  const int b0 = w >> 1;   // block of this wave's rows
   f32x4 acc0 = {0, 0, 0, 0}, acc1 = {0, 0, 0, 0};
-  float dp0 = 0.f, dp1 = 0.f, da0 = 0.f, da1 = 0.f;   // pairwise sums of thread (row tid / 16, key tid % 16) per block
-  for (int d0 = 0; d0 < Dp; d0 += DS) {
-    const int d = d0 + lane;
-    float b[8], qv[8], kv[8];
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int t = 8 * w + j;
-      const bool ok = t < n && d < D;
-      const int64_t row = t0 + (t < n ? t : 0);
-      qv[j] = ok ? ldf(qp + row * in.qk_s + d) : 0.f;
-      kv[j] = ok ? ldf(kp + row * in.qk_s + d) : 0.f;
-      b[j] = ok ? ldf(zp + row * in.z_s + d) : 0.f;
-    }
-    const float zb = d < D ? in.z_bias[h * D + d] : 0.f;
-    float run = 0.f;
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int t = 8 * w + j;
-      qv[j] *= DELTA ? rq[t] : in.qscale;
-      if (DELTA) kv[j] *= rk[t];
-      const float lg = (t < n && d < D) ? log_decay<DELTA>(b[j] + zb, rate, in.inv_tau) * LOG2E : 0.f;
-      run += fmaxf(lg, MIN_LOG2);
-      b[j] = run;
-    }
-    tot[w][lane] = run;
-    __syncthreads();
-    const float ref1 = tot[0][lane] + tot[1][lane], bend = ref1 + (tot[2][lane] + tot[3][lane]);
-    // rows of the later block are counted from its start
-    const float before = (w & 1) ? tot[w - 1][lane] : 0.f;
-    const bool fast = !__any(-ref1 > FAST_LOG2 || ref1 - bend > FAST_LOG2);   // (same in all waves)
-    const float e1 = fast_exp2(ref1);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      const int t = 8 * w + j;
-      const float bl = b[j] + before;                      // decay since the block's start
-      const float eb = fast_exp2(bl);
-      const float full = b0 ? eb * e1 : eb;                // e^(b_t)
-      b[j] = bl;
-      qs[t * LD + lane] = qv[j] * eb;
-      if (DELTA) ks[t * LD + lane] = kv[j] * eb;
-      kn[t * LD + lane] = fast ? kv[j] * fast_exp2(-bl) : 0.f;
-      if (!b0) kc[t * LD + lane] = kv[j] * fast_exp2(ref1 - bl);
-      if (d < Dp) {
-        Qo[(int64_t)t * Dp + d] = qv[j] * full;
-        if (DELTA) Wo[(int64_t)t * Dp + d] = bt[t] * kv[j] * full;
-      }
-    }
-    if (d < Dp) {
-      const float endl = b0 ? bend - ref1 : bend;   // decay up to the chunk's end, from this block's start
-#pragma unroll
-      for (int q4 = 0; q4 < 2; ++q4) {
-        f32x4 v;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = kv[4 * q4 + i] * fast_exp2(endl - b[4 * q4 + i]);
-        *reinterpret_cast<f32x4*>(Ko + (int64_t)d * CH + 8 * w + 4 * q4) = v;
-      }
-      if (w == 0) cb.E[ch * Dp + d] = fast_exp2(bend);
-    }
-    __syncthreads();
-    if (w == 2) {
-      acc0 = block_dot(qs + 16 * LD, kc, lane, acc0);
-    } else if (w == 3) {
-      if (DELTA) acc0 = block_dot(ks + 16 * LD, kc, lane, acc0);
-    } else if (fast) {
-      acc0 = block_dot(qs + 16 * w * LD, kn + 16 * w * LD, lane, acc0);
-      if (DELTA) acc1 = block_dot(ks + 16 * w * LD, kn + 16 * w * LD, lane, acc1);
-    }
-    if (!fast) {   // (uniform) pair by pair, from the plain queries, keys and running decays
+  for (int s = 0; s < NS; ++s) {
+    if (DS * s < Dp) {
+      const int d = DS * s + lane;
+      float* kss = ks + (DELTA ? s * CH * LD : 0);
+      __syncthreads();   // (tot and the previous slice's LDS are free)
+      tot[w][lane] = b[s][7];
       __syncthreads();
+      const float ref1 = tot[0][lane] + tot[1][lane], end1 = tot[2][lane] + tot[3][lane];
+      const float before = (w & 1) ? tot[w - 1][lane] : 0.f;                     // rows count from their block's start
+      const bool fast = !__any(-ref1 > FAST_LOG2 || -end1 > FAST_LOG2);          // (the same in all waves)
+      const float e1 = fast_exp2(ref1);
+      const float endl = b0 ? end1 : ref1 + end1;                                // the chunk's end from the block's start
+      f32x4 ko[2];
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
         const int t = 8 * w + j;
-        qs[t * LD + lane] = qv[j];
-        ks[t * LD + lane] = kv[j];
-        kn[t * LD + lane] = b[j];
+        const float bl = b[s][j] + before;
+        b[s][j] = bl;
+        const float eb = fast_exp2(bl);
+        qs[t * LD + lane] = qv[s][j] * eb;
+        if (DELTA) kss[t * LD + lane] = kv[s][j] * eb;
+        kn[t * LD + lane] = fast ? kv[s][j] * fast_exp2(-bl) : 0.f;
+        if (!b0) kc[t * LD + lane] = kv[s][j] * fast_exp2(ref1 - bl);
+        ko[j >> 2][j & 3] = kv[s][j] * fast_exp2(endl - bl);
+      }
+      if (w == 0) e1s[d] = e1;
+      if (d < Dp) {
+#pragma unroll
+        for (int q4 = 0; q4 < 2; ++q4)   // columns 8 w + 4 q4 .. + 3 of row d
+          *reinterpret_cast<f32x4*>(Ko + ((((d >> 4) * 2 + b0) * 64) + (2 * (w & 1) + q4) * 16 + (d & 15)) * 4) = ko[q4];
+        if (w == 0) cb.E[ch * Dp + d] = fast_exp2(ref1 + end1);
       }
       __syncthreads();
-      const int tr = threadIdx.x >> 4, kj = threadIdx.x & 15;
-      if (kj <= tr) {
-        for (int i = 0; i < DS; ++i) {
-          const int a = tr * LD + i, k = kj * LD + i;
-          const float x0 = ks[k] * fast_exp2(kn[a] - kn[k]);
-          const float x1 = ks[k + 16 * LD] * fast_exp2(kn[a + 16 * LD] - kn[k + 16 * LD]);
-          dp0 += qs[a] * x0;
-          dp1 += qs[a + 16 * LD] * x1;
-          da0 += ks[a] * x0;
-          da1 += ks[a + 16 * LD] * x1;
+      // Q fragments of the slice: wave w takes column tile w of both row blocks
+      if (DS * s + 16 * w < Dp) {
+        const int dt = (DS / 16) * s + w;
+        const f32x4 ev = *reinterpret_cast<const f32x4*>(&e1s[16 * dt + 4 * kq]);
+#pragma unroll
+        for (int rt = 0; rt < 2; ++rt) {
+          f32x4 v = *reinterpret_cast<const f32x4*>(qs + (16 * rt + m) * LD + 16 * w + 4 * kq);
+          if (rt) v *= ev;
+          *reinterpret_cast<f32x4*>(Qo + ((rt * ndt + dt) * 64 + lane) * 4) = v;
         }
       }
-    }
-    __syncthreads();   // the slice's LDS is free again
-  }
-  // accumulators -> LDS: wave 0 / 1 the blocks on the diagonal (P, A), wave 2 / 3 the block below it (P / A)
-  {
-    const int cc = lane & 15, r0 = 4 * (lane >> 4);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      if (w < 2) {
-        Ps[(16 * w + r0 + i) * 36 + 16 * w + cc] = acc0[i];
-        As[(16 * w + r0 + i) * 36 + 16 * w + cc] = acc1[i];
-      } else if (w == 2) {
-        Ps[(16 + r0 + i) * 36 + cc] = acc0[i];
-      } else {
-        As[(16 + r0 + i) * 36 + cc] = acc0[i];
+      {   // waves 0 / 1: the blocks on the diagonal, waves 2 / 3 (alike): the block below it; P, and A for the delta rule
+        const int ro = 16 * min(w, 1) * LD;
+        const float* y = w < 2 ? kn + ro : kc;   // (kn is zero in a slice whose pairs are taken one by one)
+        acc0 = block_dot(qs + ro, y, lane, acc0);
+        if (DELTA) acc1 = block_dot(kss + ro, y, lane, acc1);
+        mfma_settle();
       }
-    }
-  }
-  __syncthreads();
-  {
-    const int tr = threadIdx.x >> 4, kj = threadIdx.x & 15;
-    Ps[tr * 36 + kj] += dp0;
-    Ps[(16 + tr) * 36 + 16 + kj] += dp1;
-    As[tr * 36 + kj] += da0;
-    As[(16 + tr) * 36 + 16 + kj] += da1;
-  }
-  __syncthreads();
-  for (int i = threadIdx.x; i < CH * CH; i += NT) {
-    const int t = i / CH, j = i - t * CH;
-    cb.P[ch * CH * CH + i] = j <= t ? Ps[t * 36 + j] : 0.f;
-    if (DELTA) As[t * 36 + j] = j < t ? bt[t] * As[t * 36 + j] : 0.f;
-  }
-  if constexpr (DELTA) {
-    __syncthreads();   // (also: this workgroup's stores of beta k e^b are visible to its threads)
-    // (I + A) X = right-hand side, a thread per column: the channels of W, then the value columns
-    const int NV = (in.Dv + 15) >> 4;
-    for (int col = threadIdx.x; col < Dp + 16 * NV; col += NT) {
-      float x[CH];
-      const int vc = col - Dp;
+      if (!fast) {   // (uniform) pair by pair, from the plain queries, keys and running decays
+        __syncthreads();
 #pragma unroll
-      for (int t = 0; t < CH; ++t) {
-        if (col < Dp)
-          x[t] = Wo[(int64_t)t * Dp + col];
-        else
-          x[t] = (t < n && vc < in.Dv) ? bt[t] * ldf(in.v + (int64_t)(t0 + t) * in.v_s + (int64_t)h * in.Dv + vc) : 0.f;
-      }
-#pragma unroll
-      for (int t = 1; t < CH; ++t) {
-        float s0 = 0.f, s1 = 0.f;
-#pragma unroll
-        for (int j4 = 0; j4 < (t + 3) / 4; ++j4) {
-          const f32x4 a = *reinterpret_cast<const f32x4*>(&As[t * 36 + 4 * j4]);   // (zeros from j = t on)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            if (4 * j4 + i < t) {
-              if (i & 1) s1 += a[i] * x[4 * j4 + i];
-              else s0 += a[i] * x[4 * j4 + i];
-            }
+        for (int j = 0; j < 8; ++j) {
+          const int t = 8 * w + j;
+          qs[t * LD + lane] = qv[s][j];
+          kss[t * LD + lane] = kv[s][j];
+          kn[t * LD + lane] = b[s][j];
+        }
+        __syncthreads();
+        const int tr = threadIdx.x >> 4, kj = threadIdx.x & 15;
+        if (kj <= tr) {
+          float dp0 = 0.f, dp1 = 0.f, da0 = 0.f, da1 = 0.f;
+#pragma unroll 4
+          for (int i = 0; i < DS; ++i) {
+            const int a = tr * LD + i, k = kj * LD + i;
+            const float x0 = kss[k] * fast_exp2(kn[a] - kn[k]);
+            const float x1 = kss[k + 16 * LD] * fast_exp2(kn[a + 16 * LD] - kn[k + 16 * LD]);
+            dp0 += qs[a] * x0;
+            dp1 += qs[a + 16 * LD] * x1;
+            da0 += kss[a] * x0;
+            da1 += kss[a + 16 * LD] * x1;
+          }
+          Ps[tr * LA + kj] += dp0;
+          Ps[(16 + tr) * LA + 16 + kj] += dp1;
+          if (DELTA) {
+            As[tr * LA + kj] += da0;
+            As[(16 + tr) * LA + 16 + kj] += da1;
           }
         }
-        x[t] -= s0 + s1;
-        __builtin_amdgcn_sched_barrier(0);   // (row by row: all of A's rows in flight would not fit the registers)
-      }
-      if (col < Dp) {
+        if (DELTA) {   // the decayed keys again, for W
+          __syncthreads();
 #pragma unroll
-        for (int t = 0; t < CH; ++t) Wo[(int64_t)t * Dp + col] = x[t];
-      } else {
-        float* Uo = cb.U + (ch * 2 * NV + (vc >> 4)) * 256 + (vc & 15) * 4;
-#pragma unroll
-        for (int q = 0; q < CH / 4; ++q) {
-          const f32x4 v = {x[4 * q], x[4 * q + 1], x[4 * q + 2], x[4 * q + 3]};
-          *reinterpret_cast<f32x4*>(Uo + (int64_t)(q >> 2) * NV * 256 + (q & 3) * 64) = v;
+          for (int j = 0; j < 8; ++j) kss[(8 * w + j) * LD + lane] = kv[s][j] * fast_exp2(b[s][j]);
         }
       }
+    }
+  }
+  __syncthreads();
+  // accumulators -> LDS: waves 0 / 1 the blocks on the diagonal, wave 2 the block below it
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = 4 * kq + i;
+    if (w < 2) {
+      const int o = (16 * w + r) * LA + 16 * w + m;
+      Ps[o] = m <= r ? Ps[o] + acc0[i] : 0.f;
+      if (DELTA) At[(16 * w + m) * 20 + r] = m < r ? bt[16 * w + r] * (As[o] + acc1[i]) : 0.f;   // [key][row]
+    } else if (w == 2) {
+      Ps[(16 + r) * LA + m] = acc0[i];
+      if (DELTA) As[(16 + r) * LA + m] = bt[16 + r] * acc1[i];
+    }
+  }
+  __syncthreads();
+  if (!DELTA || w > 0) {
+    for (int i = DELTA ? threadIdx.x - 64 : threadIdx.x; i < CH * CH; i += DELTA ? NT - 64 : NT)
+      cb.P[ch * CH * CH + i] = Ps[(i >> 5) * LA + (i & 31)];
+  }
+  if constexpr (DELTA) {
+    if (w == 0) {
+      // inverses of the diagonal blocks, a lane per (block, column); lanes 32 .. 63 repeat lanes 0 .. 31
+      const int blk = kq & 1;
+      float x[16];
+#pragma unroll
+      for (int t = 0; t < 16; ++t) x[t] = t == m ? 1.0f : 0.f;
+#pragma unroll
+      for (int j = 0; j < 15; ++j) {
+#pragma unroll
+        for (int t4 = (j + 1) / 4; t4 < 4; ++t4) {
+          const f32x4 a = *reinterpret_cast<const f32x4*>(&At[(16 * blk + j) * 20 + 4 * t4]);
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (4 * t4 + i > j) x[4 * t4 + i] -= a[i] * x[j];
+        }
+      }
+      if (lane < 32) {
+#pragma unroll
+        for (int t = 0; t < 16; ++t) Tm[(16 * blk + t) * LA + 16 * blk + m] = x[t];
+      }
+      // T21 = -T22 (A21 T11); the inner product's accumulators are the outer one's right operand
+      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+      __builtin_amdgcn_wave_barrier();
+      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+      f32x4 u = {0, 0, 0, 0}, v = {0, 0, 0, 0};
+      const f32x4 a21 = *reinterpret_cast<const f32x4*>(&As[(16 + m) * LA + 4 * kq]);
+      const f32x4 t22 = *reinterpret_cast<const f32x4*>(&Tm[(16 + m) * LA + 16 + 4 * kq]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) u = mfma16f(a21[i], Tm[(4 * kq + i) * LA + m], u);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v = mfma16f(t22[i], u[i], v);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) Tm[(16 + 4 * kq + i) * LA + m] = -v[i];
+    }
+    __syncthreads();
+    // T diag(beta): fragments of its three blocks (rows t, columns j)
+    f32x4 tf[3];
+#pragma unroll
+    for (int q = 0; q < 3; ++q) {
+      const int r = q ? 16 : 0, j0 = q == 2 ? 16 : 0;
+      tf[q] = *reinterpret_cast<const f32x4*>(&Tm[(r + m) * LA + j0 + 4 * kq]);
+      const f32x4 bv = {bt[j0 + 4 * kq], bt[j0 + 4 * kq + 1], bt[j0 + 4 * kq + 2], bt[j0 + 4 * kq + 3]};
+      tf[q] *= bv;
+    }
+    float* Wo = cb.W + ch * CH * Dp;
+    for (int dt = w; dt < ndt; dt += 4) {   // transposed tiles of W: rows d, columns t
+      const float* kb = ks + (dt >> 2) * CH * LD + (dt & 3) * 16 + m;
+      const float e1 = e1s[16 * dt + m];
+      f32x4 w0 = {0, 0, 0, 0}, w1 = {0, 0, 0, 0};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float k0 = kb[(4 * kq + i) * LD], k1 = kb[(16 + 4 * kq + i) * LD] * e1;
+        w0 = mfma16f(k0, tf[0][i], w0);
+        w1 = mfma16f(k0, tf[1][i], w1);
+        w1 = mfma16f(k1, tf[2][i], w1);
+      }
+      *reinterpret_cast<f32x4*>(Wo + (dt * 64 + lane) * 4) = w0;
+      *reinterpret_cast<f32x4*>(Wo + ((ndt + dt) * 64 + lane) * 4) = w1;
+    }
+    const int NV = (in.Dv + 15) >> 4;
+    float* Uo = cb.U + ch * 2 * NV * 256;
+    for (int vt = w; vt < NV; vt += 4) {
+      const int vc = min(16 * vt + m, in.Dv - 1);
+      const AT* vp = in.v + (int64_t)h * in.Dv + vc;
+      float vv[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int t = 16 * (i >> 2) + 4 * kq + (i & 3);
+        vv[i] = ldf(vp + (int64_t)(t0 + min(t, n - 1)) * in.v_s);
+        if (t >= n || 16 * vt + m >= in.Dv) vv[i] = 0.f;
+      }
+      f32x4 u0 = {0, 0, 0, 0}, u1 = {0, 0, 0, 0};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        u0 = mfma16f(tf[0][i], vv[i], u0);
+        u1 = mfma16f(tf[1][i], vv[i], u1);
+        u1 = mfma16f(tf[2][i], vv[4 + i], u1);
+      }
+      *reinterpret_cast<f32x4*>(Uo + (vt * 64 + lane) * 4) = u0;
+      *reinterpret_cast<f32x4*>(Uo + ((NV + vt) * 64 + lane) * 4) = u1;
     }
   }
 }
 
 // One workgroup per (16 value columns, head, segment): the D x 16 slice of the state sits in the accumulators of its four
-// waves (wave w: row tiles w NTL .. w NTL + NTL - 1). An accumulator register i of lane l holds row 4 (l / 16) + i,
-// column l % 16 of its tile, which is the right operand of a product over the rows {i, 4 + i, 8 + i, 12 + i}: the
-// state enters the products straight from the registers. Per chunk: W S and (Q e^b) S over the wave's rows; the
-// waves' parts of W S are summed through LDS to U; the state's update; a quarter of P U per wave; the waves' parts of
-// the output summed through LDS. The next chunk's operands are loaded meanwhile.
-template <typename AT, int NTL, bool DELTA>
-__global__ __launch_bounds__(NT) void lin_chunk_scan_kernel(LinIn<AT> in, const int* __restrict__ vseg,
-                                                            const int* __restrict__ cs, ChunkBuf cb,
-                                                            float* __restrict__ Sst, float* __restrict__ out,
-                                                            int64_t os) {
+// waves (wave w: row tiles w NTL .. w NTL + NTL - 1; FULL: D = 64 NTL, every wave has all its tiles). An accumulator
+// register i of lane l holds row 4 (l / 16) + i, column l % 16 of its tile, which is the right operand of a product over
+// the rows {i, 4 + i, 8 + i, 12 + i}: the state enters the products straight from the registers. Per chunk: W S and
+// (Q e^b) S over the wave's rows; the waves' parts of W S are summed through LDS to U; the state's update; a quarter of
+// P U per wave; the waves' parts of the output summed through LDS. The operands of the next two chunks are in flight.
+// The column tiles of a head are given to workgroups of one XCD where the heads divide by 8: they read the same operands.
+template <typename AT, int NTL, bool FULL, bool DELTA>
+__global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(1, NTL > 2 ? 1 : 2))) void lin_chunk_scan_kernel(
+    LinIn<AT> in, const int* __restrict__ vseg, const int* __restrict__ cs, ChunkBuf cb, float* __restrict__ Sst,
+    float* __restrict__ out, int64_t os) {
   __shared__ f32x4 red[4][2][64];
   __shared__ __attribute__((aligned(16))) f32x4 redo[2][4][2][64];
-  const int vt = blockIdx.x, h = blockIdx.y, r = blockIdx.z;
-  const int first = cs[4 * r], cnt = cs[4 * r + 1], p0 = cs[4 * r + 2], slot = cs[4 * r + 3];
-  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63, m = lane & 15, kq = lane >> 4;
   const int D = in.D, Dv = in.Dv, Dp = (D + 15) & ~15, NV = (Dv + 15) >> 4, ndt = Dp >> 4;
+  int vt, h;
+  if (in.H % 8 == 0) {
+    const int q = blockIdx.x >> 3;
+    vt = q % NV;
+    h = (q / NV) * 8 + (blockIdx.x & 7);
+  } else {
+    vt = blockIdx.x % NV;
+    h = blockIdx.x / NV;
+  }
+  const int r = blockIdx.y;
+  const int first = cs[4 * r], cnt = cs[4 * r + 1], p0 = cs[4 * r + 2], slot = cs[4 * r + 3];
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), lane = threadIdx.x & 63, m = lane & 15, kq = lane >> 4;
   const int vcol = vt * 16 + m;
   float* Sp = Sst + (((int64_t)slot * in.H + h) * D) * Dv + vcol;
   f32x4 S[NTL];
@@ -628,116 +713,129 @@ __global__ __launch_bounds__(NT) void lin_chunk_scan_kernel(LinIn<AT> in, const 
       const int d = (w * NTL + a) * 16 + 4 * kq + i;
       S[a][i] = (p0 > 0 && d < D && vcol < Dv) ? Sp[(int64_t)d * Dv] : 0.f;
     }
-  f32x4 Wr[2][NTL], Qr[2][NTL], Kr[NTL][2], Er[NTL], U[2];
-  f32x2 Pr[2];
-  auto load_a = [&](int c) {
-    const int64_t ch = (int64_t)c * in.H + h;
-#pragma unroll
-    for (int a = 0; a < NTL; ++a) {
-      const int dt = w * NTL + a;
-      if (dt < ndt) {   // (uniform per wave)
-#pragma unroll
-        for (int rt = 0; rt < 2; ++rt) {
-          const int64_t o = (ch * CH + 16 * rt + m) * Dp + dt * 16 + 4 * kq;
-          Qr[rt][a] = *reinterpret_cast<const f32x4*>(cb.Q + o);
-          if (DELTA) Wr[rt][a] = *reinterpret_cast<const f32x4*>(cb.W + o);
-        }
-      }
-    }
+  struct Ops {
+    f32x4 W[2][NTL], Q[2][NTL], K[NTL][2], E[NTL], U[2];
+    f32x2 P[2];
+    int t0, n;
   };
-  auto load_b = [&](int c) {
+  Ops ops[2];
+  // a wave without a tile of its own reads the last tile and holds no state there (its key operand is zeroed): no
+  // product is conditional
+  auto tile = [&](int a) { return FULL ? w * NTL + a : min(w * NTL + a, ndt - 1); };
+  auto load_a = [&](Ops& o, int c) {
     const int64_t ch = (int64_t)c * in.H + h;
+    const float* Qp = cb.Q + ch * CH * Dp + lane * 4;
+    const float* Wp = DELTA ? cb.W + ch * CH * Dp + lane * 4 : nullptr;
+#pragma unroll
+    for (int a = 0; a < NTL; ++a)
+#pragma unroll
+      for (int rt = 0; rt < 2; ++rt) {
+        o.Q[rt][a] = *reinterpret_cast<const f32x4*>(Qp + (rt * ndt + tile(a)) * 256);
+        if (DELTA) o.W[rt][a] = *reinterpret_cast<const f32x4*>(Wp + (rt * ndt + tile(a)) * 256);
+      }
+  };
+  auto load_b = [&](Ops& o, int c) {
+    const int64_t ch = (int64_t)c * in.H + h;
+    const float* Kp = cb.K + ch * CH * Dp + lane * 4;
+    o.t0 = vseg[4 * c];
+    o.n = vseg[4 * c + 1];
 #pragma unroll
     for (int a = 0; a < NTL; ++a) {
-      const int dt = w * NTL + a;
-      if (dt < ndt) {
 #pragma unroll
-        for (int tt = 0; tt < 2; ++tt)
-          Kr[a][tt] = *reinterpret_cast<const f32x4*>(cb.K + (ch * Dp + dt * 16 + m) * CH + 16 * tt + 4 * kq);
-        Er[a] = *reinterpret_cast<const f32x4*>(cb.E + ch * Dp + dt * 16 + 4 * kq);
-      }
+      for (int tt = 0; tt < 2; ++tt) o.K[a][tt] = *reinterpret_cast<const f32x4*>(Kp + (tile(a) * 2 + tt) * 256);
+      o.E[a] = *reinterpret_cast<const f32x4*>(cb.E + ch * Dp + tile(a) * 16 + 4 * kq);
     }
 #pragma unroll
     for (int rt = 0; rt < 2; ++rt)
-      Pr[rt] = *reinterpret_cast<const f32x2*>(cb.P + ch * CH * CH + (16 * rt + m) * CH + 16 * (w >> 1) + 4 * kq + 2 * (w & 1));
+      o.P[rt] = *reinterpret_cast<const f32x2*>(cb.P + ch * CH * CH + (16 * rt + m) * CH + 16 * (w >> 1) + 4 * kq +
+                                                2 * (w & 1));
     if constexpr (DELTA) {
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt)
-        U[tt] = *reinterpret_cast<const f32x4*>(cb.U + ((ch * 2 + tt) * NV + vt) * 256 + lane * 4);
+        o.U[tt] = *reinterpret_cast<const f32x4*>(cb.U + ((ch * 2 + tt) * NV + vt) * 256 + lane * 4);
     } else {
-      const int t0 = vseg[4 * c], n = vseg[4 * c + 1];
+      const AT* vp = in.v + (int64_t)o.t0 * in.v_s + (int64_t)h * Dv + min(vcol, Dv - 1);
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = 16 * tt + 4 * kq + i;
-          U[tt][i] = (t < n && vcol < Dv) ? ldf(in.v + (int64_t)(t0 + t) * in.v_s + (int64_t)h * Dv + vcol) : 0.f;
-        }
+        for (int i = 0; i < 4; ++i) o.U[tt][i] = ldf(vp + (int64_t)min(16 * tt + 4 * kq + i, o.n - 1) * in.v_s);
     }
   };
-  if (cnt > 0) {
-    load_a(first);
-    load_b(first);
-  }
-  for (int c = first; c < first + cnt; ++c) {
+  const int last = first + cnt;
+  auto step = [&](Ops& o, int c) {
     f32x4 ws[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}}, ow[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
 #pragma unroll
-    for (int a = 0; a < NTL; ++a) {
-      if (w * NTL + a < ndt) {
+    for (int a = 0; a < NTL; ++a)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
+      for (int i = 0; i < 4; ++i)
 #pragma unroll
-          for (int rt = 0; rt < 2; ++rt) {
-            if (DELTA) ws[rt] = mfma16f(Wr[rt][a][i], S[a][i], ws[rt]);
-            ow[rt] = mfma16f(Qr[rt][a][i], S[a][i], ow[rt]);
-          }
+        for (int rt = 0; rt < 2; ++rt) {
+          if (DELTA) ws[rt] = mfma16f(o.W[rt][a][i], S[a][i], ws[rt]);
+          ow[rt] = mfma16f(o.Q[rt][a][i], S[a][i], ow[rt]);
         }
-      }
-    }
-    if (c + 1 < first + cnt) load_a(c + 1);
+    mfma_settle();
+    const int t0 = o.t0, n = o.n;
+    if (c + 2 < last) load_a(o, c + 2);
     if constexpr (DELTA) {
       red[w][0][lane] = ws[0];
       red[w][1][lane] = ws[1];
       lds_barrier();
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt)
-        U[tt] -= (red[0][tt][lane] + red[1][tt][lane]) + (red[2][tt][lane] + red[3][tt][lane]);
+        o.U[tt] -= (red[0][tt][lane] + red[1][tt][lane]) + (red[2][tt][lane] + red[3][tt][lane]);
+    } else {
+#pragma unroll
+      for (int tt = 0; tt < 2; ++tt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (16 * tt + 4 * kq + i >= n || vcol >= Dv) o.U[tt][i] = 0.f;
     }
     {
-      const f32x4 us = (w >> 1) ? U[1] : U[0];
+      const f32x4 us = (w >> 1) ? o.U[1] : o.U[0];
       const float u0 = (w & 1) ? us[2] : us[0], u1 = (w & 1) ? us[3] : us[1];
 #pragma unroll
       for (int rt = 0; rt < 2; ++rt) {
-        ow[rt] = mfma16f(Pr[rt][0], u0, ow[rt]);
-        ow[rt] = mfma16f(Pr[rt][1], u1, ow[rt]);
+        ow[rt] = mfma16f(o.P[rt][0], u0, ow[rt]);
+        ow[rt] = mfma16f(o.P[rt][1], u1, ow[rt]);
       }
     }
     f32x4* ro = &redo[c & 1][0][0][0];
     ro[(w * 2 + 0) * 64 + lane] = ow[0];
     ro[(w * 2 + 1) * 64 + lane] = ow[1];
 #pragma unroll
-    for (int a = 0; a < NTL; ++a)
-      if (w * NTL + a < ndt) S[a] *= Er[a];
+    for (int a = 0; a < NTL; ++a) {
+      S[a] *= o.E[a];
 #pragma unroll
-    for (int tt = 0; tt < 2; ++tt)
+      for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
-#pragma unroll
-        for (int a = 0; a < NTL; ++a)
-          if (w * NTL + a < ndt) S[a] = mfma16f(Kr[a][tt][i], U[tt][i], S[a]);
-    const int t0 = vseg[4 * c], n = vseg[4 * c + 1];
-    if (c + 1 < first + cnt) load_b(c + 1);
+        for (int i = 0; i < 4; ++i) {
+          const float k = FULL || w * NTL + a < ndt ? o.K[a][tt][i] : 0.f;
+          S[a] = mfma16f(k, o.U[tt][i], S[a]);
+        }
+    }
+    mfma_settle();
+    if (c + 2 < last) load_b(o, c + 2);
     lds_barrier();
     {
       const int rt = threadIdx.x >> 7, l2 = (threadIdx.x & 127) >> 1, part = threadIdx.x & 1;
       const f32x2* rp = reinterpret_cast<const f32x2*>(ro) + (rt * 64 + l2) * 2 + part;
-      const f32x2 o = (rp[0] + rp[256]) + (rp[512] + rp[768]);
+      const f32x2 ov = (rp[0] + rp[256]) + (rp[512] + rp[768]);
       const int t = 16 * rt + 4 * (l2 >> 4) + 2 * part, v = vt * 16 + (l2 & 15);
       if (v < Dv) {
-        if (t < n) out[(int64_t)(t0 + t) * os + (int64_t)h * Dv + v] = o[0];
-        if (t + 1 < n) out[(int64_t)(t0 + t + 1) * os + (int64_t)h * Dv + v] = o[1];
+        if (t < n) out[(int64_t)(t0 + t) * os + (int64_t)h * Dv + v] = ov[0];
+        if (t + 1 < n) out[(int64_t)(t0 + t + 1) * os + (int64_t)h * Dv + v] = ov[1];
       }
     }
+  };
+#pragma unroll
+  for (int k = 0; k < 2; ++k)
+    if (k < cnt) {
+      load_a(ops[k], first + k);
+      load_b(ops[k], first + k);
+    }
+  for (int c = first; c < last; c += 2) {
+    step(ops[0], c);
+    if (c + 1 < last) step(ops[1], c + 1);
   }
 #pragma unroll
   for (int a = 0; a < NTL; ++a)
@@ -746,6 +844,101 @@ __global__ __launch_bounds__(NT) void lin_chunk_scan_kernel(LinIn<AT> in, const 
       const int d = (w * NTL + a) * 16 + 4 * kq + i;
       if (d < D && vcol < Dv) Sp[(int64_t)d * Dv] = S[a][i];
     }
+}
+
+// ---- one token per segment -------------------------------------------------------------------------------------------
+// Decode steps move the whole state through once: one workgroup per (segment of one row, head, 64 value columns), thread
+// (rg, cq) keeps rows rg, 16 + rg, ... of four columns (16-byte loads, 256 contiguous bytes per row). The state's loads are
+// issued first; q, k and the decays are staged meanwhile, their norms enter as factors of the products.
+template <typename AT, int NR, bool DELTA>
+__global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void lin_step_kernel(
+    LinIn<AT> in, const int* __restrict__ seg, float* __restrict__ Sst, float* __restrict__ out, int64_t os) {
+  __shared__ float qsh[16 * NR], ksh[16 * NR], fsh[16 * NR];
+  __shared__ float nrm[2][4];
+  __shared__ __attribute__((aligned(16))) float red[2][4][64];
+  const int r = blockIdx.z, h = blockIdx.y, v0 = blockIdx.x * 64;
+  const int q0 = seg[4 * r], n = seg[4 * r + 1], p0 = seg[4 * r + 2], slot = seg[4 * r + 3];
+  if (n != 1) return;   // (uniform)
+  const int tid = threadIdx.x, w = tid >> 6, lane = tid & 63, rg = tid >> 4, cq = tid & 15;
+  const int D = in.D, Dv = in.Dv, g = h / (in.H / in.G);
+  const int c4 = v0 + 4 * cq;
+  const bool vok = c4 < Dv;
+  float* Sp = Sst + (((int64_t)slot * in.H + h) * D) * Dv + c4;
+  f32x4 S[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int d = 16 * i + rg;
+    S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (p0 > 0 && d < D && vok) S[i] = *reinterpret_cast<const f32x4*>(Sp + (int64_t)d * Dv);
+  }
+  float vx[4] = {0.f, 0.f, 0.f, 0.f};
+  if (vok) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) vx[e] = ldf(in.v + (int64_t)q0 * in.v_s + (int64_t)h * Dv + c4 + e);
+  }
+  const float beta = DELTA ? sigmoidf(ldf(in.beta + (int64_t)q0 * in.beta_s + h)) : 0.f;
+  float q = 0.f, k = 0.f;
+  if (tid < 16 * NR) {   // (channels past D: q = k = 0, decay 1)
+    float f = 1.0f;
+    if (tid < D) {
+      q = ldf(in.qk + (int64_t)q0 * in.qk_s + in.q_off + (int64_t)g * D + tid);
+      k = ldf(in.qk + (int64_t)q0 * in.qk_s + in.k_off + (int64_t)g * D + tid);
+      f = expf(log_decay<DELTA>(ldf(in.z + (int64_t)q0 * in.z_s + (int64_t)h * D + tid) + in.z_bias[h * D + tid],
+                                DELTA ? in.rate[h] : 0.f, in.inv_tau));
+    }
+    qsh[tid] = q;
+    ksh[tid] = k;
+    fsh[tid] = f;
+  }
+  if (DELTA) {
+    const float sq = wave_sum(q * q), sk = wave_sum(k * k);
+    if (lane == 0) {
+      nrm[0][w] = sq;
+      nrm[1][w] = sk;
+    }
+  }
+  lds_barrier();
+  float fq = in.qscale, fk = 1.0f;
+  if (DELTA) {
+    fq = in.qscale / sqrtf((nrm[0][0] + nrm[0][1]) + (nrm[0][2] + nrm[0][3]) + UNIT_EPS);
+    fk = 1.0f / sqrtf((nrm[1][0] + nrm[1][1]) + (nrm[1][2] + nrm[1][3]) + UNIT_EPS);
+  }
+  // sums over all rows of a column: across the wave's four row groups, then across the waves
+  auto col_sum = [&](f32x4 v, int buf) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v[e] += __shfl_xor(v[e], 16, 64);
+      v[e] += __shfl_xor(v[e], 32, 64);
+    }
+    if (lane < 16) *reinterpret_cast<f32x4*>(&red[buf][w][4 * cq]) = v;
+    lds_barrier();
+    f32x4 s = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) s += *reinterpret_cast<const f32x4*>(&red[buf][i][4 * cq]);
+    return s;
+  };
+  f32x4 u = {vx[0], vx[1], vx[2], vx[3]};
+  if constexpr (DELTA) {
+    f32x4 dot = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      S[i] *= fsh[16 * i + rg];
+      dot += S[i] * ksh[16 * i + rg];
+    }
+    dot = col_sum(dot, 0);
+    u = (u - dot * fk) * (beta * fk);   // (beta (v - S^T k), times the key's norm)
+  }
+  f32x4 o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int d = 16 * i + rg;
+    if (!DELTA) S[i] *= fsh[d];
+    S[i] += u * ksh[d];
+    o += S[i] * qsh[d];
+    if (d < D && vok) *reinterpret_cast<f32x4*>(Sp + (int64_t)d * Dv) = S[i];
+  }
+  o = col_sum(o, 1);
+  if (rg == 0 && vok) *reinterpret_cast<f32x4*>(out + (int64_t)q0 * os + (int64_t)h * Dv + c4) = o * fq;
 }
 
 static inline int ew_grid(int64_t n) { return (int)std::min<int64_t>((n + 255) / 256, 65535 * 4); }
@@ -816,23 +1009,41 @@ int kafka_hy_lin_chunk() { return CH; }
 hipError_t kafka_hy_lin_scan(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
                              const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
                              int64_t beta_s, int H, int G, int D, int Dv, float qscale, float inv_tau, const int* seg,
-                             int R, int max_n, float* S, float* out, int64_t os, hipStream_t st) {
+                             int R, int min_n, int max_n, float* S, float* out, int64_t os, hipStream_t st) {
   if (R <= 0) return hipSuccess;
   if (D < 1 || D > 256 || Dv < 1 || G < 1 || H % G || H > 65535 || R > 65535 || (rate != nullptr) != (beta != nullptr))
     return hipErrorInvalidValue;
   const dim3 grid((Dv + 63) / 64, H, R);
+  // segments of one row: the step kernel, where rows of four columns can be moved in 16-byte pieces
+  const bool step = min_n <= 1 && Dv % 4 == 0 && os % 4 == 0 && (reinterpret_cast<uintptr_t>(S) & 15) == 0 &&
+                    (reinterpret_cast<uintptr_t>(out) & 15) == 0;
   DISPATCH_AT(f32, {
     const LinIn<AT> in{(const AT*)qk, (const AT*)v, (const AT*)z, (const AT*)beta, z_bias, rate, qk_s, v_s, z_s, beta_s,
                        q_off, k_off, H, G, D, Dv, qscale, inv_tau};
-    auto a = [&](auto k) { k<<<grid, NT, 0, st>>>(in, seg, max_n, S, out, os); };
+    auto a = [&](auto k) { k<<<grid, NT, 0, st>>>(in, seg, step ? 2 : min_n, max_n, S, out, os); };
+    auto a1 = [&](auto k) { k<<<grid, NT, 0, st>>>(in, seg, S, out, os); };
     if (rate != nullptr) {
-      if (D <= 64) a(lin_scan_kernel<AT, 16, true>);
-      else if (D <= 128) a(lin_scan_kernel<AT, 32, true>);
-      else a(lin_scan_kernel<AT, 64, true>);
+      if (step) {
+        if (D <= 64) a1(lin_step_kernel<AT, 4, true>);
+        else if (D <= 128) a1(lin_step_kernel<AT, 8, true>);
+        else a1(lin_step_kernel<AT, 16, true>);
+      }
+      if (max_n > 1 || !step) {
+        if (D <= 64) a(lin_scan_kernel<AT, 16, true>);
+        else if (D <= 128) a(lin_scan_kernel<AT, 32, true>);
+        else a(lin_scan_kernel<AT, 64, true>);
+      }
     } else {
-      if (D <= 64) a(lin_scan_kernel<AT, 16, false>);
-      else if (D <= 128) a(lin_scan_kernel<AT, 32, false>);
-      else a(lin_scan_kernel<AT, 64, false>);
+      if (step) {
+        if (D <= 64) a1(lin_step_kernel<AT, 4, false>);
+        else if (D <= 128) a1(lin_step_kernel<AT, 8, false>);
+        else a1(lin_step_kernel<AT, 16, false>);
+      }
+      if (max_n > 1 || !step) {
+        if (D <= 64) a(lin_scan_kernel<AT, 16, false>);
+        else if (D <= 128) a(lin_scan_kernel<AT, 32, false>);
+        else a(lin_scan_kernel<AT, 64, false>);
+      }
     }
   });
   return hipGetLastError();
@@ -862,21 +1073,30 @@ hipError_t kafka_hy_lin_chunked(int f32, const void* qk, int64_t qk_s, int q_off
   cb.W = cb.P + N * CH * CH;
   cb.U = cb.W + N * CH * Dp;
   if (rate == nullptr) cb.W = cb.U = nullptr;
-  const dim3 g1(n_chunks, H), g2((unsigned)NV, H, R);
+  const dim3 g1(n_chunks, H), g2((unsigned)(NV * H), R);
   DISPATCH_AT(f32, {
     const LinIn<AT> in{(const AT*)qk, (const AT*)v, (const AT*)z, (const AT*)beta, z_bias, rate, qk_s, v_s, z_s, beta_s,
                        q_off, k_off, H, G, D, Dv, qscale, inv_tau};
+    auto p = [&](auto k) { k<<<g1, NT, 0, st>>>(in, vseg, cb); };
     auto b = [&](auto k) { k<<<g2, NT, 0, st>>>(in, vseg, cs, cb, S, out, os); };
     if (rate != nullptr) {
-      lin_chunk_prep_kernel<AT, true><<<g1, NT, 0, st>>>(in, vseg, cb);
-      if (D <= 64) b(lin_chunk_scan_kernel<AT, 1, true>);
-      else if (D <= 128) b(lin_chunk_scan_kernel<AT, 2, true>);
-      else b(lin_chunk_scan_kernel<AT, 4, true>);
+      if (D <= 64) p(lin_chunk_prep_kernel<AT, 1, true>);
+      else if (D <= 128) p(lin_chunk_prep_kernel<AT, 2, true>);
+      else p(lin_chunk_prep_kernel<AT, 4, true>);
+      if (D == 64) b(lin_chunk_scan_kernel<AT, 1, true, true>);
+      else if (D == 128) b(lin_chunk_scan_kernel<AT, 2, true, true>);
+      else if (D < 64) b(lin_chunk_scan_kernel<AT, 1, false, true>);
+      else if (D < 128) b(lin_chunk_scan_kernel<AT, 2, false, true>);
+      else b(lin_chunk_scan_kernel<AT, 4, false, true>);
     } else {
-      lin_chunk_prep_kernel<AT, false><<<g1, NT, 0, st>>>(in, vseg, cb);
-      if (D <= 64) b(lin_chunk_scan_kernel<AT, 1, false>);
-      else if (D <= 128) b(lin_chunk_scan_kernel<AT, 2, false>);
-      else b(lin_chunk_scan_kernel<AT, 4, false>);
+      if (D <= 64) p(lin_chunk_prep_kernel<AT, 1, false>);
+      else if (D <= 128) p(lin_chunk_prep_kernel<AT, 2, false>);
+      else p(lin_chunk_prep_kernel<AT, 4, false>);
+      if (D == 64) b(lin_chunk_scan_kernel<AT, 1, true, false>);
+      else if (D == 128) b(lin_chunk_scan_kernel<AT, 2, true, false>);
+      else if (D < 64) b(lin_chunk_scan_kernel<AT, 1, false, false>);
+      else if (D < 128) b(lin_chunk_scan_kernel<AT, 2, false, false>);
+      else b(lin_chunk_scan_kernel<AT, 4, false, false>);
     }
   });
   return hipGetLastError();

@@ -738,7 +738,7 @@ def lin_chunk_tables(seg_host):
 
 
 def lin_scan(qk, q_off: int, k_off: int, v, z, z_bias, H: int, G: int, D: int, Dv: int, tok_seg, seg, S, out,
-             tau: float = 1.0, rate=None, beta=None, chunks=None, any_short: bool = True) -> None:
+             tau: float = 1.0, rate=None, beta=None, chunks=None, rows=(1, 1 << 30)) -> None:
     """Linear attention with a decay per head and key channel over a step's segments. q / k: G heads of D columns of
     ``qk`` at q_off / k_off, head h uses q/k head h // (H / G); v [T, H Dv]; z [T, H D] raw decays, z_bias fp32 [H D].
     Per head, with q' = q D^(-1/2):
@@ -748,15 +748,17 @@ def lin_scan(qk, q_off: int, k_off: int, v, z, z_bias, H: int, G: int, D: int, D
                    S <- S + k u^T;  out = S^T q'
     S fp32 [slots, H, D, Dv], zero before a sequence's first token; out fp32 [T, H Dv]. ``chunks``: device tensors of
     ``lin_chunk_tables`` - their segments run in chunks of LIN_CHUNK tokens (the same recurrence as matrix products,
-    re-associated: fp32 rounding only), the others token by token; ``any_short`` False: there are no others."""
+    re-associated: fp32 rounding only), the others token by token. ``rows``: the shortest and the longest of those
+    others when the caller knows them (None: there are none); segments of one row have a kernel of their own."""
     if D > 256:
         raise ValueError("lin_scan: head sizes up to 256")
     if _gpu(qk):
         args = (qk, int(q_off), int(k_off), v, z, z_bias, rate, beta, int(H), int(G), int(D), int(Dv), D ** -0.5,
                 1.0 / float(tau))
         if chunks is not None:
-            ext().hy_lin_scan(*args, chunks[0], 0, chunks[1], S, out)
-        if chunks is None or any_short:
-            ext().hy_lin_scan(*args, seg, LIN_CHUNK_MIN - 1 if chunks is not None else 1 << 30, None, S, out)
+            ext().hy_lin_scan(*args, chunks[0], 0, 0, chunks[1], S, out)
+        if rows is not None:
+            hi = min(rows[1], LIN_CHUNK_MIN - 1) if chunks is not None else rows[1]
+            ext().hy_lin_scan(*args, seg, int(rows[0]), int(hi), None, S, out)
     else:
         ref.lin_scan(qk, q_off, k_off, v, z, z_bias, H, G, D, Dv, tok_seg, seg, S, out, tau, rate, beta)

@@ -218,6 +218,32 @@ def test_feed_forward_activations_and_head_gate(device, F):
             assert close(both[:, 9:], want, tol) and float(both[:, :9].abs().max()) == 0.0
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("C,taps,lengths", [(64, 4, [2100, 30]), (40, 2, [7, 19]), (128, 3, [2050, 1]), (24, 4, [1, 3])])
+def test_short_conv_vectors(C, taps, lengths):
+    """The bf16 vector form of the convolution (a thread per row, or per eight rows in long steps): two sequences from
+    NaN slots, then more of both: windows that reach into the slots' tails, over segment borders inside a thread's rows,
+    and not into the neighbouring sequence."""
+    dev = "cuda:0"
+    g = torch.Generator().manual_seed(C)
+    w = torch.randn(C, taps, generator=g).to(torch.bfloat16)
+    xs = [torch.randn(n + 2100, C + 16, generator=g).to(torch.bfloat16) for n in lengths]
+    want = [plain.silu(plain.short_conv(x[:, 8:8 + C].float(), w.float())) for x in xs]
+    state = torch.full((3, taps - 1, C), float("nan"), dtype=torch.bfloat16, device=dev)
+    at, got = [0, 0], [[], []]
+    for sizes in (lengths, [1, 1], [2, 5], [1, 1], [2090, 3]):
+        segs = [(0, sizes[0], at[0], 2), (sizes[0], sizes[1], at[1], 0)]
+        ts, seg = seg_tensors(dev, segs)
+        x = torch.cat([xs[s][at[s]:at[s] + sizes[s]] for s in (0, 1)]).to(dev)
+        out = torch.empty(x.shape[0], C, dtype=torch.bfloat16, device=dev)
+        hops.short_conv(x, 8, w.to(dev), None, ts, seg, state, out, act="silu")
+        got[0].append(out[:sizes[0]].cpu())
+        got[1].append(out[sizes[0]:].cpu())
+        at = [at[0] + sizes[0], at[1] + sizes[1]]
+    for s in (0, 1):
+        assert close(torch.cat(got[s]).float(), want[s][:at[s]], 1e-2), s
+
+
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("E,k,count,keep", [(12, 3, 4, 2), (16, 3, 2, 1), (6, 2, 1, 1), (8, 4, 8, 4), (130, 6, 10, 3),
                                             (4, 4, 2, 2), (3, 1, 3, 1)])
@@ -314,8 +340,7 @@ def test_lin_scan(device, H, G, D, Dv, delta):
                 tabs = tuple(torch.from_numpy(x).to(device) for x in tabs)
             out = torch.full((r0, H * Dv), float("nan"), device=device)
             hops.lin_scan(cat["qkv"], 0, G * D, cat["qkv"][:, 2 * G * D:], cat["z"], zb.to(device), H, G, D, Dv, ts,
-                          seg, S, out, tau, rate.to(device) if delta else None, cat["beta"] if delta else None, tabs,
-                          any(n < hops.LIN_CHUNK_MIN for _, n, _, _ in segs))
+                          seg, S, out, tau, rate.to(device) if delta else None, cat["beta"] if delta else None, tabs)
             for s, p0, n, q0 in runs:
                 got[s].append(out[q0:q0 + n].cpu())
                 at[s] += n
@@ -355,7 +380,8 @@ def test_lin_scan_in_chunks(delta, n):
             x = {k: v[p0:p0 + m].to(dev) for k, v in c.items()}
             out = torch.empty(m, H * Dv, device=dev)
             hops.lin_scan(x["qkv"], 0, G * D, x["qkv"][:, 2 * G * D:], x["z"], zb.to(dev), H, G, D, Dv, ts, seg, S, out,
-                          tau, rate.to(dev) if delta else None, x["beta"] if delta else None, tabs, tabs is None)
+                          tau, rate.to(dev) if delta else None, x["beta"] if delta else None, tabs,
+                          (m, m) if tabs is None else None)
             got.append(out.cpu())
         outs.append((torch.cat(got), S[1].cpu()))
         assert close(outs[-1][0], want, 3e-5), chunked
