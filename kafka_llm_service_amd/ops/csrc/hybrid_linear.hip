@@ -716,9 +716,11 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(1, NTL > 2 ?
   struct Ops {
     f32x4 W[2][NTL], Q[2][NTL], K[NTL][2], E[NTL], U[2];
     f32x2 P[2];
-    int t0, n;
   };
   Ops ops[2];
+  // a segment's chunks are consecutive rows, all whole but the last
+  const int last = first + cnt, row0 = cnt > 0 ? vseg[4 * first] : 0;
+  const int tail = cnt > 0 ? vseg[4 * (last - 1) + 1] : 0;
   // a wave without a tile of its own reads the last tile and holds no state there (its key operand is zeroed): no
   // product is conditional
   auto tile = [&](int a) { return FULL ? w * NTL + a : min(w * NTL + a, ndt - 1); };
@@ -737,8 +739,6 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(1, NTL > 2 ?
   auto load_b = [&](Ops& o, int c) {
     const int64_t ch = (int64_t)c * in.H + h;
     const float* Kp = cb.K + ch * CH * Dp + lane * 4;
-    o.t0 = vseg[4 * c];
-    o.n = vseg[4 * c + 1];
 #pragma unroll
     for (int a = 0; a < NTL; ++a) {
 #pragma unroll
@@ -754,14 +754,14 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(1, NTL > 2 ?
       for (int tt = 0; tt < 2; ++tt)
         o.U[tt] = *reinterpret_cast<const f32x4*>(cb.U + ((ch * 2 + tt) * NV + vt) * 256 + lane * 4);
     } else {
-      const AT* vp = in.v + (int64_t)o.t0 * in.v_s + (int64_t)h * Dv + min(vcol, Dv - 1);
+      const int rows = c + 1 < last ? CH : tail;
+      const AT* vp = in.v + (int64_t)(row0 + CH * (c - first)) * in.v_s + (int64_t)h * Dv + min(vcol, Dv - 1);
 #pragma unroll
       for (int tt = 0; tt < 2; ++tt)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) o.U[tt][i] = ldf(vp + (int64_t)min(16 * tt + 4 * kq + i, o.n - 1) * in.v_s);
+        for (int i = 0; i < 4; ++i) o.U[tt][i] = ldf(vp + (int64_t)min(16 * tt + 4 * kq + i, rows - 1) * in.v_s);
     }
   };
-  const int last = first + cnt;
   auto step = [&](Ops& o, int c) {
     f32x4 ws[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}}, ow[2] = {{0, 0, 0, 0}, {0, 0, 0, 0}};
 #pragma unroll
@@ -774,7 +774,7 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(1, NTL > 2 ?
           ow[rt] = mfma16f(o.Q[rt][a][i], S[a][i], ow[rt]);
         }
     mfma_settle();
-    const int t0 = o.t0, n = o.n;
+    const int t0 = row0 + CH * (c - first), n = c + 1 < last ? CH : tail;
     if (c + 2 < last) load_a(o, c + 2);
     if constexpr (DELTA) {
       red[w][0][lane] = ws[0];
@@ -863,13 +863,15 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void li
   const int D = in.D, Dv = in.Dv, g = h / (in.H / in.G);
   const int c4 = v0 + 4 * cq;
   const bool vok = c4 < Dv;
-  float* Sp = Sst + (((int64_t)slot * in.H + h) * D) * Dv + c4;
+  // (rows and columns past the head's read its last ones: their keys and queries are zero, nothing of them is stored)
+  float* Sp = Sst + (((int64_t)slot * in.H + h) * D) * Dv + min(c4, Dv - 4);
   f32x4 S[NR];
+  if (p0 > 0) {   // (uniform)
 #pragma unroll
-  for (int i = 0; i < NR; ++i) {
-    const int d = 16 * i + rg;
-    S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (p0 > 0 && d < D && vok) S[i] = *reinterpret_cast<const f32x4*>(Sp + (int64_t)d * Dv);
+    for (int i = 0; i < NR; ++i) S[i] = *reinterpret_cast<const f32x4*>(Sp + min(16 * i + rg, D - 1) * Dv);
+  } else {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) S[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   float vx[4] = {0.f, 0.f, 0.f, 0.f};
   if (vok) {
@@ -935,7 +937,7 @@ __global__ __launch_bounds__(NT) __attribute__((amdgpu_waves_per_eu(4))) void li
     if (!DELTA) S[i] *= fsh[d];
     S[i] += u * ksh[d];
     o += S[i] * qsh[d];
-    if (d < D && vok) *reinterpret_cast<f32x4*>(Sp + (int64_t)d * Dv) = S[i];
+    if (d < D && vok) *reinterpret_cast<f32x4*>(Sp + d * Dv) = S[i];
   }
   o = col_sum(o, 1);
   if (rg == 0 && vok) *reinterpret_cast<f32x4*>(out + (int64_t)q0 * os + (int64_t)h * Dv + c4) = o * fq;
