@@ -47,10 +47,11 @@ __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(
 constexpr int NA_MAXS = 8;   // split-K slabs of y1
 
 // One workgroup per row. VEC consecutive columns per thread and round, NV rounds in registers (d <= NT VEC NV): every
-// load of the row is in flight before the statistics, the sublayer's output and the residual stay in registers.
-template <typename AT, int VEC, int NV>
+// load of the row is in flight before the statistics, the sublayer's output and the residual stay in registers. S: slabs of
+// an fp32 y1, 0 = y1 in the activation dtype.
+template <typename AT, int VEC, int NV, int S>
 __global__ __launch_bounds__(NT) void norm_add_kernel(float* __restrict__ x, int64_t xs, const void* __restrict__ y1,
-                                                      int64_t y1s, int y1_f32, int S, int64_t slab,
+                                                      int64_t y1s, int64_t slab,
                                                       const AT* __restrict__ y2, int64_t y2s,
                                                       const float* __restrict__ w, float eps, AT* __restrict__ out,
                                                       int64_t os, int d) {
@@ -65,8 +66,9 @@ __global__ __launch_bounds__(NT) void norm_add_kernel(float* __restrict__ x, int
 #pragma unroll
     for (int e = 0; e < VEC; ++e) yv[it][e] = xv[it][e] = 0.f;
     if (i < d) {
-      if (y1_f32) {
+      if constexpr (S > 0) {
         const float* p = reinterpret_cast<const float*>(y1) + t * y1s + i;
+#pragma unroll
         for (int s = 0; s < S; ++s) {
 #pragma unroll
           for (int e = 0; e < VEC; ++e) yv[it][e] += p[s * slab + e];
@@ -971,17 +973,29 @@ hipError_t kafka_hy_norm_add(int f32, float* x, int64_t xs, const void* y1, int6
   auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
   const bool v4 = d % 4 == 0 && xs % 4 == 0 && y1s % 4 == 0 && slab % 4 == 0 && y2s % 4 == 0 && os % 4 == 0 && al(x) &&
                   al(y1) && al(y2) && al(w) && al(out);
+#define NA_LAUNCH(VEC, NV, SL) \
+  norm_add_kernel<AT, VEC, NV, SL><<<(unsigned)T, NT, 0, st>>>(x, xs, y1, y1s, slab, (const AT*)y2, y2s, w, eps, (AT*)out, os, d)
+#define NA_S(VEC, NV)                         \
+  do {                                        \
+    if (!y1_f32) NA_LAUNCH(VEC, NV, 0);       \
+    else if (S == 1) NA_LAUNCH(VEC, NV, 1);   \
+    else if (S == 2) NA_LAUNCH(VEC, NV, 2);   \
+    else if (S == 4) NA_LAUNCH(VEC, NV, 4);   \
+    else NA_LAUNCH(VEC, NV, 8);               \
+  } while (0)
+  const bool s8 = !y1_f32 || S == 1 || S == 2 || S == 4 || S == 8;
   DISPATCH_AT(f32, {
-    auto a = [&](auto k) {
-      k<<<(unsigned)T, NT, 0, st>>>(x, xs, y1, y1s, y1_f32, S, slab, (const AT*)y2, y2s, w, eps, (AT*)out, os, d);
-    };
-    if (v4 && d <= NT * 4) a(norm_add_kernel<AT, 4, 1>);
-    else if (v4 && d <= NT * 8) a(norm_add_kernel<AT, 4, 2>);
-    else if (v4 && d <= NT * 16) a(norm_add_kernel<AT, 4, 4>);
-    else if (v4 && d <= NT * 32) a(norm_add_kernel<AT, 4, 8>);
-    else if (d <= NT * 4) a(norm_add_kernel<AT, 1, 4>);
-    else a(norm_add_wide_kernel<AT>);
+    if (v4 && s8 && d <= NT * 4) NA_S(4, 1);
+    else if (v4 && s8 && d <= NT * 8) NA_S(4, 2);
+    else if (v4 && s8 && d <= NT * 16) NA_S(4, 4);
+    else if (v4 && s8 && d <= NT * 32) NA_S(4, 8);
+    else if (s8 && d <= NT * 4) NA_S(1, 4);
+    else
+      norm_add_wide_kernel<AT><<<(unsigned)T, NT, 0, st>>>(x, xs, y1, y1s, y1_f32, S, slab, (const AT*)y2, y2s, w, eps,
+                                                           (AT*)out, os, d);
   });
+#undef NA_S
+#undef NA_LAUNCH
   return hipGetLastError();
 }
 

@@ -498,6 +498,67 @@ __global__ __launch_bounds__(NT) void rope_kv_store_kernel(
   }
 }
 
+// The same for bf16 rows whose values are the key columns, without a head mix: L = D / 8 lanes per (row, query or key
+// head), a lane holds 8 consecutive elements in registers; the rotation's partner is dims / 16 lanes away. Everything in
+// 16-byte pieces (the page-wise transposed values element by element). D = 8 L with L a power of two, dims % 16 == 0.
+template <int L>
+__global__ __launch_bounds__(NT) void rope_kv_store_vec8_kernel(
+    const bf16* __restrict__ qkv, int64_t qs, int H, int G, const int64_t* __restrict__ positions,
+    const float* __restrict__ cos_sin, int dims, const float* __restrict__ qn, const float* __restrict__ kn, float eps,
+    bf16* __restrict__ kc, bf16* __restrict__ vt, const int64_t* __restrict__ slots, bf16* __restrict__ q_out,
+    int64_t qos, int64_t T) {
+  constexpr int D = 8 * L;
+  const int64_t u = (int64_t)blockIdx.x * (NT / L) + threadIdx.x / L;
+  if (u >= T * (H + G)) return;   // (whole groups of L lanes leave)
+  const int64_t t = u / (H + G);
+  const int hd = (int)(u - t * (H + G)), l = threadIdx.x % L;
+  const bf16x8 raw = load_bf16x8(qkv + t * qs + (int64_t)hd * D + 8 * l);
+  float x[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) x[j] = (float)raw[j];
+  if (qn != nullptr) {
+    const float* nw = (hd < H ? qn : kn) + 8 * l;
+    float s = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) s += x[j] * x[j];
+#pragma unroll
+    for (int o = L / 2; o > 0; o >>= 1) s += __shfl_xor(s, o, L);
+    const float rs = 1.0f / sqrtf(s / (float)D + eps);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) x[j] = x[j] * rs * nw[j];
+  }
+  if (dims > 0) {   // (uniform)
+    const int hl = dims >> 4;   // lanes of a half
+    const bool lo = l < hl, in = l < 2 * hl;
+    const int pl = lo ? l + hl : in ? l - hl : l;
+    const float* cs = cos_sin + positions[t] * dims + 8 * (in ? (lo ? l : l - hl) : 0);
+    float y[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) y[j] = __shfl(x[j], pl, L);
+    if (in) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        const float c = cs[j], sn = cs[(dims >> 1) + j];
+        x[j] = lo ? x[j] * c - y[j] * sn : x[j] * c + y[j] * sn;
+      }
+    }
+  }
+  bf16x8 r;
+#pragma unroll
+  for (int j = 0; j < 8; ++j) r[j] = (bf16)x[j];
+  if (hd < H) {
+    store_bf16x8(q_out + t * qos + (int64_t)hd * D + 8 * l, r);
+    return;
+  }
+  const int64_t slot = slots[t];
+  if (slot < 0) return;
+  const int c0 = (hd - H) * D + 8 * l;
+  store_bf16x8(kc + slot * ((int64_t)G * D) + c0, r);
+  bf16* vd = vt + ((slot / PAGE) * ((int64_t)G * D) + c0) * PAGE + (slot % PAGE);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) vd[(int64_t)j * PAGE] = raw[j];
+}
+
 }  // namespace hp
 }  // namespace kafka
 
@@ -618,6 +679,28 @@ hipError_t kafka_hy_rope_kv_store(int f32, const void* qkv, int64_t qs, int H, i
   if (dims < 0 || dims % 2 || dims > D || (dims > 0 && cos_sin == nullptr) || G < 1 || H % G ||
       (qn != nullptr) != (kn != nullptr))
     return hipErrorInvalidValue;
+  {
+    auto al = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+    const int L = D / 8;
+    if (!f32 && talk == nullptr && !pairs && v_off == H * D && Dv == D && D % 8 == 0 && L <= 64 && (L & (L - 1)) == 0 &&
+        dims % 16 == 0 && qs % 8 == 0 && qos % 8 == 0 && al(qkv) && al(q_out) && al(kc)) {
+      const unsigned grid = (unsigned)((T * (H + G) * L + NT - 1) / NT);
+      auto a = [&](auto k) {
+        k<<<grid, NT, 0, st>>>((const bf16*)qkv, qs, H, G, positions, cos_sin, dims, qn, kn, eps, (bf16*)kc, (bf16*)vt,
+                               slots, (bf16*)q_out, qos, T);
+      };
+      switch (L) {
+        case 1: a(rope_kv_store_vec8_kernel<1>); break;
+        case 2: a(rope_kv_store_vec8_kernel<2>); break;
+        case 4: a(rope_kv_store_vec8_kernel<4>); break;
+        case 8: a(rope_kv_store_vec8_kernel<8>); break;
+        case 16: a(rope_kv_store_vec8_kernel<16>); break;
+        case 32: a(rope_kv_store_vec8_kernel<32>); break;
+        default: a(rope_kv_store_vec8_kernel<64>); break;
+      }
+      return hipGetLastError();
+    }
+  }
   const int64_t fl = (int64_t)(H + G) * D + dims + (talk != nullptr ? H * H : 0);
   if (fl > kafka_hy_rope_store_max_q()) return hipErrorInvalidValue;
   const size_t lds = (size_t)fl * sizeof(float);

@@ -510,7 +510,8 @@ def qk_norm_rope_store(qkv, H: int, G: int, D: int, Dv: int, q_w, k_w, eps, posi
                                lam, k_cache, v_cache_t, slot_mapping, q_out)
 
 
-SHARED_SPLIT_WGS = 1024   # workgroups a shared-keys attention launch is split towards
+WINDOW_SPLIT_WGS = 512    # workgroups a windowed-attention launch is split towards (two per CU) ...
+SHARED_SPLIT_WGS = 1024   # ... and one with shared keys
 
 
 def window_attn_mfma_ok(q, k_cache, v_cache_t, H: int, G: int, shared_keys: bool = False) -> bool:
@@ -546,7 +547,7 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
             if window and max_keys:  # a tile's key range is at most the window and its own tokens long
                 max_keys = min(max_keys, window + tt)
             # (shared keys: few key/value heads, every workgroup walks the whole key row - more, shorter ranges)
-            ns = sig_splits(tiles.shape[0] * G, max_keys, SHARED_SPLIT_WGS if shared_keys else ATTN_SPLIT_WGS) \
+            ns = sig_splits(tiles.shape[0] * G, max_keys, SHARED_SPLIT_WGS if shared_keys else WINDOW_SPLIT_WGS) \
                 if max_keys else 1
             po = pml = None
             if ns > 1:

@@ -484,6 +484,39 @@ def test_attention_on_raw_keys_single_keys(device, H, G, D, rot, factor):
 
 
 @pytest.mark.gpu
+@pytest.mark.parametrize("H,G,D,rot", [(4, 2, 128, 128), (3, 1, 64, 32), (5, 5, 16, 16), (2, 1, 8, 0), (6, 3, 256, 96),
+                                       (2, 2, 48, 48)])
+def test_attention_inputs_bf16(H, G, D, rot):
+    """Norm, rotation and paged store of bf16 rows (registers where the head size is a power of two, LDS otherwise)
+    against the plain functions, inside wider rows, at positions far from zero."""
+    dev = "cuda:0"
+    g = torch.Generator().manual_seed(D + rot)
+    n, eps = 37, 1e-3
+    rows = torch.randn(n, (H + G) * D + 24, generator=g).to(torch.bfloat16)
+    qn, kn = 1.0 + 0.2 * torch.randn(D, generator=g), 1.0 + 0.2 * torch.randn(D, generator=g)
+    pg = Paged(dev, [500])
+    _, _, pos, sl = pg.step([(0, 401, n)])
+    kc = torch.zeros(pg.n_pages, 16, G * D, dtype=torch.bfloat16, device=dev)
+    vt = torch.zeros(pg.n_pages, G * D, 16, dtype=torch.bfloat16, device=dev)
+    cs = rotary_table(512, {"dims": rot, "base": 33.0, "scaling": {"factor": 2.0}}, dev) if rot else None
+    q = torch.empty(n, H * D, dtype=torch.bfloat16, device=dev)
+    hops.rope_kv_store(rows.to(dev), H, G, D, D, pos, cs, rot, False, None, kc, vt, sl, q, qn.to(dev), kn.to(dev), eps,
+                       v_off=H * D)
+    r = rows.double()
+    wq = plain.rms_norm(r[:, :H * D].view(n, H, D), qn.double(), eps)
+    wk = plain.rms_norm(r[:, H * D:(H + G) * D].view(n, G, D), kn.double(), eps)
+    if rot:
+        pad = torch.zeros(401, 1, 1, dtype=torch.float64)
+        wq = plain.rotate_halves(torch.cat([pad.expand(401, H, D), wq]), rot, 33.0, 2.0)[401:]
+        wk = plain.rotate_halves(torch.cat([pad.expand(401, G, D), wk]), rot, 33.0, 2.0)[401:]
+    assert close(q.float(), wq.reshape(n, -1), 1e-2)
+    assert close(kc.view(-1, G * D)[sl].float(), wk.reshape(n, -1), 1e-2)
+    v = vt.permute(0, 2, 1).reshape(-1, G * D)[sl].cpu()
+    assert torch.equal(v, rows[:, H * D:(H + G) * D])
+    assert kc.count_nonzero() == kc.view(-1, G * D)[sl].count_nonzero()      # nothing outside the rows' slots
+
+
+@pytest.mark.gpu
 @pytest.mark.parametrize("H,G,D,n", [(8, 2, 32, 300), (4, 4, 64, 700), (32, 1, 48, 200), (16, 2, 128, 1500),
                                      (2, 1, 256, 520)])
 def test_attention_on_raw_keys_matrix_cores(H, G, D, n):
