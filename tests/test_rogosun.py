@@ -360,6 +360,7 @@ def test_lin_scan_in_chunks(delta, n):
     """The chunked form against the token-by-token kernel and the plain function: every kind of last chunk, a segment
     that continues from a state, the state it leaves."""
     dev = "cuda:0"
+    assert hops.ext().hy_lin_chunk() == hops.LIN_CHUNK
     H, G, D, Dv, tau = 3, 3, 40, 50, 4.0
     g = torch.Generator().manual_seed(n)
     zb = torch.randn(H * D, generator=g)
