@@ -256,6 +256,40 @@ ROGOSUN_PRESETS: dict[str, dict] = {
 }
 
 
+def _furapel(width: int, heads: int, kv_heads: int, n_layers: int, vocab: int, ff: int, experts: int = 16, top: int = 4,
+             window: int = 1024, head_dim: int = 128) -> dict:
+    """A Furapel config dict at transformer-like sizes: layers cycle attention, mlstm (``width / 256`` heads of 128 x 256),
+    attention, latent attention (rank 512, sliding window); every layer with ``experts`` routed experts of ``ff`` rows,
+    ``top`` per token; the middle half of the depth runs twice."""
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    layers = []
+    for i in range(n_layers):
+        kind = i % 4
+        if kind in (0, 2):
+            m = {"heads": heads, "kv_heads": kv_heads, "dim": head_dim, "vdim": head_dim, "scale": head_dim ** -0.5,
+                 "rot": {"base": 500000.0, "dims": head_dim // 2,
+                         "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}
+            layers.append({"type": "attention", "mixer": m, "mlp": moe})
+        elif kind == 1:
+            layers.append({"type": "mlstm", "mixer": {"heads": max(1, width // 256), "dim": 128, "vdim": 256,
+                                                      "gate_cap": 15.0}, "mlp": moe})
+        else:
+            layers.append({"type": "latent_attention", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "kv_rank": 512,
+                                                                 "scale": 128 ** -0.5, "mask": {"size": window}},
+                           "mlp": moe})
+    q = n_layers // 4
+    return {"architecture": "Furapel", "vocab": vocab, "width": width, "layers": layers, "norm": {"eps": 1e-6},
+            "embedding": {"scale": float(width) ** 0.5}, "logit_scale": 0.25,
+            "loop": {"start": q, "stop": n_layers - max(1, q), "times": 2}}
+
+
+FURAPEL_PRESETS: dict[str, dict] = {
+    # widths, heads and vocabularies of the Llama presets above (random init)
+    "furapel-small": _furapel(1024, 8, 2, 8, 128256, 512),
+    "furapel-tiny": _furapel(512, 8, 1, 4, 32000, 256, experts=6, top=3, window=80, head_dim=64),
+}
+
+
 def _budurax_config(c: dict, name: str):
     from kafka_llm_service_amd.models.budurax import BuduraxConfig
 
@@ -286,17 +320,23 @@ def _rogosun_config(c: dict, name: str):
     return RogosunConfig.from_dict(c, name=name)
 
 
+def _furapel_config(c: dict, name: str):
+    from kafka_llm_service_amd.models.furapel import FurapelConfig
+
+    return FurapelConfig.from_dict(c, name=name)
+
+
 # config.json "architecture" (lower case) -> config class of a model family that names itself there
 ARCH_CONFIGS = {"budurax": _budurax_config, "lisorax": _lisorax_config, "mozidra": _mozidra_config,
-                "magedra": _magedra_config, "rogosun": _rogosun_config}
+                "magedra": _magedra_config, "rogosun": _rogosun_config, "furapel": _furapel_config}
 # model families whose kernels are built for float32 as well as bfloat16 (EngineConfig.dtype)
-FP32_ARCHS = ("budurax", "lisorax", "mozidra", "magedra", "rogosun")
+FP32_ARCHS = ("budurax", "lisorax", "mozidra", "magedra", "rogosun", "furapel")
 
 
 def _from_json(path: Path):
     """A config.json names its model class: ``"architecture": "Budurax"`` (models/budurax.py), ``"Lisorax"``
     (models/lisorax.py), ``"Mozidra"`` (models/mozidra.py), ``"Magedra"`` (models/magedra.py), ``"Rogosun"``
-    (models/rogosun.py), else HF Llama / Mixtral."""
+    (models/rogosun.py), ``"Furapel"`` (models/furapel.py), else HF Llama / Mixtral."""
     c = json.loads(path.read_text())
     make = ARCH_CONFIGS.get(str(c.get("architecture", "")).lower())
     if make is not None:
@@ -317,9 +357,11 @@ def get_config(name: str):
         return _magedra_config(MAGEDRA_PRESETS[name], name)
     if name in ROGOSUN_PRESETS:
         return _rogosun_config(ROGOSUN_PRESETS[name], name)
+    if name in FURAPEL_PRESETS:
+        return _furapel_config(FURAPEL_PRESETS[name], name)
     p = Path(name)
     if p.is_dir() and (p / "config.json").exists():
         return _from_json(p / "config.json")
     if p.suffix == ".json" and p.exists():
         return _from_json(p)
-    raise KeyError(f"unknown model {name!r}; presets: {sorted(PRESETS) + sorted(BUDURAX_PRESETS) + sorted(LISORAX_PRESETS) + sorted(MOZIDRA_PRESETS) + sorted(MAGEDRA_PRESETS) + sorted(ROGOSUN_PRESETS)}")
+    raise KeyError(f"unknown model {name!r}; presets: {sorted(PRESETS) + sorted(BUDURAX_PRESETS) + sorted(LISORAX_PRESETS) + sorted(MOZIDRA_PRESETS) + sorted(MAGEDRA_PRESETS) + sorted(ROGOSUN_PRESETS) + sorted(FURAPEL_PRESETS)}")

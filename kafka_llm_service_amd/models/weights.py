@@ -273,7 +273,7 @@ def build_model(cfg: ModelConfig, device, tp: int = 1, tp_rank: int = 0, seed: i
                 max_positions: int | None = None, dp_attention: tuple[int, int] | None = None, dtype=None):
     """``dp_attention = (ep, ep_rank)``: whole attention on this rank, experts sharded over the EP group.
     The model class follows ``cfg.arch`` (MODEL_CLASSES)."""
-    if cfg.arch in ("budurax", "lisorax", "mozidra", "magedra", "rogosun"):  # segment-planned families: own tensor names
+    if cfg.arch in ("budurax", "lisorax", "mozidra", "magedra", "rogosun", "furapel"):  # segment-planned: own tensor names
         if cfg.arch == "budurax":
             from kafka_llm_service_amd.models import budurax as fam
 
@@ -290,6 +290,10 @@ def build_model(cfg: ModelConfig, device, tp: int = 1, tp_rank: int = 0, seed: i
             from kafka_llm_service_amd.models import rogosun as fam
 
             cls = fam.RogosunLM
+        elif cfg.arch == "furapel":
+            from kafka_llm_service_amd.models import furapel as fam
+
+            cls = fam.FurapelLM
         else:
             from kafka_llm_service_amd.models import lisorax as fam
 

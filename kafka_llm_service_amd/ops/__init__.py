@@ -534,6 +534,17 @@ def grouped_stream_glu(x: torch.Tensor, wt: torch.Tensor, r: "MoERouting", e_lo:
     return y
 
 
+def grouped_stream_relu2(x: torch.Tensor, wt: torch.Tensor, r: "MoERouting", e_lo: int = 0) -> torch.Tensor:
+    """relu(x W_e^T)^2 for every routed (token, local expert) entry, rows in expert-sorted order [n_ent, F]: the
+    weight-streaming grouped kernel on plainly tiled expert weights (``tile_experts(w)``)."""
+    y = torch.empty(r.perm_tok.numel(), wt.shape[1] * 32, dtype=x.dtype, device=x.device)
+    if _gpu(x):
+        ext().wstream_grouped(x, wt, r.perm_tok, r.perm_w, r.expert_off, int(e_lo), int(x.shape[0]), True, y, None,
+                              GROUPED_PIN, relu2=True)
+        return y
+    return y.copy_(ref_grouped(x, untile_experts(wt), r, e_lo, gather=True).float().relu().square())
+
+
 def grouped_stream_combine(a: torch.Tensor, wt: torch.Tensor, r: "MoERouting", T: int, out: torch.Tensor,
                            e_lo: int = 0) -> torch.Tensor:
     """out[token] += w * (a[entry] @ W_e^T) over the local experts' entries (out f32 [T, N], zeroed by the caller)."""
@@ -623,11 +634,13 @@ def moe_sort(topk_w: torch.Tensor, topk_e: torch.Tensor, num_experts: int) -> Mo
 
 
 def grouped_gemm(x: torch.Tensor, w: torch.Tensor, r: MoERouting, gather: bool, e_lo: int = 0,
-                 y: torch.Tensor | None = None, combine_out: torch.Tensor | None = None) -> torch.Tensor:
+                 y: torch.Tensor | None = None, combine_out: torch.Tensor | None = None,
+                 relu2: bool = False) -> torch.Tensor:
     """Per expert segment of the routed entries: Y = X_e . W_e^T (W = [E_local, N, K], experts [e_lo, e_lo+E_local)).
 
     gather=True reads A rows as x[perm_tok[r]] (token activations), else x[r] (expert-sorted rows).
-    combine_out (f32 [T, N], zeroed by the caller) receives out[perm_tok[r]] += perm_w[r] * Y[r] instead of Y."""
+    combine_out (f32 [T, N], zeroed by the caller) receives out[perm_tok[r]] += perm_w[r] * Y[r] instead of Y.
+    relu2: Y's elements go through relu and are squared."""
     n_ent = r.perm_tok.numel()
     if combine_out is not None and combine_out.shape[0] != r.topk_w.shape[0]:
         raise ValueError("combine_out must have one row per routed token")
@@ -635,9 +648,11 @@ def grouped_gemm(x: torch.Tensor, w: torch.Tensor, r: MoERouting, gather: bool, 
         y = torch.empty(n_ent, w.shape[1], dtype=x.dtype, device=x.device)
     if _gpu(x):
         ext().grouped_gemm(x, w, r.perm_tok, r.perm_w, r.expert_off, r.tile_off, int(e_lo), int(r.max_tiles),
-                           bool(gather), y, combine_out)
+                           bool(gather), y, combine_out, bool(relu2))
     else:
         ref.grouped_gemm(x, w, r.perm_tok, r.perm_w, r.expert_off, e_lo, gather, y, combine_out)
+        if relu2:
+            y.copy_(y.float().relu().square())
     return combine_out if combine_out is not None else y
 
 

@@ -78,14 +78,14 @@ hipError_t kafka_launch_wstream_fin(int fin, const bf16* X, int64_t ldx, const b
 hipError_t kafka_launch_wstream_grouped(const bf16* X, int64_t ldx, const bf16* Wt, int e_local, int N, int K,
                                         const int* perm_tok, const float* perm_w, const int* expert_off, int e_lo,
                                         int max_rows, int gather, bf16* Y, int64_t ldy, float* out, int64_t ldo,
-                                        int pin, float glu_limit, float glu_alpha, hipStream_t st);
+                                        int pin, int relu2, float glu_limit, float glu_alpha, hipStream_t st);
 hipError_t kafka_launch_moe_route(const bf16* logits, int64_t ld, int T, int E, int K, int BM, float* topk_w,
                                   int* topk_e, int* perm_tok, float* perm_w, int* expert_off, int* tile_off,
                                   hipStream_t st);
 hipError_t kafka_launch_grouped_gemm(const bf16* X, int64_t ldx, const bf16* W, int N, int Kd, const int* perm_tok,
                                      const float* perm_w, const int* expert_off, const int* tile_off, int e_lo,
                                      int e_n, int max_tiles, int gather, bf16* Y, int64_t ldy, float* out,
-                                     int64_t ldo, hipStream_t st);
+                                     int64_t ldo, int relu2, hipStream_t st);
 hipError_t kafka_car_alloc(int64_t bytes, void** out);
 int64_t kafka_car_header_bytes();
 hipError_t kafka_car_timing(const void* own, uint64_t* ring_out, int* epoch_out);
@@ -698,11 +698,11 @@ static void wstream_gemm_cfg(at::Tensor x, at::Tensor wt, c10::optional<at::Tens
 }
 
 // Expert MLP halves on wave-tiled expert weights wt [E_local, N/32, K/16, 64, 8] (ops.tile_experts). glu: gate_up
-// with fused SwiGLU into y [n_ent, N/2]; else down with the weighted combine into out f32 [T, N]. max_rows = T
-// bounds every expert segment (a token picks an expert at most once).
+// with fused SwiGLU into y [n_ent, N/2] (relu2: an up projection alone, its relu squared into y [n_ent, N]); else down
+// with the weighted combine into out f32 [T, N]. max_rows = T bounds every expert segment (a token picks an expert at most once).
 static void wstream_grouped(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at::Tensor perm_w, at::Tensor expert_off,
                             int64_t e_lo, int64_t max_rows, bool gather, c10::optional<at::Tensor> y,
-                            c10::optional<at::Tensor> out, bool pin, double glu_limit, double glu_alpha) {
+                            c10::optional<at::Tensor> out, bool pin, double glu_limit, double glu_alpha, bool relu2) {
   CHECK_CUDA(x); CHECK_DT(x, at::kBFloat16); CHECK_DT(wt, at::kBFloat16); CHECK_LASTDIM(x);
   CHECK_DT(perm_tok, at::kInt); CHECK_DT(perm_w, at::kFloat); CHECK_DT(expert_off, at::kInt);
   TORCH_CHECK(x.dim() == 2 && x.stride(0) % 8 == 0, "wstream_grouped: x must be [rows, K] with 16-B rows");
@@ -722,12 +722,12 @@ static void wstream_grouped(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at
   int64_t ldo = 0;
   if (y.has_value()) {
     CHECK_DT(y.value(), at::kBFloat16); CHECK_LASTDIM(y.value());
-    TORCH_CHECK(!out.has_value() && y->dim() == 2 && y->size(0) >= n_ent && y->size(1) == N / 2,
-                "wstream_grouped: y must be [n_ent, N/2]");
+    TORCH_CHECK(!out.has_value() && y->dim() == 2 && y->size(0) >= n_ent && y->size(1) == (relu2 ? N : N / 2),
+                "wstream_grouped: y must be [n_ent, N/2], or [n_ent, N] with relu2");
     yp = bptr(y.value());
     ldy = y->stride(0);
   } else {
-    TORCH_CHECK(out.has_value(), "wstream_grouped: y or out required");
+    TORCH_CHECK(out.has_value() && !relu2, "wstream_grouped: y or out required, an activation with y");
     CHECK_DT(out.value(), at::kFloat); CHECK_LASTDIM(out.value());
     TORCH_CHECK(out->dim() == 2 && out->size(0) == max_rows && out->size(1) == N, "wstream_grouped: out [T, N]");
     op = out->data_ptr<float>();
@@ -736,7 +736,7 @@ static void wstream_grouped(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at
   CHECK_HIP(kafka_launch_wstream_grouped(bptr(x), x.stride(0), bptr(wt), E_local, N, K, perm_tok.data_ptr<int>(),
                                          perm_w.data_ptr<float>(), expert_off.data_ptr<int>(), (int)e_lo,
                                          (int)max_rows, gather ? 1 : 0, yp, ldy, op, ldo, pin ? 1 : 0,
-                                         (float)glu_limit, (float)glu_alpha, cur_stream()));
+                                         relu2 ? 1 : 0, (float)glu_limit, (float)glu_alpha, cur_stream()));
 }
 
 // y [M, N] bf16 = sum over the slabs p [S, M, N]
@@ -788,8 +788,9 @@ static void moe_sort(at::Tensor topk_w, at::Tensor topk_e, int64_t E, int64_t bm
 // Y (or out += w * Y) = X_e . W_e^T per expert segment of the routed entries; W = [e_n, N, K] local experts
 static void grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor perm_tok, at::Tensor perm_w, at::Tensor expert_off,
                          at::Tensor tile_off, int64_t e_lo, int64_t max_tiles, bool gather,
-                         c10::optional<at::Tensor> y, c10::optional<at::Tensor> out) {
+                         c10::optional<at::Tensor> y, c10::optional<at::Tensor> out, bool relu2) {
   CHECK_CUDA(x); CHECK_DT(x, at::kBFloat16); CHECK_DT(w, at::kBFloat16); CHECK_LASTDIM(x);
+  TORCH_CHECK(!relu2 || !out.has_value(), "grouped_gemm: an activation goes with y, not with the combine");
   TORCH_CHECK(w.dim() == 3 && w.is_contiguous(), "grouped_gemm: w must be contiguous [E_local, N, K]");
   const int e_n = w.size(0), N = w.size(1), Kd = w.size(2);
   const int E = expert_off.numel() - 1;
@@ -819,7 +820,7 @@ static void grouped_gemm(at::Tensor x, at::Tensor w, at::Tensor perm_tok, at::Te
   CHECK_HIP(kafka_launch_grouped_gemm(bptr(x), x.stride(0), bptr(w), N, Kd, perm_tok.data_ptr<int>(),
                                       perm_w.data_ptr<float>(), expert_off.data_ptr<int>(), tile_off.data_ptr<int>(),
                                       (int)e_lo, e_n, (int)max_tiles, gather ? 1 : 0, yp, ldy, op, ldo,
-                                      cur_stream()));
+                                      relu2 ? 1 : 0, cur_stream()));
 }
 
 // ---- CU-masked streams (attention partition: the compute-bound cascade tile and the bandwidth-bound suffix decode
@@ -1041,7 +1042,7 @@ PYBIND11_MODULE(_kafka_ops, m) {
   m.def("slab_reduce", &slab_reduce);
   m.def("wstream_grouped", &wstream_grouped, py::arg("x"), py::arg("wt"), py::arg("perm_tok"), py::arg("perm_w"),
         py::arg("expert_off"), py::arg("e_lo"), py::arg("max_rows"), py::arg("gather"), py::arg("y"), py::arg("out"),
-        py::arg("pin") = true, py::arg("glu_limit") = 0.0, py::arg("glu_alpha") = 1.0);
+        py::arg("pin") = true, py::arg("glu_limit") = 0.0, py::arg("glu_alpha") = 1.0, py::arg("relu2") = false);
   m.def("moe_sort", &moe_sort);
   m.def("moe_route", &moe_route);
   m.def("cu_mask_stream", &cu_mask_stream);
@@ -1062,5 +1063,7 @@ PYBIND11_MODULE(_kafka_ops, m) {
   m.def("ep_dispatch", &ep_dispatch);
   m.def("ep_recv_route", &ep_recv_route);
   m.def("ep_combine", &ep_combine);
-  m.def("grouped_gemm", &grouped_gemm);
+  m.def("grouped_gemm", &grouped_gemm, py::arg("x"), py::arg("w"), py::arg("perm_tok"), py::arg("perm_w"),
+        py::arg("expert_off"), py::arg("tile_off"), py::arg("e_lo"), py::arg("max_tiles"), py::arg("gather"),
+        py::arg("y"), py::arg("out"), py::arg("relu2") = false);
 }

@@ -88,7 +88,7 @@ hipError_t kafka_hy_moe_topk(const float* logits, int64_t ls, int E, int k, floa
 int kafka_hy_moe_rows_max_d();
 hipError_t kafka_hy_moe_rows(int f32, const void* h, int64_t hs, const void* wgu, const void* wd, const float* tw,
                              const int* te, int d, int F, int k, void* a, float* out, int64_t os, int64_t T,
-                             float limit, float alpha, hipStream_t st);
+                             int glu, float limit, float alpha, hipStream_t st);
 hipError_t kafka_hy_add2(int f32, float* x, int64_t xs, const void* y1, int64_t s1, const void* y2, int64_t s2,
                          int y2_f32, int64_t T, int d, const void* w, float eps, void* out, int64_t os, hipStream_t st);
 
@@ -110,12 +110,12 @@ int kafka_hy_window_attn_max_d();
 int kafka_hy_window_attn_max_dv();
 hipError_t kafka_hy_window_attn(int f32, const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                 int bt_stride, const int* tok_seg, const int64_t* positions, int H, int G, int D,
-                                int Dv, float scale, int window, const float* sink, void* out, int64_t os, int64_t T,
+                                int Dv, float scale, int window, const float* sink, const void* gate, int64_t gs, void* out, int64_t os, int64_t T,
                                 int shared_keys, float out_scale, hipStream_t st);
 int kafka_hy_window_attn_mfma_ok(int page, int D, int Dv, int rep);
 hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                      int bt_stride, const int* items, int n_items, const int64_t* positions, int H,
-                                     int G, int D, int Dv, float scale, int window, const float* sink, void* out,
+                                     int G, int D, int Dv, float scale, int window, const float* sink, const void* gate, int64_t gs, void* out,
                                      int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
                                      float out_scale, hipStream_t st);
 int kafka_hy_grouped_router_max_e();
@@ -163,6 +163,11 @@ hipError_t kafka_hy_lin_scan(int f32, const void* qk, int64_t qk_s, int q_off, i
                              const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
                              int64_t beta_s, int H, int G, int D, int Dv, float qscale, float inv_tau, const int* seg,
                              int R, int min_n, int max_n, float* S, float* out, int64_t os, hipStream_t st);
+int kafka_hy_add_tanh_norm_max_slabs();
+hipError_t kafka_hy_add_tanh_norm(int f32, float* x, int64_t xs, const void* y1, int64_t y1s, int y1_f32, int S,
+                                  int64_t slab, const float* y2, int64_t y2s, int assign, int n_norms,
+                                  const float* alpha, const float* const* w, const float* const* b, void* const* out,
+                                  const int64_t* os, void* copy, int64_t cs, int64_t T, int d, hipStream_t st);
 int64_t kafka_hy_lin_chunk_scratch(int D, int Dv, int delta);
 hipError_t kafka_hy_lin_chunked(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
                                 const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
@@ -719,15 +724,15 @@ void moe_topk(at::Tensor logits, at::Tensor tw, at::Tensor te) {
 }
 
 void moe_rows(at::Tensor h, at::Tensor wgu, at::Tensor wd, at::Tensor tw, at::Tensor te, at::Tensor a, at::Tensor out,
-              double limit, double alpha) {
+              double limit, double alpha, bool glu) {
   rows2d(h, "h"); rows2d(out, "out"); f32t(out, "out"); f32t(tw, "weights");
   const int f32 = act_f32(h);
   same_act(f32, {&wgu, &wd, &a});
   const int64_t T = h.size(0), d = h.size(1);
   TORCH_CHECK(wd.is_contiguous() && wd.dim() == 3 && wd.size(1) == d, "moe_rows: w_down [E, d, F]");
   const int64_t E = wd.size(0), F = wd.size(2);
-  TORCH_CHECK(wgu.is_contiguous() && wgu.dim() == 3 && wgu.size(0) == E && wgu.size(1) == 2 * F && wgu.size(2) == d,
-              "moe_rows: w_gu [E, 2 F, d]");
+  TORCH_CHECK(wgu.is_contiguous() && wgu.dim() == 3 && wgu.size(0) == E && wgu.size(1) == (glu ? 2 * F : F) &&
+                  wgu.size(2) == d, "moe_rows: w_gu [E, 2 F, d], or [E, F, d] without a gate");
   TORCH_CHECK(tw.is_contiguous() && tw.dim() == 2 && tw.size(0) == T && te.is_cuda() && te.is_contiguous() &&
                   te.scalar_type() == at::kInt && te.sizes() == tw.sizes(), "moe_rows: routing [T, k]");
   const int64_t k = tw.size(1);
@@ -738,7 +743,7 @@ void moe_rows(at::Tensor h, at::Tensor wgu, at::Tensor wd, at::Tensor tw, at::Te
   // expert ids index the weight stacks on the device: the router kernel writes ids in [0, E) only
   HY_HIP(kafka_hy_moe_rows(f32, h.data_ptr(), h.stride(0), wgu.data_ptr(), wd.data_ptr(), tw.data_ptr<float>(),
                            te.data_ptr<int>(), (int)d, (int)F, (int)k, a.data_ptr(), out.data_ptr<float>(),
-                           out.stride(0), T, (float)limit, (float)alpha, stream()));
+                           out.stride(0), T, glu ? 1 : 0, (float)limit, (float)alpha, stream()));
 }
 
 void add2(at::Tensor x, at::Tensor y1, OptT y2, OptT w, double eps, OptT out) {
@@ -868,9 +873,17 @@ void qk_norm_rope_store(at::Tensor qkv, int64_t H, int64_t G, int64_t D, int64_t
                                      slots.data_ptr<int64_t>(), q_out.data_ptr(), q_out.stride(0), T, stream()));
 }
 
+// the raw gates of a row's heads: columns [off, off + H) of ``gate``, in the activation dtype
+const void* head_gate_ptr(const OptT& gate, int64_t off, int f32, int64_t T, int64_t H) {
+  if (!gate.has_value()) return nullptr;
+  rows2d(*gate, "gate"); same_act(f32, {&*gate});
+  TORCH_CHECK(gate->size(0) == T && off >= 0 && off + H <= gate->size(1), "gate: columns [off, off + H) of every row");
+  return static_cast<const char*>(gate->data_ptr()) + off * gate->element_size();
+}
+
 void window_attn(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::Tensor tok_seg, at::Tensor positions,
                  int64_t H, int64_t G, double scale, int64_t window, OptT sink, at::Tensor out, bool shared_keys,
-                 double out_scale) {
+                 double out_scale, OptT gate, int64_t gate_off) {
   rows2d(q, "q"); rows2d(out, "out");
   const int f32 = act_f32(q);
   same_act(f32, {&kc, &vt, &out});
@@ -889,15 +902,17 @@ void window_attn(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::
                   positions.is_contiguous() && positions.numel() == T, "window_attn: block tables / tok_seg / positions");
   HY_HIP(kafka_hy_window_attn(f32, q.data_ptr(), q.stride(0), kc.data_ptr(), vt.data_ptr(), bt.data_ptr<int>(),
                               (int)bt.stride(0), tok_seg.data_ptr<int>(), positions.data_ptr<int64_t>(), (int)H, (int)G,
-                              (int)D, (int)Dv, (float)scale, (int)window, sink_ptr(sink, H), out.data_ptr(),
-                              out.stride(0), T, shared_keys ? 1 : 0, (float)out_scale, stream()));
+                              (int)D, (int)Dv, (float)scale, (int)window, sink_ptr(sink, H),
+                              head_gate_ptr(gate, gate_off, f32, T, H), gate.has_value() ? gate->stride(0) : 0,
+                              out.data_ptr(), out.stride(0), T, shared_keys ? 1 : 0, (float)out_scale, stream()));
 }
 
 // the matrix-core kernel: items int32 [n, 4] = (first row, tokens, segment, 0), each at most 32 (token, query head of
 // one key/value head) rows of one segment
 void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::Tensor items, int64_t tile_tokens,
                       at::Tensor positions, int64_t H, int64_t G, double scale, int64_t window, OptT sink,
-                      at::Tensor out, int64_t nsplit, OptT po, OptT pml, bool shared_keys, double out_scale) {
+                      at::Tensor out, int64_t nsplit, OptT po, OptT pml, bool shared_keys, double out_scale,
+                      OptT gate, int64_t gate_off) {
   for (const at::Tensor* t : {&q, &kc, &vt, &out})
     TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16, "window_attn_mfma: bf16 GPU tensors");
   rows2d(q, "q"); rows2d(out, "out");
@@ -929,8 +944,9 @@ void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt,
   HY_HIP(kafka_hy_window_attn_mfma(q.data_ptr(), q.stride(0), kc.data_ptr(), vt.data_ptr(), bt.data_ptr<int>(),
                                    (int)bt.stride(0), items.data_ptr<int>(), (int)items.size(0),
                                    positions.data_ptr<int64_t>(), (int)H, (int)G, (int)D, (int)Dv, (float)scale,
-                                   (int)window, sink_ptr(sink, H), out.data_ptr(), out.stride(0), (int)nsplit, pop,
-                                   pmlp, T, shared_keys ? 1 : 0, (float)out_scale, stream()));
+                                   (int)window, sink_ptr(sink, H), head_gate_ptr(gate, gate_off, 0, T, H),
+                                   gate.has_value() ? gate->stride(0) : 0, out.data_ptr(), out.stride(0), (int)nsplit,
+                                   pop, pmlp, T, shared_keys ? 1 : 0, (float)out_scale, stream()));
 }
 
 void moe_topk_grouped(at::Tensor logits, int64_t E, OptT corr, int64_t groups, int64_t keep, double eps,
@@ -1113,6 +1129,60 @@ void norm_add(at::Tensor x, at::Tensor y1, OptT y2, at::Tensor w, double eps, Op
                            w.data_ptr<float>(), (float)eps, op, os, T, (int)d, stream()));
 }
 
+// x (+)= y1 + y2, then up to two tanh norms of the new x and a copy of it in the activation dtype
+void add_tanh_norm(at::Tensor x, OptT y1, OptT y2, bool assign, std::vector<double> alpha, std::vector<at::Tensor> w,
+                   std::vector<at::Tensor> b, std::vector<at::Tensor> outs, OptT copy) {
+  rows2d(x, "x"); f32t(x, "x");
+  const int64_t T = x.size(0), d = x.size(1);
+  TORCH_CHECK(x.stride(0) >= d, "add_tanh_norm: rows of x must not overlap");
+  const size_t n = outs.size();
+  TORCH_CHECK(n <= 2 && alpha.size() == n && w.size() == n && b.size() == n, "add_tanh_norm: up to two norms");
+  TORCH_CHECK(y1.has_value() || (!assign && !y2.has_value()), "add_tanh_norm: y2 and assign need y1");
+  int f32 = -1;   // the activation dtype: that of the outputs, else of y1
+  float al[2]; const float *wp[2], *bp[2]; void* op[2]; int64_t os[2];
+  auto dest = [&](const at::Tensor& o) {
+    rows2d(o, "output");
+    if (f32 < 0) f32 = act_f32(o);
+    same_act(f32, {&o});
+    TORCH_CHECK(o.size(0) == T && o.size(1) == d && o.stride(0) >= d, "add_tanh_norm: output shape");
+  };
+  for (size_t k = 0; k < n; ++k) {
+    dest(outs[k]);
+    f32t(w[k], "w"); f32t(b[k], "b"); vec(w[k], d, "w"); vec(b[k], d, "b");
+    al[k] = (float)alpha[k]; wp[k] = w[k].data_ptr<float>(); bp[k] = b[k].data_ptr<float>();
+    op[k] = outs[k].data_ptr(); os[k] = outs[k].stride(0);
+  }
+  if (copy.has_value()) dest(*copy);
+  const void* p1 = nullptr; int64_t s1 = 0, slab = 0, S = 1; int y1f = 0;
+  if (y1.has_value()) {
+    TORCH_CHECK(y1->is_cuda(), "add_tanh_norm: y1 on the GPU");
+    y1f = act_f32(*y1);
+    if (y1->dim() == 3) {   // split-K slabs
+      TORCH_CHECK(y1f && y1->stride(2) == 1 && y1->size(1) == T && y1->size(2) == d && y1->size(0) >= 1 &&
+                      y1->size(0) <= kafka_hy_add_tanh_norm_max_slabs(), "add_tanh_norm: slabs fp32 [splits, T, d]");
+      S = y1->size(0); slab = y1->stride(0); s1 = y1->stride(1);
+    } else {
+      rows2d(*y1, "y1");
+      TORCH_CHECK(y1->size(0) == T && y1->size(1) == d, "add_tanh_norm: y1 shape");
+      s1 = y1->stride(0);
+    }
+    if (f32 < 0) f32 = y1f;
+    TORCH_CHECK(y1f || !f32, "add_tanh_norm: y1 is fp32 or of the activation dtype");
+    p1 = y1->data_ptr();
+  }
+  const float* p2 = nullptr; int64_t s2 = 0;
+  if (y2.has_value()) {
+    rows2d(*y2, "y2"); f32t(*y2, "y2");
+    TORCH_CHECK(y2->size(0) == T && y2->size(1) == d, "add_tanh_norm: y2 fp32 [T, d]");
+    p2 = y2->data_ptr<float>(); s2 = y2->stride(0);
+  }
+  if (f32 < 0) return;   // nothing to do
+  HY_HIP(kafka_hy_add_tanh_norm(f32, x.data_ptr<float>(), x.stride(0), p1, s1, y1f, (int)S, slab, p2, s2,
+                                assign ? 1 : 0, (int)n, al, wp, bp, op, os,
+                                copy.has_value() ? copy->data_ptr() : nullptr, copy.has_value() ? copy->stride(0) : 0,
+                                T, (int)d, stream()));
+}
+
 void ff_act(at::Tensor u, at::Tensor out, bool glu) {
   rows2d(u, "u"); rows2d(out, "out");
   const int f32 = act_f32(u);
@@ -1210,7 +1280,7 @@ void kafka_bind_hybrid(pybind11::module_& m) {
         py::arg("eps"), py::arg("out"), py::arg("scale") = 1.0, py::arg("silu") = false);
   m.def("hy_moe_topk", &moe_topk);
   m.def("hy_moe_rows", &moe_rows, py::arg("h"), py::arg("wgu"), py::arg("wd"), py::arg("tw"), py::arg("te"),
-        py::arg("a"), py::arg("out"), py::arg("limit") = 0.0, py::arg("alpha") = 1.0);
+        py::arg("a"), py::arg("out"), py::arg("limit") = 0.0, py::arg("alpha") = 1.0, py::arg("glu") = true);
   m.def("hy_add2", &add2, py::arg("x"), py::arg("y1"), py::arg("y2") = py::none(), py::arg("w") = py::none(),
         py::arg("eps") = 0.0, py::arg("out") = py::none());
   m.def("hy_stream_step", &stream_step, py::arg("xs"), py::arg("y") = py::none(), py::arg("mix") = py::none(),
@@ -1221,13 +1291,15 @@ void kafka_bind_hybrid(pybind11::module_& m) {
   m.def("hy_qk_norm_rope_store", &qk_norm_rope_store);
   m.def("hy_window_attn", &window_attn, py::arg("q"), py::arg("kc"), py::arg("vt"), py::arg("bt"), py::arg("tok_seg"),
         py::arg("positions"), py::arg("H"), py::arg("G"), py::arg("scale"), py::arg("window"), py::arg("sink"),
-        py::arg("out"), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0);
+        py::arg("out"), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0, py::arg("gate") = py::none(),
+        py::arg("gate_off") = 0);
   m.def("hy_window_attn_mfma_ok",
         [](int page, int D, int Dv, int rep) { return kafka_hy_window_attn_mfma_ok(page, D, Dv, rep) != 0; });
   m.def("hy_window_attn_mfma", &window_attn_mfma, py::arg("q"), py::arg("kc"), py::arg("vt"), py::arg("bt"),
         py::arg("items"), py::arg("tile_tokens"), py::arg("positions"), py::arg("H"), py::arg("G"), py::arg("scale"),
         py::arg("window"), py::arg("sink"), py::arg("out"), py::arg("nsplit") = 1, py::arg("po") = py::none(),
-        py::arg("pml") = py::none(), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0);
+        py::arg("pml") = py::none(), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0,
+        py::arg("gate") = py::none(), py::arg("gate_off") = 0);
   m.def("hy_moe_topk_grouped", &moe_topk_grouped);
   m.def("hy_act_norm", &act_norm);
   m.def("hy_gate_mul", &gate_mul);
@@ -1239,6 +1311,8 @@ void kafka_bind_hybrid(pybind11::module_& m) {
   m.def("hy_rope_kv_store", &rope_kv_store);
   m.def("hy_norm_add", &norm_add);
   m.def("hy_ff_act", &ff_act);
+  m.def("hy_add_tanh_norm", &add_tanh_norm, py::arg("x"), py::arg("y1"), py::arg("y2"), py::arg("assign"),
+        py::arg("alpha"), py::arg("w"), py::arg("b"), py::arg("outs"), py::arg("copy") = py::none());
   m.def("hy_lin_scan", &lin_scan);
   m.def("hy_lin_chunk", []() { return kafka_hy_lin_chunk(); });
   m.def("hy_sigmoid_attn_mfma_ok",

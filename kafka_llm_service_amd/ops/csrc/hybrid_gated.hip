@@ -730,7 +730,8 @@ __device__ __forceinline__ float glu_act(float g, float u, float limit, float al
   return g / (1.0f + expf(-g)) * u;
 }
 
-template <typename AT>
+// GLU false: a single up projection [E][F][d] and a[pair][f] = relu(W_up[e] h)^2
+template <typename AT, bool GLU>
 __global__ __launch_bounds__(NT) void moe_gate_up_kernel(const AT* __restrict__ h, int64_t hs,
                                                          const AT* __restrict__ wgu, const int* __restrict__ te, int d,
                                                          int F, int k, int FB, AT* __restrict__ a, float limit,
@@ -742,7 +743,7 @@ __global__ __launch_bounds__(NT) void moe_gate_up_kernel(const AT* __restrict__ 
   for (int i = threadIdx.x; i < d; i += NT) hsh[i] = ldf(h + t * hs + i);
   __syncthreads();
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const AT* wg = wgu + (int64_t)e * 2 * F * d;
+  const AT* wg = wgu + (int64_t)e * (GLU ? 2 : 1) * F * d;
   const int f1 = min(F, (int)(blockIdx.y + 1) * FB);
   for (int f = blockIdx.y * FB + wave; f < f1; f += NT / 64) {
     const AT* g = wg + (int64_t)f * d;
@@ -751,11 +752,16 @@ __global__ __launch_bounds__(NT) void moe_gate_up_kernel(const AT* __restrict__ 
     for (int i = lane; i < d; i += 64) {
       const float x = hsh[i];
       sg += x * ldf(g + i);
-      su += x * ldf(u + i);
+      if constexpr (GLU) su += x * ldf(u + i);
     }
     sg = wave_sum(sg);
-    su = wave_sum(su);
-    if (lane == 0) stf(a + pair * F + f, glu_act(sg, su, limit, alpha));
+    if constexpr (GLU) {
+      su = wave_sum(su);
+      if (lane == 0) stf(a + pair * F + f, glu_act(sg, su, limit, alpha));
+    } else {
+      sg = fmaxf(sg, 0.f);
+      if (lane == 0) stf(a + pair * F + f, sg * sg);
+    }
   }
 }
 
@@ -1014,7 +1020,7 @@ hipError_t kafka_hy_moe_topk(const float* logits, int64_t ls, int E, int k, floa
 int kafka_hy_moe_rows_max_d() { return MOE_MAXD; }
 
 hipError_t kafka_hy_moe_rows(int f32, const void* h, int64_t hs, const void* wgu, const void* wd, const float* tw,
-                             const int* te, int d, int F, int k, void* a, float* out, int64_t os, int64_t T,
+                             const int* te, int d, int F, int k, void* a, float* out, int64_t os, int64_t T, int glu,
                              float limit, float alpha, hipStream_t st) {
   if (T <= 0) return hipSuccess;
   if (d > MOE_MAXD || F > MOE_MAXD) return hipErrorInvalidValue;
@@ -1026,8 +1032,11 @@ hipError_t kafka_hy_moe_rows(int f32, const void* h, int64_t hs, const void* wgu
   while (T * ((d + cb - 1) / cb) < 1024 && cb > 8) cb = (cb + 1) / 2;
   const dim3 g1((unsigned)pairs, (F + fb - 1) / fb), g2((unsigned)T, (d + cb - 1) / cb);
   DISPATCH_AT(f32, {
-    moe_gate_up_kernel<AT><<<g1, NT, d * sizeof(float), st>>>((const AT*)h, hs, (const AT*)wgu, te, d, F, k, fb, (AT*)a,
-                                                              limit, alpha);
+    auto up = [&](auto kern) {
+      kern<<<g1, NT, d * sizeof(float), st>>>((const AT*)h, hs, (const AT*)wgu, te, d, F, k, fb, (AT*)a, limit, alpha);
+    };
+    if (glu) up(moe_gate_up_kernel<AT, true>);
+    else up(moe_gate_up_kernel<AT, false>);
     moe_down_kernel<AT><<<g2, NT, (size_t)F * sizeof(float), st>>>((const AT*)a, (const AT*)wd, tw, te, d, F, k, cb,
                                                                        out, os);
   });

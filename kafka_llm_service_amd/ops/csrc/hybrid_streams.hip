@@ -273,6 +273,10 @@ __global__ __launch_bounds__(NT) void qk_norm_rope_store_kernel(
 }
 
 // ---- windowed softmax attention with a sink -----------------------------------------------------------------------
+// sigmoid of a head's raw gate: a factor on the head's whole output
+template <typename T>
+__device__ __forceinline__ float head_gate(const T* p) { return 1.0f / (1.0f + expf(-ldf(p))); }
+
 constexpr int WA_MAXD = 1024;  // query / key size (the query row sits in LDS as fp32)
 constexpr int WA_NV = 8;      // value size up to 64 * WA_NV
 
@@ -283,8 +287,10 @@ __global__ __launch_bounds__(NT) void window_attn_kernel(const AT* __restrict__ 
                                                          const int* __restrict__ tok_seg,
                                                          const int64_t* __restrict__ positions, int H, int G, int D,
                                                          int Dv, int Ck, int kstep, float scale_log2e, int window,
-                                                         const float* __restrict__ sink, AT* __restrict__ out,
-                                                         int64_t os, int64_t pairs, float out_scale) {
+                                                         const float* __restrict__ sink,
+                                                         const AT* __restrict__ gate, int64_t gs,
+                                                         AT* __restrict__ out, int64_t os, int64_t pairs,
+                                                         float out_scale) {
   // D: size of a query row and of the key it meets; key/value head g's key starts at column g * kstep of a key row of
   // Ck columns (kstep = D: one key head per key/value head; kstep = 0, D = Ck: every query row meets the whole key row)
   __shared__ float qsh[NT / 64][WA_MAXD];
@@ -349,7 +355,8 @@ __global__ __launch_bounds__(NT) void window_attn_kernel(const AT* __restrict__ 
       }
     }
   }
-  const float inv = out_scale / l;
+  float inv = out_scale / l;
+  if (gate != nullptr) inv *= head_gate(gate + t * gs + h);
 #pragma unroll
   for (int i = 0; i < WA_NV; ++i) {
     const int v = lane + 64 * i;
@@ -380,7 +387,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
     const bf16* __restrict__ q, int64_t qs, const bf16* __restrict__ kc, const bf16* __restrict__ vt,
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ items, const int64_t* __restrict__ positions,
     int H, int G, int D, int Dv, int Ck, int kstep, float scale_log2e, int window, const float* __restrict__ sink,
-    bf16* __restrict__ out, int64_t os, float* __restrict__ po, float* __restrict__ pml, int64_t T, float out_scale) {
+    const bf16* __restrict__ gate, int64_t gs, bf16* __restrict__ out, int64_t os, float* __restrict__ po, float* __restrict__ pml, int64_t T, float out_scale) {
   // (D, Ck, kstep as in window_attn_kernel: kstep = 0 and D = Ck when every query row meets the whole key row)
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int nks = D >> 4, qstride = D + 8;
@@ -524,7 +531,8 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
     const int h = g * rep + r % rep;
     if (nsplit == 1) {
       if (sink != nullptr) l += fast_exp2(sink[h] * LOG2E - m[i]);
-      const float inv = out_scale / l;
+      float inv = out_scale / l;
+      if (gate != nullptr) inv *= head_gate(gate + t * gs + h);
 #pragma unroll
       for (int tw = 0; tw < TW; ++tw) {
         const int col = (w * TW + tw) * 32 + lr;
@@ -547,8 +555,8 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
 
 // out[t][h] = sum_z 2^(m_z - m) O_z / (sum_z 2^(m_z - m) l_z + 2^(sink_h - m)) over the key-range splits
 __global__ void window_merge_kernel(const float* __restrict__ po, const float* __restrict__ pml, int nsplit, int64_t T,
-                                    int H, int Dv, const float* __restrict__ sink, bf16* __restrict__ out, int64_t os,
-                                    float out_scale) {
+                                    int H, int Dv, const float* __restrict__ sink, const bf16* __restrict__ gate,
+                                    int64_t gs, bf16* __restrict__ out, int64_t os, float out_scale) {
   const int64_t th = blockIdx.x;  // t * H + h
   const int64_t t = th / H;
   const int h = (int)(th - t * H);
@@ -561,7 +569,8 @@ __global__ void window_merge_kernel(const float* __restrict__ po, const float* _
     if (mz != -INFINITY) den += fast_exp2(mz - mx) * pml[2 * (z * zs + th) + 1];
   }
   if (sink != nullptr) den += fast_exp2(sink[h] * LOG2E - mx);
-  const float inv = out_scale / den;
+  float inv = out_scale / den;
+  if (gate != nullptr) inv *= head_gate(gate + t * gs + h);
   for (int d = threadIdx.x; d < Dv; d += blockDim.x) {
     float a = 0.f;
     for (int z = 0; z < nsplit; ++z) {
@@ -798,8 +807,8 @@ int kafka_hy_window_attn_max_dv() { return 64 * WA_NV; }
 
 hipError_t kafka_hy_window_attn(int f32, const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                 int bt_stride, const int* tok_seg, const int64_t* positions, int H, int G, int D,
-                                int Dv, float scale, int window, const float* sink, void* out, int64_t os, int64_t T,
-                                int shared_keys, float out_scale, hipStream_t st) {
+                                int Dv, float scale, int window, const float* sink, const void* gate, int64_t gs,
+                                void* out, int64_t os, int64_t T, int shared_keys, float out_scale, hipStream_t st) {
   // shared_keys: D is the whole key row's size and every query row meets all G key heads of a token at once
   if (T <= 0) return hipSuccess;
   if (D > WA_MAXD || Dv > 64 * WA_NV || G < 1 || H % G || window < 0) return hipErrorInvalidValue;
@@ -809,7 +818,7 @@ hipError_t kafka_hy_window_attn(int f32, const void* q, int64_t qs, const void* 
   DISPATCH_AT(f32, {
     window_attn_kernel<AT><<<grid, NT, 0, st>>>((const AT*)q, qs, (const AT*)kc, (const AT*)vt, bt, bt_stride, tok_seg,
                                                 positions, H, G, D, Dv, Ck, kstep, scale * LOG2E, window, sink,
-                                                (AT*)out, os, pairs, out_scale);
+                                                (const AT*)gate, gs, (AT*)out, os, pairs, out_scale);
   });
   return hipGetLastError();
 }
@@ -821,8 +830,8 @@ int kafka_hy_window_attn_mfma_ok(int page, int D, int Dv, int rep) {
 
 hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                      int bt_stride, const int* items, int n_items, const int64_t* positions, int H,
-                                     int G, int D, int Dv, float scale, int window, const float* sink, void* out,
-                                     int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
+                                     int G, int D, int Dv, float scale, int window, const float* sink,
+                                     const void* gate, int64_t gs, void* out, int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
                                      float out_scale, hipStream_t st) {
   if (n_items <= 0) return hipSuccess;
   const int Ck = shared_keys ? D : G * D, kstep = shared_keys ? 0 : D;
@@ -832,8 +841,8 @@ hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, 
   const dim3 grid((unsigned)n_items, (unsigned)G, (unsigned)nsplit);
   auto a = [&](auto k) {
     k<<<grid, 256, lds, st>>>((const bf16*)q, qs, (const bf16*)kc, (const bf16*)vt, bt, bt_stride, items, positions, H,
-                              G, D, Dv, Ck, kstep, scale * LOG2E, window, sink, (bf16*)out, os, po, pml, T,
-                              out_scale);
+                              G, D, Dv, Ck, kstep, scale * LOG2E, window, sink, (const bf16*)gate, gs, (bf16*)out, os, po, pml,
+                              T, out_scale);
   };
   const int nks = D / 16, tw = ((Dv + 31) / 32 + 3) / 4;
   if (tw == 1 && nks <= 4) a(window_attn_mfma_kernel<1, 4>);
@@ -842,8 +851,8 @@ hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, 
   else if (nks <= 8) a(window_attn_mfma_kernel<2, 8>);
   else a(window_attn_mfma_kernel<2, 16>);
   if (nsplit > 1)
-    window_merge_kernel<<<(unsigned)(T * H), 64, 0, st>>>(po, pml, nsplit, T, H, Dv, sink, (bf16*)out, os,
-                                                             out_scale);
+    window_merge_kernel<<<(unsigned)(T * H), 64, 0, st>>>(po, pml, nsplit, T, H, Dv, sink, (const bf16*)gate, gs,
+                                                          (bf16*)out, os, out_scale);
   return hipGetLastError();
 }
 

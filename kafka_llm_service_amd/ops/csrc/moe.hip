@@ -17,7 +17,7 @@
 //   Expert parallelism: only experts [e_lo, e_lo + e_n) are resident (W = their weights). Modes:
 //     * gather:  A row r = X[perm_tok[r]]            (the first expert GEMM reads the un-permuted activations),
 //     * direct:  A row r = X[r]                       (the second GEMM reads the expert-sorted intermediate),
-//     * output:  bf16 Y[r, :] through an LDS transpose (16-B coalesced row stores), or
+//     * output:  bf16 Y[r, :], or with relu2 its relu squared, through an LDS transpose (16-B coalesced row stores), or
 //     * combine: out_f32[perm_tok[r], :] += perm_w[r] * Y[r, :] with float atomics — a token receives exactly k
 //                contributions onto a zeroed buffer, and for k = 2 IEEE addition makes the order irrelevant.
 //
@@ -145,7 +145,7 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(const bf16* __restric
                                                             const int* __restrict__ expert_off,
                                                             const int* __restrict__ tile_off, int e_lo, int e_n,
                                                             bf16* __restrict__ Y, int64_t ldy,
-                                                            float* __restrict__ out, int64_t ldo) {
+                                                            float* __restrict__ out, int64_t ldo, int relu2) {
   __shared__ __attribute__((aligned(16))) char lds[2 * GG_STAGE];
   // experts [e_lo, e_lo + e_n) are local (expert parallelism: W holds only those)
   const int tile = blockIdx.x + tile_off[e_lo];
@@ -242,7 +242,8 @@ __global__ __launch_bounds__(256) void grouped_gemm_kernel(const bf16* __restric
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       const int r = wr + (i & 3) + 8 * (i >> 2) + 4 * fh;
-      ct[r * GG_BN + wc + 32 * j + fr] = (bf16)acc[j][i];
+      const float v = acc[j][i], p = fmaxf(v, 0.f);
+      ct[r * GG_BN + wc + 32 * j + fr] = (bf16)(relu2 ? p * p : v);
     }
   __syncthreads();
 #pragma unroll
@@ -267,23 +268,23 @@ extern "C" hipError_t kafka_launch_grouped_gemm(const bf16* X, int64_t ldx, cons
                                                const int* perm_tok, const float* perm_w, const int* expert_off,
                                                const int* tile_off, int e_lo, int e_n, int max_tiles, int gather,
                                                bf16* Y,
-                                               int64_t ldy, float* out, int64_t ldo, hipStream_t st) {
-  if (N % GG_BN || Kd % GG_BK) return hipErrorInvalidValue;
+                                               int64_t ldy, float* out, int64_t ldo, int relu2, hipStream_t st) {
+  if (N % GG_BN || Kd % GG_BK || (out && relu2)) return hipErrorInvalidValue;
   dim3 grid(max_tiles, N / GG_BN);
   if (out) {
     if (gather)
       grouped_gemm_kernel<true, true><<<grid, 256, 0, st>>>(X, ldx, W, N, Kd, perm_tok, perm_w, expert_off,
-                                                            tile_off, e_lo, e_n, Y, ldy, out, ldo);
+                                                            tile_off, e_lo, e_n, Y, ldy, out, ldo, relu2);
     else
       grouped_gemm_kernel<false, true><<<grid, 256, 0, st>>>(X, ldx, W, N, Kd, perm_tok, perm_w, expert_off,
-                                                             tile_off, e_lo, e_n, Y, ldy, out, ldo);
+                                                             tile_off, e_lo, e_n, Y, ldy, out, ldo, relu2);
   } else {
     if (gather)
       grouped_gemm_kernel<true, false><<<grid, 256, 0, st>>>(X, ldx, W, N, Kd, perm_tok, perm_w, expert_off,
-                                                             tile_off, e_lo, e_n, Y, ldy, out, ldo);
+                                                             tile_off, e_lo, e_n, Y, ldy, out, ldo, relu2);
     else
       grouped_gemm_kernel<false, false><<<grid, 256, 0, st>>>(X, ldx, W, N, Kd, perm_tok, perm_w, expert_off,
-                                                              tile_off, e_lo, e_n, Y, ldy, out, ldo);
+                                                              tile_off, e_lo, e_n, Y, ldy, out, ldo, relu2);
   }
   return hipGetLastError();
 }

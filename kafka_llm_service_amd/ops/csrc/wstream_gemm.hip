@@ -663,6 +663,7 @@ __global__ __launch_bounds__(256 * KW) void wstream_gemm_kernel(const bf16* __re
 //   GATHER: A row = X[perm_tok[entry]] (token activations), else X[entry] (expert-sorted intermediate).
 //   Epilogue GLU (GLU-interleaved tiles): Y[entry, :N/2] = silu(gate) * up, bf16 — the SwiGLU of the expert MLP; with
 //   glu_limit > 0 the clamped form g' sigmoid(glu_alpha g') (u' + 1), g' = min(gate, limit), u' = clamp(up, +-limit).
+//   Epilogue relu2 (plain tiles): Y[entry, :N] = relu(y)^2, bf16.
 //   Epilogue COMBINE: out_f32[perm_tok[entry], n] += perm_w[entry] * y (a token gets exactly k contributions).
 // (MT = 4: at most 256 registers so two workgroups share a CU — left free the compiler took 316, one wave per SIMD:
 // the 128-row expert tiles streamed 8 % slower, Mixtral 128 threads 5,155 vs 5,234 tok/s, profiles/r06/mixtral/;
@@ -674,8 +675,8 @@ __global__ __launch_bounds__(256, MT == 4 ? 2 : 1) void wstream_grouped_kernel(c
                                                                const float* __restrict__ perm_w,
                                                                const int* __restrict__ expert_off, int e_lo,
                                                                bf16* __restrict__ Y, int64_t ldy,
-                                                               float* __restrict__ out, int64_t ldo, float glu_limit,
-                                                               float glu_alpha) {
+                                                               float* __restrict__ out, int64_t ldo, int relu2,
+                                                               float glu_limit, float glu_alpha) {
   constexpr int ROWS = 32 * MT;
   constexpr int CPR = KC / 8;
   constexpr int XL = ROWS * CPR / 256;
@@ -774,8 +775,26 @@ __global__ __launch_bounds__(256, MT == 4 ? 2 : 1) void wstream_grouped_kernel(c
   } else {
     compute(0, wa);
   }
+  // the last products' results are complete before anything reads them, whatever branches lie in between
+  __builtin_amdgcn_sched_barrier(0);
+  asm volatile("s_nop 15");
+  __builtin_amdgcn_sched_barrier(0);
 
   if constexpr (!COMBINE) {
+    if (relu2) {  // (uniform) an up projection without a gate: relu squared, every wave its own 32 columns
+      __syncthreads();
+      if (!active) return;
+      const int n = nb * 32 + r;
+#pragma unroll
+      for (int mt = 0; mt < MT; ++mt)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+          const int m = mt * 32 + (i & 3) + 8 * (i >> 2) + 4 * h;
+          const float p = fmaxf(acc[mt][i], 0.f);
+          if (m < rows) Y[(int64_t)(seg0 + row0 + m) * ldy + n] = (bf16)(p * p);
+        }
+      return;
+    }
     // SwiGLU epilogue: odd waves hand their up tile to the even wave of the pair through LDS
     float* red = reinterpret_cast<float*>(&xs[0][0]);
     __syncthreads();
@@ -1003,12 +1022,13 @@ extern "C" hipError_t kafka_launch_slab_reduce(const float* P, int S, int M, int
 
 namespace kafka {
 // Grouped streaming GEMM for the expert MLP (see wstream_grouped_kernel). max_rows bounds any expert's segment
-// (the token count T: a token picks an expert at most once); glu: gate_up with fused SwiGLU into Y [n_ent, N/2];
+// (the token count T: a token picks an expert at most once); glu: gate_up with fused SwiGLU into Y [n_ent, N/2]
+// (relu2: an up projection into Y [n_ent, N]);
 // else combine into out_f32 [T, N].
 extern "C" hipError_t kafka_launch_wstream_grouped(const bf16* X, int64_t ldx, const bf16* Wt, int e_local, int N,
                                                   int K, const int* perm_tok, const float* perm_w,
                                                   const int* expert_off, int e_lo, int max_rows, int gather,
-                                                  bf16* Y, int64_t ldy, float* out, int64_t ldo, int pin,
+                                                  bf16* Y, int64_t ldy, float* out, int64_t ldo, int pin, int relu2,
                                                   float glu_limit, float glu_alpha, hipStream_t st) {
   if (max_rows < 1 || e_local < 1) return hipSuccess;
   if (N % 64 != 0 || K % 256 != 0 || (out == nullptr) == (Y == nullptr)) return hipErrorInvalidValue;
@@ -1032,11 +1052,11 @@ extern "C" hipError_t kafka_launch_wstream_grouped(const bf16* X, int64_t ldx, c
     if (pin)                                                                                                   \
       wstream_grouped_kernel<MT_, KC_, G_, C_, true><<<grid, 256, 0, st>>>(X, ldx, wt, N, K, perm_tok, perm_w,      \
                                                                            expert_off, e_lo, Y, ldy, out, ldo,   \
-                                                                           glu_limit, glu_alpha);               \
+                                                                           relu2, glu_limit, glu_alpha);               \
     else                                                                                                       \
       wstream_grouped_kernel<MT_, KC_, G_, C_, false><<<grid, 256, 0, st>>>(X, ldx, wt, N, K, perm_tok, perm_w,     \
                                                                             expert_off, e_lo, Y, ldy, out, ldo,  \
-                                                                            glu_limit, glu_alpha);              \
+                                                                            relu2, glu_limit, glu_alpha);              \
   } while (0)
   const bool comb = out != nullptr;
   if (MT == 1) {

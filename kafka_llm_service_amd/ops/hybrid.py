@@ -370,7 +370,7 @@ def moe_router(h, w, b, k: int):
     return tw, te
 
 
-GLU_ACTS = ("silu", "swish_clamp")
+GLU_ACTS = ("silu", "swish_clamp")   # of gated experts; "relu2" experts have no gate
 
 
 def _glu_act(act: str, limit: float, alpha: float) -> tuple[float, float]:
@@ -388,24 +388,26 @@ def moe_rows(h, w_gu, w_down, topk_w, topk_e, out, act: str = "silu", limit: flo
     """Routed experts evaluated per (row, chosen expert) pair, any sizes and both dtypes:
     out[t] = sum_j topk_w[t, j] W_down[e_tj] act(W_gate[e_tj] h_t, W_up[e_tj] h_t) with w_gu [E, 2 F, d] = gate
     rows then up rows and w_down [E, d, F]; the pairs of a row are summed in order j = 0, 1, ... (fp32).
-    ``act``: "silu" = silu(g) * u, or "swish_clamp" (see ``swish_clamp_mul``)."""
-    lim, al = _glu_act(act, limit, alpha)
+    ``act``: "silu" = silu(g) * u, or "swish_clamp" (see ``swish_clamp_mul``); "relu2": experts without a gate, w_gu
+    [E, F, d] alone and W_down relu(W_up h)^2."""
+    glu = act != "relu2"
+    lim, al = _glu_act(act, limit, alpha) if glu else (0.0, 1.0)
     if _gpu(h):
         T, k = topk_e.shape
         a = torch.empty(T * k, w_down.shape[2], dtype=h.dtype, device=h.device)
-        ext().hy_moe_rows(h, w_gu, w_down, topk_w, topk_e, a, out, lim, al)
+        ext().hy_moe_rows(h, w_gu, w_down, topk_w, topk_e, a, out, lim, al, glu)
     else:
-        ref.moe_rows(h, w_gu, w_down, topk_w, topk_e, out, lim, al)
+        ref.moe_rows(h, w_gu, w_down, topk_w, topk_e, out, lim, al, glu)
 
 
 MOE_STREAM_MAX_T = 640  # steps of up to this many rows run tiled expert weights on the grouped streaming kernel
 
 
-def moe_grouped_ok(h, w_gu, w_down) -> bool:
+def moe_grouped_ok(h, w_gu, w_down, glu: bool = True) -> bool:
     """bf16 GPU tensors of sizes the expert-sorted matrix-core kernels take (ops.grouped_gemm)."""
     E, F2, d = w_gu.shape
-    return bool(h.is_cuda and h.dtype == torch.bfloat16 and F2 % 128 == 0 and d % 128 == 0 and (F2 // 2) % 64 == 0 and
-                h.stride(0) % 8 == 0)
+    return bool(h.is_cuda and h.dtype == torch.bfloat16 and F2 % 128 == 0 and d % 128 == 0 and
+                (F2 // 2 if glu else F2) % 64 == 0 and h.stride(0) % 8 == 0)
 
 
 def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None, act: str = "silu",
@@ -415,17 +417,25 @@ def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None
     gathered rows, silu * up, down GEMM with the weighted combine in its epilogue (fp32 adds, two entries per row
     commute), or the grouped weight-streaming kernels when tiled expert weights are given and the step is small -
     everything else is evaluated per (row, expert) pair by ``moe_rows``. ``act`` as in ``moe_rows`` (the streaming
-    kernel applies it in its epilogue; between the two expert-sorted GEMMs it is a launch of its own)."""
+    kernel applies it in its epilogue; between the two expert-sorted GEMMs it is a launch of its own, "relu2" is part
+    of the first)."""
     from kafka_llm_service_amd import ops
 
     T = h.shape[0]
-    if T and moe_grouped_ok(h, w_gu, w_down):
+    glu = act != "relu2"
+    if T and moe_grouped_ok(h, w_gu, w_down, glu):
         r = ops.moe_sort(topk_w, topk_e, w_gu.shape[0])
         out.zero_()
         if w_gu_t is not None and w_down_t is not None and T <= MOE_STREAM_MAX_T:
-            lim, al = _glu_act(act, limit, alpha)
-            a = ops.grouped_stream_glu(h, w_gu_t, r, limit=lim, alpha=al)
+            if glu:
+                lim, al = _glu_act(act, limit, alpha)
+                a = ops.grouped_stream_glu(h, w_gu_t, r, limit=lim, alpha=al)
+            else:
+                a = ops.grouped_stream_relu2(h, w_gu_t, r)
             ops.grouped_stream_combine(a, w_down_t, r, T, out)
+        elif not glu:
+            a = ops.grouped_gemm(h, w_gu, r, gather=True, relu2=True)
+            ops.grouped_gemm(a, w_down, r, gather=False, combine_out=out)
         else:
             gu = ops.grouped_gemm(h, w_gu, r, gather=True)
             if act == "silu":
@@ -527,7 +537,8 @@ def window_attn_mfma_ok(q, k_cache, v_cache_t, H: int, G: int, shared_keys: bool
 
 
 def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int, G: int, scale: float, window: int,
-                sink, out, tiles=None, max_keys: int = 0, shared_keys: bool = False, out_scale: float = 1.0) -> None:
+                sink, out, tiles=None, max_keys: int = 0, shared_keys: bool = False, out_scale: float = 1.0, gate=None,
+                gate_off: int = 0) -> None:
     """Causal softmax attention over paged keys [pages, page, G D] and page-wise transposed values [pages, G Dv, page]:
     row t at position p, head h (key/value head h // (H / G)) sees the keys p - window < j <= p (window 0: all j <= p);
         out = sum_j e^(s_j) v_j / (sum_j e^(s_j) + e^(sink[h])),  s_j = (q . k_j) scale
@@ -538,7 +549,9 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
     over more workgroups (``sig_splits``); a merge pass combines them.
     ``shared_keys``: q is [T, H G D] - every query head is a row of the whole key row's size and its score is the
     product with ALL G key heads of a token (queries that hold a mix over the heads, see ``rope_kv_store``); values
-    stay per key/value head. The result is multiplied by ``out_scale``; ``out`` may be a column slice."""
+    stay per key/value head. The result is multiplied by ``out_scale``; ``out`` may be a column slice.
+    ``gate``: rows whose columns [gate_off, gate_off + H) hold one raw gate per head - head h's output is multiplied by
+    sigmoid(gate[t, gate_off + h])."""
     if window < 0:
         raise ValueError("window_attn: window must be positive (0 = every earlier position)")
     if _gpu(q):
@@ -555,13 +568,13 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
                 pml = torch.empty(ns, q.shape[0], H, 2, dtype=torch.float32, device=q.device)
             ext().hy_window_attn_mfma(q, k_cache, v_cache_t, block_tables, tiles, tt, positions, int(H), int(G),
                                       float(scale), int(window), sink, out, ns, po, pml, bool(shared_keys),
-                                      float(out_scale))
+                                      float(out_scale), gate, int(gate_off))
         else:
             ext().hy_window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, int(H), int(G), float(scale),
-                                 int(window), sink, out, bool(shared_keys), float(out_scale))
+                                 int(window), sink, out, bool(shared_keys), float(out_scale), gate, int(gate_off))
     else:
         ref.window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H, G, scale, window, sink, out,
-                        shared_keys, out_scale)
+                        shared_keys, out_scale, gate, gate_off)
 
 
 def moe_router_grouped(h, w, correction, k: int, groups: int, keep: int, eps: float = 0.0, extra_gate: bool = False,
@@ -763,3 +776,37 @@ def lin_scan(qk, q_off: int, k_off: int, v, z, z_bias, H: int, G: int, D: int, D
             ext().hy_lin_scan(*args, seg, int(rows[0]), int(hi), None, S, out)
     else:
         ref.lin_scan(qk, q_off, k_off, v, z, z_bias, H, G, D, Dv, tok_seg, seg, S, out, tau, rate, beta)
+
+
+# ---- residual with element-wise tanh norms, products with fp32 results ----------------------------------------------
+class TanhNorm:
+    """An element-wise norm tanh(alpha x) * w + b: alpha a number, w and b fp32 [d]."""
+    __slots__ = ("alpha", "w", "b")
+
+    def __init__(self, alpha: float, w: torch.Tensor, b: torch.Tensor):
+        self.alpha, self.w, self.b = float(alpha), w, b
+
+
+def add_tanh_norm(x, y1=None, y2=None, norms=(), outs=(), copy=None, assign: bool = False) -> None:
+    """One element-wise pass over the fp32 stream x [T, d], every part optional:
+      x += y1 + y2, or with ``assign`` x = y1 + y2 (y1 [T, d] in the activation dtype or fp32, or the fp32 split-K slabs
+      [S, T, d] of a projection, summed here; y2 fp32);
+      outs[k] = norms[k](new x), up to two ``TanhNorm``; copy = new x in its dtype (both may be column slices)."""
+    if len(norms) != len(outs) or len(norms) > 2:
+        raise ValueError("add_tanh_norm: up to two norms, an output each")
+    if y1 is None and (y2 is not None or assign):
+        raise ValueError("add_tanh_norm: y2 and assign need y1")
+    if _gpu(x):
+        ext().hy_add_tanh_norm(x, y1, y2, bool(assign), [n.alpha for n in norms], [n.w for n in norms],
+                               [n.b for n in norms], list(outs), copy)
+    else:
+        ref.add_tanh_norm(x, y1, y2, norms, outs, copy, assign)
+
+
+def linear_f32(x, w) -> torch.Tensor:
+    """x @ w^T with an fp32 result for operands in the activation dtype (one matrix product, nothing rounded to it)."""
+    if x.dtype == torch.float32:
+        return torch.nn.functional.linear(x, w)
+    if _gpu(x):
+        return torch.mm(x, w.t(), out_dtype=torch.float32)
+    return torch.nn.functional.linear(x.float(), w.float())

@@ -295,9 +295,10 @@ def _glu(gu, Fh, limit, alpha):
     return F.silu(g) * u
 
 
-def moe_rows(h, w_gu, w_down, topk_w, topk_e, out, limit=0.0, alpha=1.0):
+def moe_rows(h, w_gu, w_down, topk_w, topk_e, out, limit=0.0, alpha=1.0, glu=True):
     """out[t] = sum_j topk_w[t, j] W_down[e] act(W_gate[e] h_t, W_up[e] h_t), e = topk_e[t, j]; w_gu [E, 2 F, d]
-    = gate rows then up rows, w_down [E, d, F]; act = silu(g) * u, or with a limit the clamped swish form."""
+    = gate rows then up rows, w_down [E, d, F]; act = silu(g) * u, or with a limit the clamped swish form. Without
+    ``glu`` w_gu [E, F, d] are up rows alone and the activation is relu squared."""
     T, k = topk_e.shape
     Fh = w_down.shape[2]
     hf = h.float()
@@ -305,7 +306,7 @@ def moe_rows(h, w_gu, w_down, topk_w, topk_e, out, limit=0.0, alpha=1.0):
     for j in range(k):
         e = topk_e[:, j].long()
         gu = torch.einsum("tfd,td->tf", w_gu[e].float(), hf)
-        a = _glu(gu, Fh, limit, alpha).to(h.dtype).float()
+        a = (_glu(gu, Fh, limit, alpha) if glu else torch.relu(gu).square()).to(h.dtype).float()
         acc += topk_w[:, j:j + 1].float() * torch.einsum("tdf,tf->td", w_down[e].float(), a)
     out.copy_(acc)
 
@@ -361,7 +362,7 @@ def qk_norm_rope_store(qkv, H, G, D, Dv, q_w, k_w, eps, positions, cos_sin, rot_
 
 
 def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H, G, scale, window, sink, out,
-                shared_keys=False, out_scale=1.0):
+                shared_keys=False, out_scale=1.0, gate=None, gate_off=0):
     """``shared_keys``: every query head is a row of the whole key row's size and meets all G key heads at once
     (queries that already hold a mix over the heads); values stay per key/value head."""
     T = q.shape[0]
@@ -382,6 +383,8 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H, G, s
             s = torch.cat([s, sink.float()[:, None]], 1)
         pw = torch.softmax(s, -1)[:, :n - lo]
         o = torch.einsum("hj,jhv->hv", pw, v.repeat_interleave(rep, 1)) * out_scale
+        if gate is not None:
+            o = o * torch.sigmoid(gate[t, gate_off:gate_off + H].float())[:, None]
         out[t] = o.reshape(H * Dv).to(out.dtype)
 
 
@@ -535,3 +538,19 @@ def lin_scan(qk, q_off, k_off, v, z, z_bias, H, G, D, Dv, tok_seg, seg, S, out, 
             St = St + k[t][:, :, None] * u[:, None, :]
             out[t] = torch.einsum("hdv,hd->hv", St, q[t]).reshape(-1)
         S[slot] = St
+
+
+def add_tanh_norm(x, y1, y2, norms, outs, copy, assign):
+    """x (+)= y1 + y2 (y1 may be split-K slabs [S, T, d]); outs[k] = tanh(alpha_k x) w_k + b_k; copy = x."""
+    if y1 is not None:
+        y = y1.float().sum(0) if y1.dim() == 3 else y1.float()
+        if y2 is not None:
+            y = y + y2.float()
+        if assign:
+            x.copy_(y)
+        else:
+            x += y
+    if copy is not None:
+        copy.copy_(x)
+    for n, o in zip(norms, outs):
+        o.copy_(torch.tanh(n.alpha * x) * n.w + n.b)
