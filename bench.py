@@ -110,7 +110,9 @@ def parse(argv=None):
                          "experts, 2 per token, and a shared one, of a third of the dense feed-forward each), magedra "
                          "(latent attention, minGRU and parallel head-mixed attention + HGRN2 layers over 4 residual "
                          "streams, the dense clamped feed-forward), rogosun (gated linear attention and parallel "
-                         "attention + gated delta rule layers; dense squared-relu and routed feed-forwards in turn)")
+                         "attention + gated delta rule layers; dense squared-relu and routed feed-forwards in turn), furapel "
+                         "(head-gated attention, windowed latent attention and mlstm layers in parallel with 16 routed "
+                         "squared-relu experts, 4 per token; one layer fewer than the others, one of them run twice)")
     return ap.parse_args(argv)
 
 
@@ -121,7 +123,9 @@ def arch_compare(args) -> int:
     import torch
 
     from kafka_llm_service_amd.engine.engine import EngineConfig, LLMEngine
-    from kafka_llm_service_amd.models.config import ModelConfig, _budurax, _lisorax, _magedra, _mozidra, _rogosun
+    from kafka_llm_service_amd.models.config import (ModelConfig, _budurax, _furapel, _lisorax, _magedra, _mozidra,
+                                                     _rogosun)
+    from kafka_llm_service_amd.models.furapel import FurapelConfig
     from kafka_llm_service_amd.models.magedra import MagedraConfig
     from kafka_llm_service_amd.models.budurax import BuduraxConfig
     from kafka_llm_service_amd.models.lisorax import LisoraxConfig
@@ -143,6 +147,10 @@ def arch_compare(args) -> int:
             "magedra": MagedraConfig.from_dict(_magedra(w, heads, 2, L, vocab, ff), name=f"magedra-w{w}-l{L}"),
             "rogosun": RogosunConfig.from_dict(_rogosun(w, heads, 2, L, vocab, ff, expert_ff=ff // 3 // 256 * 256),
                                                name=f"rogosun-w{w}-l{L}"),
+            # (experts without a gate: 4 of 3 / 8 of the dense feed-forward's rows each have its multiply-adds)
+            "furapel": FurapelConfig.from_dict(_furapel(w, heads, max(1, heads // 4), max(2, L - 1), vocab,
+                                                        ff * 3 // 8 // 256 * 256, loop=(1, 2, 2)),
+                                               name=f"furapel-w{w}-l{L}"),
             "llama": ModelConfig(name=f"llama-w{w}-l{L}", hidden_size=w, intermediate_size=ff, num_layers=L,
                                  num_heads=heads, num_kv_heads=max(1, heads // 4), vocab_size=vocab,
                                  max_position_embeddings=131072, bos_token_id=1, eos_token_ids=[2])}

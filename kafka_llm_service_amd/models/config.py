@@ -257,10 +257,10 @@ ROGOSUN_PRESETS: dict[str, dict] = {
 
 
 def _furapel(width: int, heads: int, kv_heads: int, n_layers: int, vocab: int, ff: int, experts: int = 16, top: int = 4,
-             window: int = 1024, head_dim: int = 128) -> dict:
+             window: int = 1024, head_dim: int = 128, loop: tuple | None = None) -> dict:
     """A Furapel config dict at transformer-like sizes: layers cycle attention, mlstm (``width / 256`` heads of 128 x 256),
     attention, latent attention (rank 512, sliding window); every layer with ``experts`` routed experts of ``ff`` rows,
-    ``top`` per token; the middle half of the depth runs twice."""
+    ``top`` per token; layers ``loop`` = (start, stop, times) are looped over (default: the middle half, twice)."""
     moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
     layers = []
     for i in range(n_layers):
@@ -278,9 +278,10 @@ def _furapel(width: int, heads: int, kv_heads: int, n_layers: int, vocab: int, f
                                                                  "scale": 128 ** -0.5, "mask": {"size": window}},
                            "mlp": moe})
     q = n_layers // 4
+    start, stop, times = loop or (q, n_layers - max(1, q), 2)
     return {"architecture": "Furapel", "vocab": vocab, "width": width, "layers": layers, "norm": {"eps": 1e-6},
             "embedding": {"scale": float(width) ** 0.5}, "logit_scale": 0.25,
-            "loop": {"start": q, "stop": n_layers - max(1, q), "times": 2}}
+            "loop": {"start": start, "stop": stop, "times": times}}
 
 
 FURAPEL_PRESETS: dict[str, dict] = {
