@@ -220,6 +220,25 @@ class SegMeta:
     max_keys: int = 0         # longest context of the step (first position + rows over the runs)
     cache: dict = field(default_factory=dict)   # per-step device tables derived from seg_host (chunk plans)
 
+    def chunks(self, chunk: int, min_rows: int):
+        """(device tensors of ``hops.chunk_tables`` or None, (fewest, most rows) of the segments that are too short for
+        chunks or None), built once per step. On the CPU nothing runs in chunks."""
+        key = ("chunk tables", chunk, min_rows)
+        if key not in self.cache:
+            tabs, short = None, (1, 1 << 30)
+            if self.seg.is_cuda and self.seg_host is not None and len(self.seg_host):
+                tabs = hops.chunk_tables(self.seg_host, chunk, min_rows)
+                rows = self.seg_host[:, 1]
+                if tabs is not None:
+                    rows = rows[rows < min_rows]
+                short = (int(rows.min()), int(rows.max())) if len(rows) else None
+                if tabs is not None:
+                    n = tabs[0].size
+                    up = torch.cat([torch.from_numpy(t).view(-1) for t in tabs]).to(self.seg.device)
+                    tabs = (up[:n].view(-1, 4), up[n:].view(-1, 4))
+            self.cache[key] = (tabs, short)
+        return self.cache[key]
+
 
 @dataclass
 class RecurrentState:

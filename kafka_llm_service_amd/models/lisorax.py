@@ -491,7 +491,8 @@ class LisoraxLM:
         proj = self._lin(hm, lw.w_in, getattr(lw, "w_in_t", None))                # [q | k | v | output gate]
         gates = torch.addmm(lw.gate_b, hm.float(), lw.gate_w.t())                  # fp32 [T, 2 H]: input | forget
         o = torch.empty(T, H * Dv, dtype=torch.float32, device=dev)
-        hops.mlstm_scan(proj, gates, H, D, Dv, lw.cap, m.tok_seg, m.seg, st["S"], st["n"], st["m"], o)
+        chunks, short = m.chunks(hops.MLSTM_CHUNK, hops.MLSTM_CHUNK_MIN)
+        hops.mlstm_scan(proj, gates, H, D, Dv, lw.cap, m.tok_seg, m.seg, st["S"], st["n"], st["m"], o, chunks, short)
         on = torch.empty(T, H * Dv, dtype=dt, device=dev)
         hops.head_norm_gate(o, lw.mnorm, proj, 2 * H * D + H * Dv, H, self.cfg.norm_eps, on)
         return self._lin(on, lw.o, getattr(lw, "o_t", None))

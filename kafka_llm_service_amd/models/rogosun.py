@@ -495,32 +495,13 @@ class RogosunLM:
         hops.rms_norm(xs, self.final_norm, eps, hf)
         return self._lin(hf, self.head, getattr(self, "head_t", None)).float()[:, :cfg.vocab_size]
 
-    def _chunks(self, m: SegMeta):
-        """(chunk tables on the device or None, fewest and most rows of the segments that are scanned token by token or
-        None), built once per step."""
-        if "lin" not in m.cache:
-            tabs, short = None, (1, 1 << 30)
-            if self.device.type == "cuda" and m.seg_host is not None and len(m.seg_host):
-                tabs = hops.lin_chunk_tables(m.seg_host)
-                rows = m.seg_host[:, 1]
-                if tabs is not None:
-                    rows = rows[rows < hops.LIN_CHUNK_MIN]
-                short = (int(rows.min()), int(rows.max())) if len(rows) else None
-                if tabs is not None:
-                    nv = tabs[0].size
-                    up = torch.from_numpy(tabs[0]).view(-1)
-                    up = torch.cat([up, torch.from_numpy(tabs[1]).view(-1)]).to(self.device)
-                    tabs = (up[:nv].view(-1, 4), up[nv:].view(-1, 4))
-            m.cache["lin"] = (tabs, short)
-        return m.cache["lin"]
-
     def _gla(self, lw, h, m: SegMeta, st: dict) -> torch.Tensor:
         H, D, Dv = (int(lw.m[k]) for k in ("heads", "dim", "vdim"))
         T, dt, dev, off = h.shape[0], self.dtype, self.device, lw.off
         proj = self._lin(h, lw.w_in, getattr(lw, "w_in_t", None))                 # [q | k | v | g | a1]
         z = F.linear(proj[:, off["a1"]:off["a1"] + lw.low.shape[1]], lw.low)      # raw decays
         o = torch.empty(T, H * Dv, dtype=torch.float32, device=dev)
-        chunks, short = self._chunks(m)
+        chunks, short = m.chunks(hops.LIN_CHUNK, hops.LIN_CHUNK_MIN)
         hops.lin_scan(proj, off["q"], off["k"], proj[:, off["v"]:off["v"] + H * Dv], z, lw.z_bias, H, H, D, Dv,
                       m.tok_seg, m.seg, st["S"], o, tau=lw.tau, chunks=chunks, rows=short)
         on = torch.empty(T, H * Dv, dtype=dt, device=dev)
@@ -546,7 +527,7 @@ class RogosunLM:
         hops.short_conv(proj, off["conv"], lw.conv, None, m.tok_seg, m.seg, st["conv"], qkv, act="silu")
         low = F.linear(proj[:, off["low"]:off["low"] + lw.low.shape[1]], lw.low)  # raw decays | output gate
         o = torch.empty(T, Hr * Dvr, dtype=torch.float32, device=dev)
-        chunks, short = self._chunks(m)
+        chunks, short = m.chunks(hops.LIN_CHUNK, hops.LIN_CHUNK_MIN)
         hops.lin_scan(qkv, 0, Gr * Dr, qkv[:, 2 * Gr * Dr:], low[:, :Hr * Dr], lw.z_bias, Hr, Gr, Dr, Dvr, m.tok_seg,
                       m.seg, st["S"], o, rate=lw.rate, beta=proj[:, off["b"]:off["b"] + Hr], chunks=chunks,
                       rows=short)

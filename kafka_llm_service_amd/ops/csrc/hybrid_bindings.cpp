@@ -75,9 +75,20 @@ hipError_t kafka_hy_rglru_scan_chunked(int f32, float* gates, int64_t gs, const 
                                        int64_t us, const float* rate, const int* seg, int R, int nch, float* ab,
                                        float* state, void* out, int64_t os, int64_t T, int W, hipStream_t st);
 int kafka_hy_mlstm_max_d();
+int kafka_hy_mlstm_cols();
 hipError_t kafka_hy_mlstm_scan(int f32, const void* qkv, int64_t qs, const float* gates, int64_t gs, int H, int D,
+                               int Dv, float cap, const int* seg, int R, int min_n, int max_n, float* S, float* nrm,
+                               float* mx, float* fin, float* out, int64_t os, hipStream_t st);
+int kafka_hy_mlstm_step_ok(int D, int Dv);
+hipError_t kafka_hy_mlstm_step(int f32, const void* qkv, int64_t qs, const float* gates, int64_t gs, int H, int D,
                                int Dv, float cap, const int* seg, int R, float* S, float* nrm, float* mx, float* out,
                                int64_t os, hipStream_t st);
+int kafka_hy_mlstm_chunk();
+int kafka_hy_mlstm_chunk_ok(int H, int D, int Dv, int64_t qs);
+int64_t kafka_hy_mlstm_chunk_scratch(int D, int Dv);
+hipError_t kafka_hy_mlstm_chunked(const void* qkv, int64_t qs, const float* gates, int64_t gs, int H, int D, int Dv,
+                                  float cap, const int* vseg, int n_chunks, const int* cs, int R, float* scratch,
+                                  float* S, float* nrm, float* mx, float* out, int64_t os, hipStream_t st);
 hipError_t kafka_hy_head_norm_gate(int f32, const float* o, int64_t os_, const void* w, const void* g, int64_t gs,
                                    int g_off, int H, int Dv, float eps, void* out, int64_t outs, int64_t T,
                                    float scale, int silu, hipStream_t st);
@@ -669,12 +680,14 @@ void rglru_scan(at::Tensor gates, at::Tensor proj, at::Tensor u, at::Tensor rate
                              state.data_ptr<float>(), out.data_ptr(), out.stride(0), (int)W, stream()));
 }
 
+// seg: segments of min_n .. max_n rows token by token; or vseg / cs (ops.hybrid.chunk_tables, which keeps chunks inside
+// their segments and numbers them 0 .. n - 1): the segments of cs in chunks
 void mlstm_scan(at::Tensor qkv, at::Tensor gates, int64_t H, int64_t D, int64_t Dv, double cap, at::Tensor seg,
-                at::Tensor S, at::Tensor nrm, at::Tensor mx, at::Tensor out) {
+                int64_t min_n, int64_t max_n, OptT cs, at::Tensor S, at::Tensor nrm, at::Tensor mx, at::Tensor out) {
   rows2d(qkv, "qkv"); rows2d(gates, "gates"); rows2d(out, "out");
   f32t(gates, "gates"); f32t(S, "S"); f32t(nrm, "n"); f32t(mx, "m"); f32t(out, "out");
   const int f32 = act_f32(qkv);
-  const int64_t T = qkv.size(0);
+  const int64_t T = qkv.size(0), R = seg.size(0);
   seg_only(seg);
   TORCH_CHECK(H >= 1 && D >= 1 && Dv >= 1 && D <= kafka_hy_mlstm_max_d(), "mlstm_scan: head sizes (dim up to ",
               kafka_hy_mlstm_max_d(), ")");
@@ -686,10 +699,33 @@ void mlstm_scan(at::Tensor qkv, at::Tensor gates, int64_t H, int64_t D, int64_t 
                   nrm.is_contiguous() && nrm.dim() == 3 && nrm.size(0) == slots && nrm.size(1) == H &&
                   nrm.size(2) == D && mx.is_contiguous() && mx.dim() == 2 && mx.size(0) == slots && mx.size(1) == H,
               "mlstm_scan: state S [slots, H, D, Dv], n [slots, H, D], m [slots, H]");
+  auto f32o = at::TensorOptions().dtype(at::kFloat).device(qkv.device());
+  float *Sp = S.data_ptr<float>(), *np = nrm.data_ptr<float>(), *mp = mx.data_ptr<float>(), *op = out.data_ptr<float>();
+  if (cs.has_value()) {
+    seg_only(*cs);
+    TORCH_CHECK(!f32 && kafka_hy_mlstm_chunk_ok((int)H, (int)D, (int)Dv, qkv.stride(0)) && out.stride(0) % 4 == 0 &&
+                    (reinterpret_cast<uintptr_t>(qkv.data_ptr()) & 15) == 0 &&
+                    (reinterpret_cast<uintptr_t>(op) & 15) == 0, "mlstm_scan: sizes not supported in chunks");
+    at::Tensor scratch = at::empty({R * H * kafka_hy_mlstm_chunk_scratch((int)D, (int)Dv)}, f32o);
+    HY_HIP(kafka_hy_mlstm_chunked(qkv.data_ptr(), qkv.stride(0), gates.data_ptr<float>(), gates.stride(0), (int)H,
+                                  (int)D, (int)Dv, (float)cap, seg.data_ptr<int>(), (int)R, cs->data_ptr<int>(),
+                                  (int)cs->size(0), scratch.data_ptr<float>(), Sp, np, mp, op, out.stride(0),
+                                  stream()));
+    return;
+  }
+  if (min_n <= 1 && kafka_hy_mlstm_step_ok((int)D, (int)Dv) && (reinterpret_cast<uintptr_t>(Sp) & 15) == 0) {
+    HY_HIP(kafka_hy_mlstm_step(f32, qkv.data_ptr(), qkv.stride(0), gates.data_ptr<float>(), gates.stride(0), (int)H,
+                               (int)D, (int)Dv, (float)cap, seg.data_ptr<int>(), (int)R, Sp, np, mp, op,
+                               out.stride(0), stream()));
+    min_n = 2;
+  }
+  if (max_n < min_n) return;
+  at::Tensor fin;
+  if (Dv > kafka_hy_mlstm_cols()) fin = at::empty({R * H * (D + 1)}, f32o);
   HY_HIP(kafka_hy_mlstm_scan(f32, qkv.data_ptr(), qkv.stride(0), gates.data_ptr<float>(), gates.stride(0), (int)H,
-                             (int)D, (int)Dv, (float)cap, seg.data_ptr<int>(), (int)seg.size(0), S.data_ptr<float>(),
-                             nrm.data_ptr<float>(), mx.data_ptr<float>(), out.data_ptr<float>(), out.stride(0),
-                             stream()));
+                             (int)D, (int)Dv, (float)cap, seg.data_ptr<int>(), (int)R,
+                             (int)min_n, (int)std::min<int64_t>(max_n, 0x7fffffff), Sp, np, mp,
+                             fin.defined() ? fin.data_ptr<float>() : nullptr, op, out.stride(0), stream()));
 }
 
 void head_norm_gate(at::Tensor o, at::Tensor w, OptT g, int64_t g_off, int64_t H, double eps, at::Tensor out,
@@ -1275,7 +1311,12 @@ void kafka_bind_hybrid(pybind11::module_& m) {
   m.def("hy_sigmoid_attn", &sigmoid_attn);
   m.def("hy_rglru_scan", &rglru_scan, py::arg("gates"), py::arg("proj"), py::arg("u"), py::arg("rate"), py::arg("seg"),
         py::arg("state"), py::arg("out"), py::arg("max_rows") = 0);
-  m.def("hy_mlstm_scan", &mlstm_scan);
+  m.def("hy_mlstm_scan", &mlstm_scan, py::arg("qkv"), py::arg("gates"), py::arg("H"), py::arg("D"), py::arg("Dv"),
+        py::arg("cap"), py::arg("seg"), py::arg("min_n"), py::arg("max_n"), py::arg("cs"), py::arg("S"), py::arg("nrm"),
+        py::arg("mx"), py::arg("out"));
+  m.def("hy_mlstm_chunk", []() { return kafka_hy_mlstm_chunk(); });
+  m.def("hy_mlstm_chunk_ok",
+        [](int H, int D, int Dv, int64_t qs) { return kafka_hy_mlstm_chunk_ok(H, D, Dv, qs) != 0; });
   m.def("hy_head_norm_gate", &head_norm_gate, py::arg("o"), py::arg("w"), py::arg("g"), py::arg("g_off"), py::arg("H"),
         py::arg("eps"), py::arg("out"), py::arg("scale") = 1.0, py::arg("silu") = false);
   m.def("hy_moe_topk", &moe_topk);

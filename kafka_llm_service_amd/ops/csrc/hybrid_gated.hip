@@ -484,9 +484,10 @@ constexpr int ML_TB = 8;   // tokens per staged block
 template <typename AT, int RD>
 __global__ __launch_bounds__(NT) void mlstm_scan_kernel(const AT* __restrict__ qkv, int64_t qs,
                                                         const float* __restrict__ gates, int64_t gs, int H, int D,
-                                                        int Dv, float cap, const int* __restrict__ seg,
-                                                        float* __restrict__ Sst, float* __restrict__ nst,
-                                                        float* __restrict__ mst, float* __restrict__ out, int64_t os) {
+                                                        int Dv, float cap, const int* __restrict__ seg, int min_n,
+                                                        int max_n, float* __restrict__ Sst, float* __restrict__ nst,
+                                                        float* __restrict__ mst, float* __restrict__ fin,
+                                                        float* __restrict__ out, int64_t os) {
   constexpr int DMAX = ML_DG * RD;
   constexpr int NQK = (2 * DMAX * ML_TB + NT - 1) / NT;   // staged q | k elements per thread
   constexpr int NV = (64 * ML_TB + NT - 1) / NT;          // staged value elements per thread
@@ -497,6 +498,7 @@ __global__ __launch_bounds__(NT) void mlstm_scan_kernel(const AT* __restrict__ q
   __shared__ float msh[ML_TB];
   const int r = blockIdx.z, h = blockIdx.y, v0 = blockIdx.x * ML_VS;
   const int q0 = seg[4 * r], n = seg[4 * r + 1], p0 = seg[4 * r + 2], slot = seg[4 * r + 3];
+  if (n < min_n || n > max_n) return;   // (uniform) another kernel's segment
   const int dg = threadIdx.x >> 6, vv = threadIdx.x & 63;
   const bool is_n = vv == ML_VS;                 // the normaliser's lane
   const bool vok = !is_n && v0 + vv < Dv;
@@ -606,10 +608,25 @@ __global__ __launch_bounds__(NT) void mlstm_scan_kernel(const AT* __restrict__ q
     const int d = dg * RD + i;
     if (d < D) {
       if (vok) Sp[(int64_t)d * Dv] = S[i];
-      if (is_n && blockIdx.x == 0) np[d] = S[i];
+      if (is_n && blockIdx.x == 0) (fin != nullptr ? fin + ((int64_t)r * H + h) * (D + 1) : np)[d] = S[i];
     }
   }
-  if (blockIdx.x == 0 && threadIdx.x == 0) mst[(int64_t)slot * H + h] = m;
+  if (blockIdx.x == 0 && threadIdx.x == 0) {
+    if (fin != nullptr) fin[((int64_t)r * H + h) * (D + 1) + D] = m;
+    else mst[(int64_t)slot * H + h] = m;
+  }
+}
+
+// Several workgroups of a (segment, head) start from its normaliser and maximum, at any time: the new ones are left in
+// fin [R][H][D + 1] and stored when all are done.
+__global__ __launch_bounds__(NT) void mlstm_commit_kernel(const float* __restrict__ fin, const int* __restrict__ seg,
+                                                          int min_n, int max_n, int H, int D, float* __restrict__ nst,
+                                                          float* __restrict__ mst) {
+  const int r = blockIdx.y, h = blockIdx.x, n = seg[4 * r + 1], slot = seg[4 * r + 3];
+  if (n < min_n || n > max_n) return;
+  const float* f = fin + ((int64_t)r * H + h) * (D + 1);
+  for (int d = threadIdx.x; d < D; d += NT) nst[((int64_t)slot * H + h) * D + d] = f[d];
+  if (threadIdx.x == 0) mst[(int64_t)slot * H + h] = f[D];
 }
 
 template <typename AT>
@@ -956,21 +973,28 @@ hipError_t kafka_hy_rglru_scan_chunked(int f32, float* gates, int64_t gs, const 
 }
 
 int kafka_hy_mlstm_max_d() { return ML_DG * 64; }
+int kafka_hy_mlstm_cols() { return ML_VS; }
 
 hipError_t kafka_hy_mlstm_scan(int f32, const void* qkv, int64_t qs, const float* gates, int64_t gs, int H, int D,
-                               int Dv, float cap, const int* seg, int R, float* S, float* nrm, float* mx, float* out,
-                               int64_t os, hipStream_t st) {
+                               int Dv, float cap, const int* seg, int R, int min_n, int max_n, float* S, float* nrm,
+                               float* mx, float* fin, float* out, int64_t os, hipStream_t st) {
+  // fin: R H (D + 1) floats of scratch where a head takes more than one workgroup (ML_VS value columns each)
   if (R <= 0) return hipSuccess;
-  if (D > ML_DG * 64 || D < 1 || Dv < 1) return hipErrorInvalidValue;
+  if (D > ML_DG * 64 || D < 1 || Dv < 1 || R > 65535 || H > 65535) return hipErrorInvalidValue;
   const dim3 grid((Dv + ML_VS - 1) / ML_VS, H, R);
+  if (grid.x == 1) fin = nullptr;
+  else if (fin == nullptr) return hipErrorInvalidValue;
 #define ML_LAUNCH(RD)                                                                                              \
-  mlstm_scan_kernel<AT, RD><<<grid, NT, 0, st>>>((const AT*)qkv, qs, gates, gs, H, D, Dv, cap, seg, S, nrm, mx, out, os)
+  mlstm_scan_kernel<AT, RD><<<grid, NT, 0, st>>>((const AT*)qkv, qs, gates, gs, H, D, Dv, cap, seg, min_n, max_n, S, nrm, mx,   \
+                                           fin, out, os)
   DISPATCH_AT(f32, {
     if (D <= ML_DG * 16) ML_LAUNCH(16);
     else if (D <= ML_DG * 32) ML_LAUNCH(32);
     else ML_LAUNCH(64);
   });
 #undef ML_LAUNCH
+  if (fin != nullptr)
+    mlstm_commit_kernel<<<dim3(H, R), NT, 0, st>>>(fin, seg, min_n, max_n, H, D, nrm, mx);
   return hipGetLastError();
 }
 

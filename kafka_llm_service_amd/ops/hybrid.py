@@ -187,6 +187,24 @@ def ssm_scan(xbc, proj, dt_off: int, dt_bias, A_log, D, heads, P, N, G, tok_seg,
         ref.ssm_scan(xbc, proj, dt_off, dt_bias, A_log, D, heads, P, N, G, tok_seg, seg, state, y)
 
 
+def chunk_tables(seg_host, chunk: int, min_rows: int):
+    """Chunk tables of a step: (vseg, cs) as numpy int32, or None when no segment is long enough - every segment of at
+    least ``min_rows`` rows cut into chunks of ``chunk``: vseg[c] = (first row, rows, 0, 0), cs[r] = (first chunk,
+    chunks, first position, state slot)."""
+    import numpy as np
+
+    if seg_host is None:
+        return None
+    vs, cs = [], []
+    for q0, n, p0, slot in seg_host.tolist():
+        if n >= min_rows:
+            cs.append((len(vs), -(-n // chunk), p0, slot))
+            vs += [(q0 + a, min(chunk, n - a), 0, 0) for a in range(0, n, chunk)]
+    if not cs:
+        return None
+    return np.asarray(vs, dtype=np.int32), np.asarray(cs, dtype=np.int32)
+
+
 SCAN_CHUNK = 256        # tokens per chunk of the chunk-parallel scan
 SCAN_CHUNK_MIN = 512    # a step is scanned in chunks when its longest segment has at least this many rows ...
 SCAN_CHUNK_WORK = 2048  # ... and it has fewer (segment, head) pairs than this (else the plain scan fills the GPU)
@@ -328,16 +346,40 @@ def rglru_scan(gates, proj, u, rate, tok_seg, seg, state, out, max_rows: int = 0
         ref.rglru_scan(gates, proj, u, rate, tok_seg, seg, state, out)
 
 
-def mlstm_scan(qkv, gates, H: int, D: int, Dv: int, cap: float, tok_seg, seg, S, nrm, mx, out) -> None:
+MLSTM_CHUNK = 128       # tokens of a chunk (the kernels' constant)
+MLSTM_CHUNK_MIN = 48    # segments of at least this many rows are scanned in chunks
+
+
+def mlstm_chunk_ok(H: int, D: int, Dv: int, qkv) -> bool:
+    """bf16 GPU rows of sizes the chunked matrix-memory kernels take (dim a multiple of 16 up to 256, vdim of 8)."""
+    return qkv.is_cuda and qkv.dtype == torch.bfloat16 and qkv.data_ptr() % 16 == 0 and \
+        bool(ext().hy_mlstm_chunk_ok(int(H), int(D), int(Dv), qkv.stride(0)))
+
+
+def mlstm_scan(qkv, gates, H: int, D: int, Dv: int, cap: float, tok_seg, seg, S, nrm, mx, out, chunks=None,
+               rows=(1, 1 << 30)) -> None:
     """The matrix-memory recurrence (mLSTM) over a step's segments. qkv [T, >= H (2 D + Dv)] = q | k | v heads,
     gates fp32 [T, 2 H] = raw input | forget gate (biases included). Per head, with i = cap tanh(g_i / cap),
     f = logsigmoid(cap tanh(g_f / cap)), q' = q D^(-1/2):
         m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T;  n <- e^(f + m - m') n + e^(i - m') k;
         out = S^T q' / (max(|n . q'|, e^(-m')) + 1e-6).
     State per slot, all fp32 and all zero (m too) before a sequence's first token: S [slots, H, D, Dv],
-    nrm [slots, H, D], mx [slots, H]. out fp32 [T, H Dv]."""
+    nrm [slots, H, D], mx [slots, H]. out fp32 [T, H Dv].
+    ``chunks``: device tensors of ``chunk_tables(seg_host, MLSTM_CHUNK, MLSTM_CHUNK_MIN)`` - where the sizes allow
+    (``mlstm_chunk_ok``) their segments run in chunks (the same recurrence as matrix products, re-associated: fp32
+    rounding only), the others token by token. ``rows``: the shortest and the longest of those others when the caller
+    knows them (None: there are none); segments of one row have a kernel of their own."""
     if _gpu(qkv):
-        ext().hy_mlstm_scan(qkv, gates, int(H), int(D), int(Dv), float(cap), seg, S, nrm, mx, out)
+        if chunks is not None and mlstm_chunk_ok(H, D, Dv, qkv):
+            ext().hy_mlstm_scan(qkv, gates, int(H), int(D), int(Dv), float(cap), chunks[0], 0, 0, chunks[1], S, nrm, mx,
+                                out)
+            if rows is not None:
+                rows = (rows[0], min(rows[1], MLSTM_CHUNK_MIN - 1))
+        elif chunks is not None:
+            rows = (1, 1 << 30)
+        if rows is not None:
+            ext().hy_mlstm_scan(qkv, gates, int(H), int(D), int(Dv), float(cap), seg, int(rows[0]), int(rows[1]), None, S,
+                                nrm, mx, out)
     else:
         ref.mlstm_scan(qkv, gates, H, D, Dv, cap, tok_seg, seg, S, nrm, mx, out)
 
@@ -734,21 +776,9 @@ LIN_CHUNK_MIN = 64    # segments of at least this many rows are scanned in chunk
 
 
 def lin_chunk_tables(seg_host):
-    """Chunk tables of a step for ``lin_scan``: (vseg, cs) as numpy int32, or None when no segment is long enough -
-    every segment of at least LIN_CHUNK_MIN rows cut into chunks of LIN_CHUNK: vseg[c] = (first row, rows, 0, 0),
-    cs[r] = (first chunk, chunks, first position, state slot). Shorter segments stay with the token-by-token kernel."""
-    import numpy as np
-
-    if seg_host is None:
-        return None
-    vs, cs = [], []
-    for q0, n, p0, slot in seg_host.tolist():
-        if n >= LIN_CHUNK_MIN:
-            cs.append((len(vs), -(-n // LIN_CHUNK), p0, slot))
-            vs += [(q0 + a, min(LIN_CHUNK, n - a), 0, 0) for a in range(0, n, LIN_CHUNK)]
-    if not cs:
-        return None
-    return np.asarray(vs, dtype=np.int32), np.asarray(cs, dtype=np.int32)
+    """Chunk tables of a step for ``lin_scan`` (see ``chunk_tables``). Shorter segments stay with the token-by-token
+    kernel."""
+    return chunk_tables(seg_host, LIN_CHUNK, LIN_CHUNK_MIN)
 
 
 def lin_scan(qk, q_off: int, k_off: int, v, z, z_bias, H: int, G: int, D: int, Dv: int, tok_seg, seg, S, out,

@@ -440,6 +440,16 @@ def _mlstm_want(qkv, gates, H, D, Dv, cap):
     return plain.mlstm_scan(q.reshape(n, H, D) * D ** -0.5, k.reshape(n, H, D), v.reshape(n, H, Dv), ig, fg).reshape(n, -1)
 
 
+def _chunks(device, segs):
+    tabs = hops.chunk_tables(np.asarray(segs, dtype=np.int32), hops.MLSTM_CHUNK, hops.MLSTM_CHUNK_MIN)
+    return None if tabs is None or device == "cpu" else tuple(torch.from_numpy(x).to(device) for x in tabs)
+
+
+def _head_errs(o, want, H, Dv):
+    """Per (row, head) against its own size (a read-out is divided by |n . q|, which may be small)."""
+    return (o - want).view(-1, H, Dv).abs().amax(-1) / (want.view(-1, H, Dv).abs().amax(-1) + 1e-3)
+
+
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("H,D,Dv", MLSTM_SIZES)
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
@@ -466,17 +476,63 @@ def test_mlstm_scan(device, H, D, Dv, dtype):
         rows = torch.cat([cases[s][0][p0:p0 + n] for s, p0, n, _ in runs]).to(device)
         gates = torch.cat([cases[s][1][p0:p0 + n] for s, p0, n, _ in runs]).to(device)
         out = torch.full((r0, H * Dv), float("nan"), device=device)
-        hops.mlstm_scan(rows, gates, H, D, Dv, cap, ts, seg, S, nrm, mx, out)
+        hops.mlstm_scan(rows, gates, H, D, Dv, cap, ts, seg, S, nrm, mx, out, _chunks(device, segs))
         for s, p0, n, q0 in runs:
             got[s].append(out[q0:q0 + n].cpu())
             at[s] += n
     assert at == lengths
     for s in (0, 1):
-        # (a read-out is divided by |n . q|, which may be small: rows against their own size)
-        o = torch.cat(got[s]).double()
-        e = (o - want[s]).view(-1, H, Dv).abs().amax(-1) / (want[s].view(-1, H, Dv).abs().amax(-1) + 1e-3)
+        e = _head_errs(torch.cat(got[s]).double(), want[s], H, Dv)
         assert e.median() < 1e-5 and (e < 5e-3).all() and (e < 2e-4).double().mean() > 0.99, s
     assert not torch.isnan(S[1:]).any() and torch.isnan(S[0]).all()
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,D,Dv", [(3, 48, 72), (2, 16, 8), (2, 128, 256), (1, 256, 64), (4, 144, 40), (9, 64, 128)])
+def test_mlstm_in_chunks(H, D, Dv):
+    """The chunked form against the token-by-token kernel and the plain function: every kind of last chunk, segments that
+    continue from a state beside fresh ones, heads inside wider rows, the state it leaves and what single tokens make of
+    it."""
+    dev = "cuda:0"
+    assert hops.ext().hy_mlstm_chunk() == hops.MLSTM_CHUNK
+    g = torch.Generator().manual_seed(D)
+    cap, lengths = 9.0, [21 + 48 + 2, 150 + 257 + 3, 128 + 129 + 1]
+    cases = []
+    for s, n in enumerate(lengths):
+        qkv, gates = _mlstm_case(g, n, H, D, Dv, cap, s == 1)
+        cases.append((torch.cat([qkv, torch.randn(n, 8, generator=g)], 1).to(torch.bfloat16), gates))
+    want = [_mlstm_want(q[:, :-8], z, H, D, Dv, cap) for q, z in cases]
+    steps = [[(0, 21), (1, 150)], [(2, 128), (1, 257), (0, 48)], [(0, 1), (2, 129)], [(1, 1), (0, 1), (2, 1)],
+             [(1, 2)]]
+    res = []
+    for chunked in (False, True):
+        S = torch.full((4, H, D, Dv), float("nan"), device=dev)
+        nrm, mx = torch.full((4, H, D), float("nan"), device=dev), torch.full((4, H), float("nan"), device=dev)
+        at, got = [0, 0, 0], [[], [], []]
+        for st in steps:
+            segs, r0 = [], 0
+            for s, n in st:
+                segs.append((r0, n, at[s], 3 - s))
+                r0 += n
+            rows = torch.cat([cases[s][0][at[s]:at[s] + n] for s, n in st]).to(dev)
+            gates = torch.cat([cases[s][1][at[s]:at[s] + n] for s, n in st]).to(dev)
+            ts, seg = seg_tensors(dev, segs)
+            out = torch.full((r0, H * Dv), float("nan"), device=dev)
+            assert hops.mlstm_chunk_ok(H, D, Dv, rows)
+            hops.mlstm_scan(rows, gates, H, D, Dv, cap, ts, seg, S, nrm, mx, out, _chunks(dev, segs) if chunked else None)
+            r0 = 0
+            for s, n in st:
+                got[s].append(out[r0:r0 + n].cpu())
+                at[s] += n
+                r0 += n
+        assert at == lengths
+        res.append([torch.cat(x).double() for x in got] + [S[1:].cpu(), nrm[1:].cpu(), mx[1:].cpu()])
+        for s in range(3):
+            e = _head_errs(res[-1][s], want[s], H, Dv)
+            assert e.median() < 1e-5 and (e < 5e-3).all() and (e < 2e-4).double().mean() > 0.99, (chunked, s)
+        assert torch.isnan(S[0]).all()
+    for a, b in zip(res[0][3:], res[1][3:]):
+        assert close(b, a, 1e-5)
 
 
 @pytest.mark.parametrize("device", DEVICES)
