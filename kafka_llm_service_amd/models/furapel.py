@@ -278,8 +278,8 @@ class FurapelLM:
     def load_tensors(self, W: dict[str, torch.Tensor]) -> "FurapelLM":
         """Checkpoint tensors (any float dtype) -> device tensors: projections that read the same input fused into
         one GEMM weight in the model dtype (rows padded to a multiple of 32), per-head up-projections reshaped for the
-        batched latent products, experts stacked; the tanh norms, the recurrence's gate projections and the router
-        fp32, the embedding scale folded into an fp32 copy of the table."""
+        batched latent products, experts stacked; the tanh norms, gate biases and the router fp32, the embedding scale
+        folded into an fp32 copy of the table."""
         cfg, dev, dt = self.cfg, self.device, self.dtype
         self.runs = cfg.runs()
         for k, shp in tensor_shapes(cfg).items():
@@ -350,7 +350,7 @@ class FurapelLM:
                 tiles.add(hops.tile_tokens(H))
             else:
                 lw.w_in = fused([q + n for n in ("q", "k", "v", "g")], multiple=32)
-                lw.gate_w = fused([q + "i", q + "f"], torch.float32)
+                lw.gate_w = fused([q + "i", q + "f"])
                 lw.gate_b = fused([q + "i.b", q + "f.b"], torch.float32)
                 lw.mnorm = act(q + "norm")
                 lw.cap = float(m["gate_cap"])
@@ -362,6 +362,8 @@ class FurapelLM:
                 if not 1 <= lw.top <= lw.E:
                     raise ValueError(f"layer {i}: top {lw.top} of {lw.E} experts")
                 lw.norm2, lw.router = norm(p + "norm2"), f32(p + "mlp.router")
+                low = lw.router.to(dt)                                              # where it is exact: one kernel
+                lw.router_a = keep(low) if dt != torch.float32 and torch.equal(low.float(), lw.router) else None
                 lw.w_up = keep(torch.stack([W[f"{p}mlp.e{e}.up"] for e in range(lw.E)]).to(device=dev, dtype=dt))
                 lw.w_down = keep(torch.stack([W[f"{p}mlp.e{e}.down"] for e in range(lw.E)]).to(device=dev, dtype=dt))
             self.layers.append(lw)
@@ -517,7 +519,7 @@ class FurapelLM:
         H, D, Dv = (int(lw.m[k]) for k in ("heads", "dim", "vdim"))
         T, dt, dev = h.shape[0], self.dtype, self.device
         proj = self._lin(h, lw.w_in, getattr(lw, "w_in_t", None))                 # [q | k | v | output gate]
-        gates = torch.addmm(lw.gate_b, h.float(), lw.gate_w.t())                   # fp32 [T, 2 H]: input | forget
+        gates = hops.linear_f32(h, lw.gate_w, lw.gate_b)                           # fp32 [T, 2 H]: input | forget
         o = torch.empty(T, H * Dv, dtype=torch.float32, device=dev)
         chunks, short = m.chunks(hops.MLSTM_CHUNK, hops.MLSTM_CHUNK_MIN)
         hops.mlstm_scan(proj, gates, H, D, Dv, lw.cap, m.tok_seg, m.seg, st["S"], st["n"], st["m"], o, chunks, short)
@@ -527,7 +529,7 @@ class FurapelLM:
 
     def _experts(self, lw, h) -> torch.Tensor:
         """The routed experts' weighted sum, fp32 [T, d]."""
-        tw, te, _ = hops.moe_router_grouped(h, lw.router, None, lw.top, 1, 1, norm=False)
+        tw, te, _ = hops.moe_router_grouped(h, lw.router, None, lw.top, 1, 1, norm=False, w_act=lw.router_a)
         out = torch.empty(h.shape[0], self.cfg.hidden_size, dtype=torch.float32, device=self.device)
         hops.moe_experts(h, lw.w_up, lw.w_down, tw, te, out, getattr(lw, "w_up_t", None), getattr(lw, "w_down_t", None),
                          act="relu2")

@@ -556,6 +556,34 @@ def grouped_stream_combine(a: torch.Tensor, wt: torch.Tensor, r: "MoERouting", T
     return out
 
 
+def grouped_wide(x: torch.Tensor, wt: torch.Tensor, r: "MoERouting", epilogue: str, gather: bool,
+                 out: torch.Tensor | None = None, limit: float = 0.0, alpha: float = 1.0) -> torch.Tensor:
+    """The expert products of a long step on wave-tiled expert weights (128-row tiles; K % 128 == 0, N % 64 == 0).
+    ``epilogue``: "glu" (``tile_experts(w13, glu=True)``; silu(gate) * up, or with a limit the clamped form, [n_ent,
+    N/2]), "relu2" (relu squared, [n_ent, N]) or "combine" (out[token] += w * row, out f32 [T, N] zeroed by the caller).
+    ``gather``: rows are x[token of the entry], else x[entry]."""
+    n_ent = r.perm_tok.numel()
+    N = wt.shape[1] * 32
+    y = None
+    if epilogue != "combine":
+        y = torch.empty(n_ent, N // 2 if epilogue == "glu" else N, dtype=x.dtype, device=x.device)
+    if _gpu(x):
+        ext().grouped_wide(x, wt, r.perm_tok, r.perm_w, r.expert_off, bool(gather),
+                           ("glu", "relu2", "combine").index(epilogue), y, out, float(limit), float(alpha))
+        return out if y is None else y
+    if epilogue == "combine":
+        ref.grouped_gemm(x, untile_experts(wt), r.perm_tok, r.perm_w, r.expert_off, 0, gather, None, out)
+        return out
+    h = ref_grouped(x, untile_experts(wt, glu=epilogue == "glu"), r, 0, gather).float()
+    F = N // 2
+    if epilogue == "relu2":
+        return y.copy_(h.relu().square())
+    if limit > 0:
+        g, u = h[:, :F].clamp(max=limit), h[:, F:].clamp(min=-limit, max=limit)
+        return y.copy_(g * torch.sigmoid(alpha * g) * (u + 1.0))
+    return y.copy_(torch.nn.functional.silu(h[:, :F]) * h[:, F:])
+
+
 def ref_grouped(x, w, r, e_lo, gather):
     y = torch.zeros(r.perm_tok.numel(), w.shape[1], dtype=x.dtype)
     ref.grouped_gemm(x, w, r.perm_tok, r.perm_w, r.expert_off, e_lo, gather, y, None)

@@ -82,6 +82,19 @@ hipError_t kafka_launch_wstream_grouped(const bf16* X, int64_t ldx, const bf16* 
 hipError_t kafka_launch_moe_route(const bf16* logits, int64_t ld, int T, int E, int K, int BM, float* topk_w,
                                   int* topk_e, int* perm_tok, float* perm_w, int* expert_off, int* tile_off,
                                   hipStream_t st);
+int kafka_moe_sort_max_e();
+hipError_t kafka_launch_moe_sort(const float* topk_w, const int* topk_e, int n, int k, int E, int bm, int* perm_tok,
+                                 float* perm_w, int* expert_off, int* tile_off, hipStream_t st);
+hipError_t kafka_launch_grouped_wide(const bf16* X, int64_t ldx, const bf16* Wt, int E, int N, int K,
+                                     const int* perm_tok, const float* perm_w, const int* expert_off, int n_ent,
+                                     int gather, int epi, bf16* Y, int64_t ldy, float* out, int64_t ldo,
+                                     float glu_limit, float glu_alpha, hipStream_t st);
+int kafka_narrow_ok(int N, int K, int64_t xs);
+int kafka_narrow_max_k();
+hipError_t kafka_launch_narrow_linear(const bf16* x, int64_t xs, const bf16* w, const float* bias, int N, int K,
+                                      float* out, int64_t os, int64_t T, hipStream_t st);
+hipError_t kafka_launch_narrow_route(const bf16* x, int64_t xs, const bf16* w, int N, int K, int k, int norm, float scale,
+                                     float* tw, int* te, int64_t T, hipStream_t st);
 hipError_t kafka_launch_grouped_gemm(const bf16* X, int64_t ldx, const bf16* W, int N, int Kd, const int* perm_tok,
                                      const float* perm_w, const int* expert_off, const int* tile_off, int e_lo,
                                      int e_n, int max_tiles, int gather, bf16* Y, int64_t ldy, float* out,
@@ -739,6 +752,73 @@ static void wstream_grouped(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at
                                          relu2 ? 1 : 0, (float)glu_limit, (float)glu_alpha, cur_stream()));
 }
 
+// The same products for long steps (128 x 256 tiles; every expert of the routing resident). epi: 0 gate_up with silu * up
+// or its clamped form into y [n_ent, N/2], 1 relu squared into y [n_ent, N], 2 the weighted combine into out f32 [T, N].
+// Expert ids were in [0, E) when the entries were sorted, so perm_tok / expert_off stay inside x and wt.
+static void grouped_wide(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at::Tensor perm_w, at::Tensor expert_off,
+                         bool gather, int64_t epi, c10::optional<at::Tensor> y, c10::optional<at::Tensor> out,
+                         double glu_limit, double glu_alpha) {
+  CHECK_CUDA(x); CHECK_DT(x, at::kBFloat16); CHECK_DT(wt, at::kBFloat16); CHECK_LASTDIM(x);
+  CHECK_DT(perm_tok, at::kInt); CHECK_DT(perm_w, at::kFloat); CHECK_DT(expert_off, at::kInt);
+  TORCH_CHECK(x.dim() == 2 && x.stride(0) % 8 == 0 && (reinterpret_cast<uintptr_t>(x.data_ptr()) & 15) == 0,
+              "grouped_wide: x must be [rows, K] with 16-B rows");
+  TORCH_CHECK(wt.dim() == 5 && wt.is_contiguous() && wt.size(3) == 64 && wt.size(4) == 8,
+              "grouped_wide: wt must be contiguous [E, N/32, K/16, 64, 8]");
+  const int64_t E = wt.size(0), N = wt.size(1) * 32, K = wt.size(2) * 16, n_ent = perm_tok.numel();
+  TORCH_CHECK(x.size(1) == K && K % 128 == 0 && N % 64 == 0, "grouped_wide: K / N");
+  TORCH_CHECK(perm_w.numel() == n_ent && perm_tok.is_contiguous() && perm_w.is_contiguous() &&
+                  expert_off.is_contiguous() && expert_off.numel() == E + 1, "grouped_wide: routing of these experts");
+  TORCH_CHECK(gather || x.size(0) >= n_ent, "grouped_wide: one x row per entry");
+  TORCH_CHECK(epi >= 0 && epi <= 2 && (epi == 2) == out.has_value() && (epi != 2) == y.has_value(), "grouped_wide: epilogue");
+  bf16* yp = nullptr; int64_t ldy = 0; float* op = nullptr; int64_t ldo = 0;
+  if (epi == 2) {
+    CHECK_DT(out.value(), at::kFloat); CHECK_LASTDIM(out.value());
+    TORCH_CHECK(out->dim() == 2 && out->size(1) == N, "grouped_wide: out [T, N]");
+    op = out->data_ptr<float>(); ldo = out->stride(0);
+  } else {
+    CHECK_DT(y.value(), at::kBFloat16); CHECK_LASTDIM(y.value());
+    TORCH_CHECK(y->dim() == 2 && y->size(0) >= n_ent && y->size(1) == (epi == 0 ? N / 2 : N), "grouped_wide: y");
+    yp = bptr(y.value()); ldy = y->stride(0);
+  }
+  CHECK_HIP(kafka_launch_grouped_wide(bptr(x), x.stride(0), bptr(wt), (int)E, (int)N, (int)K, perm_tok.data_ptr<int>(),
+                                      perm_w.data_ptr<float>(), expert_off.data_ptr<int>(), (int)n_ent, gather ? 1 : 0,
+                                      (int)epi, yp, ldy, op, ldo, (float)glu_limit, (float)glu_alpha, cur_stream()));
+}
+
+static void narrow_args(const at::Tensor& x, const at::Tensor& w) {
+  CHECK_CUDA(x); CHECK_DT(x, at::kBFloat16); CHECK_DT(w, at::kBFloat16); CHECK_LASTDIM(x);
+  TORCH_CHECK(x.dim() == 2 && w.dim() == 2 && w.is_cuda() && w.is_contiguous() && w.size(1) == x.size(1) &&
+                  (reinterpret_cast<uintptr_t>(x.data_ptr()) & 15) == 0 &&
+                  (reinterpret_cast<uintptr_t>(w.data_ptr()) & 15) == 0 &&
+                  kafka_narrow_ok((int)w.size(0), (int)w.size(1), x.stride(0)), "narrow product: sizes");
+}
+
+// out fp32 [T, N] = x w^T (+ bias) for up to 64 rows of w
+static void narrow_linear(at::Tensor x, at::Tensor w, c10::optional<at::Tensor> bias, at::Tensor out) {
+  narrow_args(x, w);
+  const int64_t T = x.size(0), N = w.size(0);
+  CHECK_DT(out, at::kFloat); CHECK_LASTDIM(out);
+  TORCH_CHECK(out.dim() == 2 && out.size(0) == T && out.size(1) == N, "narrow_linear: out [T, N]");
+  if (bias.has_value()) {
+    CHECK_DT(bias.value(), at::kFloat);
+    TORCH_CHECK(bias->is_cuda() && bias->is_contiguous() && bias->numel() == N, "narrow_linear: bias [N]");
+  }
+  CHECK_HIP(kafka_launch_narrow_linear(bptr(x), x.stride(0), bptr(w), bias.has_value() ? bias->data_ptr<float>() : nullptr,
+                                       (int)N, (int)w.size(1), out.data_ptr<float>(), out.stride(0), T, cur_stream()));
+}
+
+// softmax of x w^T over all rows of w, the k largest with their scores
+static void narrow_route(at::Tensor x, at::Tensor w, bool norm, double scale, at::Tensor tw, at::Tensor te) {
+  narrow_args(x, w);
+  const int64_t T = x.size(0), N = w.size(0);
+  CHECK_DT(tw, at::kFloat); CHECK_DT(te, at::kInt);
+  TORCH_CHECK(tw.dim() == 2 && tw.is_contiguous() && te.is_contiguous() && te.sizes() == tw.sizes() && tw.size(0) == T &&
+                  tw.size(1) >= 1 && tw.size(1) <= N && tw.size(1) <= kafka_narrow_max_k(), "narrow_route: choices [T, k]");
+  CHECK_HIP(kafka_launch_narrow_route(bptr(x), x.stride(0), bptr(w), (int)N, (int)w.size(1), (int)tw.size(1),
+                                      norm ? 1 : 0, (float)scale, tw.data_ptr<float>(), te.data_ptr<int>(), T,
+                                      cur_stream()));
+}
+
 // y [M, N] bf16 = sum over the slabs p [S, M, N]
 static void slab_reduce(at::Tensor p, at::Tensor y) {
   CHECK_CUDA(p); CHECK_DT(p, at::kFloat); CHECK_DT(y, at::kBFloat16); CHECK_LASTDIM(y);
@@ -780,6 +860,12 @@ static void moe_sort(at::Tensor topk_w, at::Tensor topk_e, int64_t E, int64_t bm
   TORCH_CHECK(perm_tok.numel() == T * k && perm_w.numel() == T * k && expert_off.numel() == E + 1 &&
                   tile_off.numel() == E + 1 && perm_tok.is_contiguous() && perm_w.is_contiguous(),
               "moe_sort: output sizes");
+  if (E <= kafka_moe_sort_max_e() && T * k < (int64_t)1 << 30) {
+    CHECK_HIP(kafka_launch_moe_sort(topk_w.data_ptr<float>(), topk_e.data_ptr<int>(), (int)(T * k), (int)k, (int)E,
+                                    (int)bm, perm_tok.data_ptr<int>(), perm_w.data_ptr<float>(),
+                                    expert_off.data_ptr<int>(), tile_off.data_ptr<int>(), cur_stream()));
+    return;
+  }
   CHECK_HIP(kafka_launch_moe_route(nullptr, 0, (int)T, (int)E, (int)k, (int)bm, topk_w.data_ptr<float>(),
                                    topk_e.data_ptr<int>(), perm_tok.data_ptr<int>(), perm_w.data_ptr<float>(),
                                    expert_off.data_ptr<int>(), tile_off.data_ptr<int>(), cur_stream()));
@@ -1063,6 +1149,10 @@ PYBIND11_MODULE(_kafka_ops, m) {
   m.def("ep_dispatch", &ep_dispatch);
   m.def("ep_recv_route", &ep_recv_route);
   m.def("ep_combine", &ep_combine);
+  m.def("grouped_wide", &grouped_wide);
+  m.def("narrow_linear", &narrow_linear);
+  m.def("narrow_route", &narrow_route);
+  m.def("narrow_ok", [](int N, int K, int64_t xs) { return kafka_narrow_ok(N, K, xs) != 0; });
   m.def("grouped_gemm", &grouped_gemm, py::arg("x"), py::arg("w"), py::arg("perm_tok"), py::arg("perm_w"),
         py::arg("expert_off"), py::arg("tile_off"), py::arg("e_lo"), py::arg("max_tiles"), py::arg("gather"),
         py::arg("y"), py::arg("out"), py::arg("relu2") = false);

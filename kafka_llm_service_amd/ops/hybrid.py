@@ -442,7 +442,8 @@ def moe_rows(h, w_gu, w_down, topk_w, topk_e, out, act: str = "silu", limit: flo
         ref.moe_rows(h, w_gu, w_down, topk_w, topk_e, out, lim, al, glu)
 
 
-MOE_STREAM_MAX_T = 640  # steps of up to this many rows run tiled expert weights on the grouped streaming kernel
+MOE_STREAM_MAX_T = 640  # steps of up to this many rows run tiled expert weights on the grouped streaming kernel, longer
+                        # ones on the wide one (ops.grouped_wide)
 
 
 def moe_grouped_ok(h, w_gu, w_down, glu: bool = True) -> bool:
@@ -457,9 +458,9 @@ def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None
     """out (fp32 [T, d]) = the routed experts' weighted sum for every row. Sizes the framework's expert-sorted
     matrix-core kernels take (bf16) go through them - entries sorted by expert (``ops.moe_sort``), gate/up GEMM on
     gathered rows, silu * up, down GEMM with the weighted combine in its epilogue (fp32 adds, two entries per row
-    commute), or the grouped weight-streaming kernels when tiled expert weights are given and the step is small -
-    everything else is evaluated per (row, expert) pair by ``moe_rows``. ``act`` as in ``moe_rows`` (the streaming
-    kernel applies it in its epilogue; between the two expert-sorted GEMMs it is a launch of its own, "relu2" is part
+    commute), or with tiled expert weights the grouped weight-streaming kernels (steps of few rows) and the wide ones -
+    everything else is evaluated per (row, expert) pair by ``moe_rows``. ``act`` as in ``moe_rows`` (the kernels on tiled
+    weights apply it in their epilogue; between the two expert-sorted GEMMs it is a launch of its own, "relu2" is part
     of the first)."""
     from kafka_llm_service_amd import ops
 
@@ -468,13 +469,15 @@ def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None
     if T and moe_grouped_ok(h, w_gu, w_down, glu):
         r = ops.moe_sort(topk_w, topk_e, w_gu.shape[0])
         out.zero_()
-        if w_gu_t is not None and w_down_t is not None and T <= MOE_STREAM_MAX_T:
-            if glu:
-                lim, al = _glu_act(act, limit, alpha)
-                a = ops.grouped_stream_glu(h, w_gu_t, r, limit=lim, alpha=al)
+        if w_gu_t is not None and w_down_t is not None:
+            lim, al = _glu_act(act, limit, alpha) if glu else (0.0, 1.0)
+            if T > MOE_STREAM_MAX_T:
+                a = ops.grouped_wide(h, w_gu_t, r, "glu" if glu else "relu2", True, limit=lim, alpha=al)
+                ops.grouped_wide(a, w_down_t, r, "combine", False, out)
             else:
-                a = ops.grouped_stream_relu2(h, w_gu_t, r)
-            ops.grouped_stream_combine(a, w_down_t, r, T, out)
+                a = ops.grouped_stream_glu(h, w_gu_t, r, limit=lim, alpha=al) if glu else \
+                    ops.grouped_stream_relu2(h, w_gu_t, r)
+                ops.grouped_stream_combine(a, w_down_t, r, T, out)
         elif not glu:
             a = ops.grouped_gemm(h, w_gu, r, gather=True, relu2=True)
             ops.grouped_gemm(a, w_down, r, gather=False, combine_out=out)
@@ -620,14 +623,17 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
 
 
 def moe_router_grouped(h, w, correction, k: int, groups: int, keep: int, eps: float = 0.0, extra_gate: bool = False,
-                       score: str = "softmax", group_score: str = "max", norm: bool = True, scale: float = 1.0):
+                       score: str = "softmax", group_score: str = "max", norm: bool = True, scale: float = 1.0,
+                       w_act=None):
     """Group-limited router: fp32 logits h W^T over the first E rows of ``w`` (fp32 [E (+ 1), d]); s = softmax over
     all E or (``score`` "sigmoid") sigmoid of each; the choice looks at s + correction (None: at s), only within the
     ``keep`` groups (of ``groups`` equal groups of neighbouring experts) with the largest group score - the largest
     value of a group, or (``group_score`` "top2") the sum of its two largest - and takes the k largest there (ties:
     the lower index); the weights are s of the chosen, divided by (their sum + eps) unless ``norm`` is off, times
     ``scale``. With ``extra_gate`` the last row of ``w`` is a gate vector and sigmoid of its product is returned per
-    row. Returns (weights fp32 [T, k], experts int32 [T, k], gate fp32 [T] or None)."""
+    row. Returns (weights fp32 [T, k], experts int32 [T, k], gate fp32 [T] or None).
+    ``w_act``: the same weights in h's dtype when they are exact in it - then a plain choice (softmax, no groups, no
+    correction) of up to 64 experts is one kernel, product included (bf16 products, fp32 sums: the same logits)."""
     T = h.shape[0]
     E = w.shape[0] - (1 if extra_gate else 0)
     if E < 1 or groups < 1 or E % groups or not 1 <= keep <= groups or not 1 <= k <= keep * (E // groups):
@@ -639,7 +645,10 @@ def moe_router_grouped(h, w, correction, k: int, groups: int, keep: int, eps: fl
     tw = torch.empty(T, k, dtype=torch.float32, device=h.device)
     te = torch.empty(T, k, dtype=torch.int32, device=h.device)
     gate = torch.empty(T, dtype=torch.float32, device=h.device) if extra_gate else None
-    if _gpu(h):
+    if w_act is not None and groups == 1 and correction is None and gate is None and score == "softmax" and eps == 0.0 \
+            and narrow_ok(h, w_act) and k <= 16:
+        ext().narrow_route(h, w_act, bool(norm), float(scale), tw, te)
+    elif _gpu(h):
         # logits as one full-precision fp32 matrix product (the engine switches reduced-precision matrix modes off),
         # then the choice kernel
         ext().hy_moe_topk_grouped(torch.mm(h.float(), w.t()), int(E), correction, int(groups), int(keep), float(eps),
@@ -833,10 +842,20 @@ def add_tanh_norm(x, y1=None, y2=None, norms=(), outs=(), copy=None, assign: boo
         ref.add_tanh_norm(x, y1, y2, norms, outs, copy, assign)
 
 
-def linear_f32(x, w) -> torch.Tensor:
-    """x @ w^T with an fp32 result for operands in the activation dtype (one matrix product, nothing rounded to it)."""
-    if x.dtype == torch.float32:
-        return torch.nn.functional.linear(x, w)
-    if _gpu(x):
-        return torch.mm(x, w.t(), out_dtype=torch.float32)
-    return torch.nn.functional.linear(x.float(), w.float())
+def narrow_ok(x, w) -> bool:
+    """bf16 GPU operands of the kernel for products with few weight rows (up to 64, K a multiple of 32)."""
+    return x.is_cuda and x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and x.data_ptr() % 16 == 0 and \
+        bool(ext().narrow_ok(w.shape[0], w.shape[1], x.stride(0)))
+
+
+def linear_f32(x, w, bias=None) -> torch.Tensor:
+    """x @ w^T (+ bias fp32) with an fp32 result for operands in the activation dtype: one matrix product, nothing rounded
+    to it. Few weight rows (gate projections) have a kernel of their own."""
+    if _gpu(x) and x.dtype == torch.bfloat16:
+        if narrow_ok(x, w):
+            out = torch.empty(x.shape[0], w.shape[0], dtype=torch.float32, device=x.device)
+            ext().narrow_linear(x, w, bias, out)
+            return out
+        y = torch.mm(x, w.t(), out_dtype=torch.float32)
+        return y if bias is None else y.add_(bias)
+    return torch.nn.functional.linear(x.float(), w.float(), bias)

@@ -591,15 +591,89 @@ def test_experts_on_the_matrix_cores(E, k, T):
         assert close(r, want, 0.02)
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("n_exp,k,T", [(1, 1, 3), (3, 2, 5), (16, 4, 64), (16, 4, 2048), (70, 8, 333), (512, 16, 700),
+                                       (8, 2, 8192)])
+def test_sort_by_expert(n_exp, k, T):
+    """Entries by expert, in token order inside an expert; experts without entries, stretches that end inside a wave."""
+    from kafka_llm_service_amd import ops
+
+    g = torch.Generator().manual_seed(T)
+    te = torch.stack([torch.randperm(n_exp, generator=g)[:k] for _ in range(T)]).int()
+    if n_exp > 8:
+        te[:, 0] = torch.where(te[:, 0] == 5, (te[:, 1] + 1) % n_exp, te[:, 0])
+        te[T // 2:, 1] = 7
+    tw = torch.rand(T, k, generator=g)
+    a, b = ops.moe_sort(tw.cuda(), te.cuda(), n_exp), ops.moe_sort(tw, te, n_exp)
+    for n in ("perm_tok", "perm_w", "expert_off", "tile_off"):
+        assert torch.equal(getattr(a, n).cpu(), getattr(b, n)), n
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("E,k,T,d,ff", [(6, 3, 700, 256, 256), (3, 1, 130, 512, 320), (70, 8, 900, 128, 64),
+                                        (2, 2, 1000, 384, 576)])
+def test_wide_expert_products(E, k, T, d, ff):
+    """The kernels for long steps on tiled weights, every epilogue against the CPU functions: row tiles that end inside an
+    expert, experts without rows, column tiles that end inside a workgroup."""
+    from kafka_llm_service_amd import ops
+
+    g = torch.Generator().manual_seed(E)
+    te = torch.stack([torch.randperm(E, generator=g)[:k] for _ in range(T)]).int()
+    if E > 4:
+        te[te == 2] = 3
+    tw = torch.rand(T, k, generator=g)
+    h = torch.randn(T, d, generator=g).to(torch.bfloat16)
+    gu = (torch.randn(E, 2 * ff, d, generator=g) / d ** 0.5).to(torch.bfloat16)
+    down = (torch.randn(E, 128, 2 * ff, generator=g) / ff ** 0.5).to(torch.bfloat16)
+    r, rc = ops.moe_sort(tw.cuda(), te.cuda(), E), ops.moe_sort(tw, te, E)
+    gd, dd = gu.cuda(), down.cuda()
+    for kw in ({}, {"limit": 1.5, "alpha": 1.7}):
+        a = ops.grouped_wide(h.cuda(), ops.tile_experts(gd, glu=True), r, "glu", True, **kw)
+        assert close(a.float(), ops.grouped_wide(h, ops.tile_experts(gu, glu=True), rc, "glu", True, **kw).float(), 1e-2)
+    a = ops.grouped_wide(h.cuda(), ops.tile_experts(gd), r, "relu2", True)
+    ac = ops.grouped_wide(h, ops.tile_experts(gu), rc, "relu2", True)
+    assert close(a.float(), ac.float(), 1e-2)
+    if 2 * ff % 128 == 0:
+        out, oc = torch.zeros(T, 128, device="cuda"), torch.zeros(T, 128)
+        ops.grouped_wide(a, ops.tile_experts(dd), r, "combine", False, out)
+        ops.grouped_wide(a.cpu(), ops.tile_experts(down), rc, "combine", False, oc)
+        assert close(out, oc, 1e-2)
+
+
 @pytest.mark.parametrize("device", DEVICES)
 def test_products_with_fp32_results(device):
+    """Few weight rows (their own kernel in bf16) and many, with and without a bias."""
     g = torch.Generator().manual_seed(1)
-    for M, N, K in ((1, 8, 16), (5, 256, 64), (300, 40, 96)):
-        x, w = torch.randn(M, K, generator=g), torch.randn(N, K, generator=g)
+    for M, N, K in ((1, 8, 16), (5, 256, 64), (300, 40, 96), (16, 64, 1024), (17, 3, 32), (33, 17, 4096), (2, 1, 64)):
+        x, w, b = torch.randn(M, K, generator=g), torch.randn(N, K, generator=g), torch.randn(N, generator=g)
         for dt in (torch.float32, torch.bfloat16):
-            a, b = x.to(dt), w.to(dt)
-            y = hops.linear_f32(a.to(device), b.to(device))
-            assert y.dtype == torch.float32 and close(y, a.double() @ b.double().T, 1e-6)
+            a, c = x.to(dt), w.to(dt)
+            for bias in (None, b):
+                y = hops.linear_f32(a.to(device), c.to(device), None if bias is None else bias.to(device))
+                want = a.double() @ c.double().T + (0.0 if bias is None else b.double())
+                assert y.dtype == torch.float32 and close(y, want, 2e-6)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("E,k,d,T", [(16, 4, 256, 70), (1, 1, 32, 3), (64, 16, 96, 33), (37, 5, 512, 1), (16, 16, 64, 16),
+                                     (48, 8, 4096, 40)])
+def test_router_with_its_product(E, k, d, T):
+    """The router in one kernel against the two-step form and the plain function: ties take the lower index, weights as they
+    are, normalised and scaled."""
+    g = torch.Generator().manual_seed(E)
+    h = torch.randn(T, d, generator=g).to(torch.bfloat16)
+    w = (2.0 * torch.randn(E, d, generator=g) / d ** 0.5).to(torch.bfloat16)
+    if E > 8:
+        w[7] = w[3]
+    hd, wd = h.cuda(), w.cuda()
+    assert hops.narrow_ok(hd, wd)
+    want = plain.route(h.double() @ w.double().T, k)
+    for norm, scale in ((False, 1.0), (True, 2.5)):
+        tw, te, _ = hops.moe_router_grouped(hd, wd.float(), None, k, 1, 1, norm=norm, scale=scale, w_act=wd)
+        t2, e2, _ = hops.moe_router_grouped(hd, wd.float(), None, k, 1, 1, norm=norm, scale=scale)
+        got = torch.zeros(T, E, dtype=torch.float64).scatter_(1, te.long().cpu(), tw.double().cpu())
+        ref = want * scale / (want.sum(-1, keepdim=True) if norm else 1.0)
+        assert close(got, ref, 1e-5) and close(tw, t2.cpu(), 1e-5) and (te == e2).float().mean() > 0.99
 
 
 # ---- the model in the engine ---------------------------------------------------------------------------------------
