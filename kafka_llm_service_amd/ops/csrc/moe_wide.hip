@@ -12,8 +12,8 @@
 //   moe_sort       stable sort of (token, choice) entries by expert, one workgroup: every wave counts and then places
 //                  its stretch of the entries 64 at a time, equal experts found by ballots over the bits of their ids
 //   narrow         fp32 products of bf16 rows with up to 64 bf16 weight rows (router logits, gate projections): 16 rows a
-//                  workgroup, the waves split K, 16x16x32 products; with a bias, or followed in place by the choice of
-//                  the k largest scores
+//                  workgroup, its 16 (or 8) waves split K, 16x16x32 products; with a bias, or followed in place by the
+//                  choice of the k largest scores, a wave per row
 #include "common.h"
 
 namespace kafka {
@@ -288,17 +288,19 @@ __global__ __launch_bounds__(SORT_NT) void moe_sort_kernel(const float* __restri
 
 // ---- narrow products --------------------------------------------------------------------------------------------------
 constexpr int NR_ROWS = 16, NR_MAXN = 64, NR_MAXK = 16;
-constexpr int NR_LD = NR_MAXN + 1;
+// waves of a workgroup and row length of their parts in LDS, TN: tiles of 16 weight rows
+__host__ __device__ constexpr int nr_waves(int TN) { return TN <= 2 ? 16 : 8; }
+__host__ __device__ constexpr int nr_ld(int TN) { return 16 * TN + 1; }
 typedef float f32x4v __attribute__((ext_vector_type(4)));
 
 __device__ __forceinline__ f32x4v mfma16(bf16x8 a, bf16x8 b, f32x4v c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
 
-// z[row][n] = x[row] . w[n] for 16 rows, the waves' parts summed through LDS: part [4][16][NR_LD] -> z in part[0]
+// z[row][n] = x[row] . w[n] for 16 rows, the waves' parts summed through LDS -> z in part[0]
 template <int TN>
 __device__ __forceinline__ void narrow_product(const bf16* __restrict__ x, int64_t xs, int64_t T, const bf16* __restrict__ wt,
-                                               int N, int K, float (*part)[NR_ROWS][NR_LD]) {
+                                               int N, int K, float (*part)[NR_ROWS][nr_ld(TN)]) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r = lane & 15, q = lane >> 4;
   const int64_t t = min((int64_t)blockIdx.x * NR_ROWS + r, T - 1);
   const bf16* xp = x + t * xs + 8 * q;
@@ -310,7 +312,8 @@ __device__ __forceinline__ void narrow_product(const bf16* __restrict__ x, int64
   for (int j = 0; j < TN; ++j) acc[j] = f32x4v{0.f, 0.f, 0.f, 0.f};
   constexpr int PF = TN <= 2 ? 8 : 4;              // steps in flight
   const int ns = K / 32;
-  for (int s0 = w * PF; s0 < ns; s0 += 4 * PF) {
+  constexpr int NW = nr_waves(TN);
+  for (int s0 = w * PF; s0 < ns; s0 += NW * PF) {
     bf16x8 a[PF], b[PF][TN];
 #pragma unroll
     for (int p = 0; p < PF; ++p) {
@@ -333,21 +336,24 @@ __device__ __forceinline__ void narrow_product(const bf16* __restrict__ x, int64
 #pragma unroll
     for (int i = 0; i < 4; ++i) part[w][4 * q + i][16 * j + r] = acc[j][i];
   __syncthreads();
-  for (int i = threadIdx.x; i < NR_ROWS * 16 * TN; i += 256) {
+  for (int i = threadIdx.x; i < NR_ROWS * 16 * TN; i += 64 * NW) {
     const int row = i / (16 * TN), n = i - row * 16 * TN;
-    part[0][row][n] = (part[0][row][n] + part[1][row][n]) + (part[2][row][n] + part[3][row][n]);
+    float z = 0.f;
+#pragma unroll
+    for (int k = 0; k < NW; ++k) z += part[k][row][n];
+    part[0][row][n] = z;
   }
   __syncthreads();
 }
 
 template <int TN>
-__global__ __launch_bounds__(256) void narrow_linear_kernel(const bf16* __restrict__ x, int64_t xs,
+__global__ __launch_bounds__(64 * nr_waves(TN)) void narrow_linear_kernel(const bf16* __restrict__ x, int64_t xs,
                                                             const bf16* __restrict__ wt, const float* __restrict__ bias,
                                                             int N, int K, float* __restrict__ out, int64_t os,
                                                             int64_t T) {
-  __shared__ float part[4][NR_ROWS][NR_LD];
+  __shared__ float part[nr_waves(TN)][NR_ROWS][nr_ld(TN)];
   narrow_product<TN>(x, xs, T, wt, N, K, part);
-  for (int i = threadIdx.x; i < NR_ROWS * N; i += 256) {
+  for (int i = threadIdx.x; i < NR_ROWS * N; i += 64 * nr_waves(TN)) {
     const int row = i / N, n = i - row * N;
     const int64_t t = (int64_t)blockIdx.x * NR_ROWS + row;
     if (t < T) out[t * os + n] = part[0][row][n] + (bias != nullptr ? bias[n] : 0.f);
@@ -355,17 +361,17 @@ __global__ __launch_bounds__(256) void narrow_linear_kernel(const bf16* __restri
 }
 
 // softmax over all N experts, the k largest (ties: the lower index), their scores as weights (norm: divided by their sum)
-// times scale; a wave takes four rows, lane = expert
+// times scale; lane = expert
 template <int TN>
-__global__ __launch_bounds__(256) void narrow_route_kernel(const bf16* __restrict__ x, int64_t xs,
+__global__ __launch_bounds__(64 * nr_waves(TN)) void narrow_route_kernel(const bf16* __restrict__ x, int64_t xs,
                                                            const bf16* __restrict__ wt, int N, int K, int k, bool norm,
                                                            float scale, float* __restrict__ tw, int* __restrict__ te,
                                                            int64_t T) {
-  __shared__ float part[4][NR_ROWS][NR_LD];
+  __shared__ float part[nr_waves(TN)][NR_ROWS][nr_ld(TN)];
   narrow_product<TN>(x, xs, T, wt, N, K, part);
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
 #pragma unroll 1
-  for (int row = 4 * w; row < 4 * w + 4; ++row) {
+  for (int row = w; row < NR_ROWS; row += nr_waves(TN)) {
     const int64_t t = (int64_t)blockIdx.x * NR_ROWS + row;
     if (t >= T) break;   // (uniform)
     const float z = lane < N ? part[0][row][lane] : -INFINITY;
@@ -451,11 +457,11 @@ hipError_t kafka_launch_narrow_linear(const bf16* x, int64_t xs, const bf16* w, 
   if (T <= 0) return hipSuccess;
   if (!kafka_narrow_ok(N, K, xs)) return hipErrorInvalidValue;
   const unsigned g = (unsigned)((T + NR_ROWS - 1) / NR_ROWS);
-  auto a = [&](auto kern) { kern<<<g, 256, 0, st>>>(x, xs, w, bias, N, K, out, os, T); };
-  if (N <= 16) a(narrow_linear_kernel<1>);
-  else if (N <= 32) a(narrow_linear_kernel<2>);
-  else if (N <= 48) a(narrow_linear_kernel<3>);
-  else a(narrow_linear_kernel<4>);
+  auto a = [&](auto kern, int tn) { kern<<<g, 64 * nr_waves(tn), 0, st>>>(x, xs, w, bias, N, K, out, os, T); };
+  if (N <= 16) a(narrow_linear_kernel<1>, 1);
+  else if (N <= 32) a(narrow_linear_kernel<2>, 2);
+  else if (N <= 48) a(narrow_linear_kernel<3>, 3);
+  else a(narrow_linear_kernel<4>, 4);
   return hipGetLastError();
 }
 
@@ -464,11 +470,13 @@ hipError_t kafka_launch_narrow_route(const bf16* x, int64_t xs, const bf16* w, i
   if (T <= 0) return hipSuccess;
   if (!kafka_narrow_ok(N, K, xs) || k < 1 || k > N || k > NR_MAXK) return hipErrorInvalidValue;
   const unsigned g = (unsigned)((T + NR_ROWS - 1) / NR_ROWS);
-  auto a = [&](auto kern) { kern<<<g, 256, 0, st>>>(x, xs, w, N, K, k, norm != 0, scale, tw, te, T); };
-  if (N <= 16) a(narrow_route_kernel<1>);
-  else if (N <= 32) a(narrow_route_kernel<2>);
-  else if (N <= 48) a(narrow_route_kernel<3>);
-  else a(narrow_route_kernel<4>);
+  auto a = [&](auto kern, int tn) {
+    kern<<<g, 64 * nr_waves(tn), 0, st>>>(x, xs, w, N, K, k, norm != 0, scale, tw, te, T);
+  };
+  if (N <= 16) a(narrow_route_kernel<1>, 1);
+  else if (N <= 32) a(narrow_route_kernel<2>, 2);
+  else if (N <= 48) a(narrow_route_kernel<3>, 3);
+  else a(narrow_route_kernel<4>, 4);
   return hipGetLastError();
 }
 

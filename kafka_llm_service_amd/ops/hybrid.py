@@ -442,8 +442,10 @@ def moe_rows(h, w_gu, w_down, topk_w, topk_e, out, act: str = "silu", limit: flo
         ref.moe_rows(h, w_gu, w_down, topk_w, topk_e, out, lim, al, glu)
 
 
-MOE_STREAM_MAX_T = 640  # steps of up to this many rows run tiled expert weights on the grouped streaming kernel, longer
-                        # ones on the wide one (ops.grouped_wide)
+# tiled expert weights: steps of up to MOE_STREAM_MAX_T rows with fewer than MOE_WIDE_ROWS rows per expert on average run
+# on the grouped streaming kernel, the others on the wide one (ops.grouped_wide)
+MOE_STREAM_MAX_T = 640
+MOE_WIDE_ROWS = 112
 
 
 def moe_grouped_ok(h, w_gu, w_down, glu: bool = True) -> bool:
@@ -471,7 +473,7 @@ def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None
         out.zero_()
         if w_gu_t is not None and w_down_t is not None:
             lim, al = _glu_act(act, limit, alpha) if glu else (0.0, 1.0)
-            if T > MOE_STREAM_MAX_T:
+            if T > MOE_STREAM_MAX_T or T * topk_e.shape[1] >= MOE_WIDE_ROWS * w_gu.shape[0]:
                 a = ops.grouped_wide(h, w_gu_t, r, "glu" if glu else "relu2", True, limit=lim, alpha=al)
                 ops.grouped_wide(a, w_down_t, r, "combine", False, out)
             else:
