@@ -23,7 +23,7 @@ Experts           router logits in fp32, softmax over all of them, the ``top`` l
 
 How the engine runs it. A layer's projections of norm1(x) are one GEMM. The add to the residual, both norms of the next
 layer and, in front of a pass, the residual's copy into the loop product's input are one element-wise kernel, which also
-sums a split-K projection's slabs. The head gates are applied by the attention kernels as they write their output. The
+sums a split-K projection's slabs and, in long steps, gathers every token's expert rows. The head gates are applied by the attention kernels as they write their output. The
 squared relu is part of the expert products. Long portions run the matrix memory in chunks of matrix products.
 
 Per sequence the engine keeps, for every layer RUN (a looped layer counts once per pass), pages (keys and page-wise
@@ -527,12 +527,14 @@ class FurapelLM:
         hops.head_norm_gate(o, lw.mnorm, proj, 2 * H * D + H * Dv, H, self.cfg.norm_eps, on)
         return self._lin(on, lw.o, getattr(lw, "o_t", None), slabs=True)
 
-    def _experts(self, lw, h) -> torch.Tensor:
-        """The routed experts' weighted sum, fp32 [T, d]."""
+    def _experts(self, lw, h):
+        """The routed experts' weighted sum, fp32 [T, d], or of a long step its rows (``hops.ExpertRows``)."""
         tw, te, _ = hops.moe_router_grouped(h, lw.router, None, lw.top, 1, 1, norm=False, w_act=lw.router_a)
-        out = torch.empty(h.shape[0], self.cfg.hidden_size, dtype=torch.float32, device=self.device)
-        hops.moe_experts(h, lw.w_up, lw.w_down, tw, te, out, getattr(lw, "w_up_t", None), getattr(lw, "w_down_t", None),
-                         act="relu2")
+        T, up_t, down_t = h.shape[0], getattr(lw, "w_up_t", None), getattr(lw, "w_down_t", None)
+        if up_t is not None and hops.moe_wide(T, lw.top, lw.E):
+            return hops.moe_expert_rows(h, up_t, down_t, tw, te, lw.E)
+        out = torch.empty(T, self.cfg.hidden_size, dtype=torch.float32, device=self.device)
+        hops.moe_experts(h, lw.w_up, lw.w_down, tw, te, out, up_t, down_t, act="relu2")
         return out
 
 

@@ -560,7 +560,8 @@ def grouped_wide(x: torch.Tensor, wt: torch.Tensor, r: "MoERouting", epilogue: s
                  out: torch.Tensor | None = None, limit: float = 0.0, alpha: float = 1.0) -> torch.Tensor:
     """The expert products of a long step on wave-tiled expert weights (128-row tiles; K % 128 == 0, N % 64 == 0).
     ``epilogue``: "glu" (``tile_experts(w13, glu=True)``; silu(gate) * up, or with a limit the clamped form, [n_ent,
-    N/2]), "relu2" (relu squared, [n_ent, N]) or "combine" (out[token] += w * row, out f32 [T, N] zeroed by the caller).
+    N/2]), "relu2" (relu squared, [n_ent, N]), "combine" (out[token] += w * row, out f32 [T, N] zeroed by the caller) or
+    "rows" (w * row, [n_ent, N], entry order).
     ``gather``: rows are x[token of the entry], else x[entry]."""
     n_ent = r.perm_tok.numel()
     N = wt.shape[1] * 32
@@ -569,7 +570,7 @@ def grouped_wide(x: torch.Tensor, wt: torch.Tensor, r: "MoERouting", epilogue: s
         y = torch.empty(n_ent, N // 2 if epilogue == "glu" else N, dtype=x.dtype, device=x.device)
     if _gpu(x):
         ext().grouped_wide(x, wt, r.perm_tok, r.perm_w, r.expert_off, bool(gather),
-                           ("glu", "relu2", "combine").index(epilogue), y, out, float(limit), float(alpha))
+                           ("glu", "relu2", "combine", "rows").index(epilogue), y, out, float(limit), float(alpha))
         return out if y is None else y
     if epilogue == "combine":
         ref.grouped_gemm(x, untile_experts(wt), r.perm_tok, r.perm_w, r.expert_off, 0, gather, None, out)
@@ -578,6 +579,8 @@ def grouped_wide(x: torch.Tensor, wt: torch.Tensor, r: "MoERouting", epilogue: s
     F = N // 2
     if epilogue == "relu2":
         return y.copy_(h.relu().square())
+    if epilogue == "rows":
+        return y.copy_(h * r.perm_w[:, None])
     if limit > 0:
         g, u = h[:, :F].clamp(max=limit), h[:, F:].clamp(min=-limit, max=limit)
         return y.copy_(g * torch.sigmoid(alpha * g) * (u + 1.0))
@@ -608,9 +611,10 @@ rope_cos_sin = ref.rope_cos_sin
 
 class MoERouting:
     """Device-side routing of one MoE layer (csrc/moe.hip ``moe_route``): everything the grouped GEMMs need."""
-    __slots__ = ("topk_w", "topk_e", "perm_tok", "perm_w", "expert_off", "tile_off", "num_experts", "max_tiles")
+    __slots__ = ("topk_w", "topk_e", "perm_tok", "perm_w", "expert_off", "tile_off", "num_experts", "max_tiles", "inv")
 
-    def __init__(self, topk_w, topk_e, perm_tok, perm_w, expert_off, tile_off, num_experts):
+    def __init__(self, topk_w, topk_e, perm_tok, perm_w, expert_off, tile_off, num_experts, inv=None):
+        self.inv = inv   # every entry's place in the sorted order [T, k] (moe_sort(inverse=True))
         self.topk_w, self.topk_e = topk_w, topk_e
         self.perm_tok, self.perm_w = perm_tok, perm_w
         self.expert_off, self.tile_off = expert_off, tile_off
@@ -638,18 +642,19 @@ def moe_route(logits: torch.Tensor, k: int) -> MoERouting:
     return MoERouting(tw, te, pt, pw, eo, to, E)
 
 
-def moe_sort(topk_w: torch.Tensor, topk_e: torch.Tensor, num_experts: int) -> MoERouting:
+def moe_sort(topk_w: torch.Tensor, topk_e: torch.Tensor, num_experts: int, inverse: bool = False) -> MoERouting:
     """MoERouting of entries routed elsewhere (weights fp32 [T, k], expert ids int32 [T, k]): the stable sort by expert
-    of ``moe_route`` alone, for any number of experts and choices."""
+    of ``moe_route`` alone, for any number of experts and choices. ``inverse``: also ``inv`` (up to 512 experts)."""
     T, k = topk_e.shape
     dev = topk_e.device
+    inv = torch.empty(T, k, dtype=torch.int32, device=dev) if inverse else None
     if _gpu(topk_e):
         pt = torch.empty(T * k, dtype=torch.int32, device=dev)
         pw = torch.empty(T * k, dtype=torch.float32, device=dev)
         eo = torch.empty(num_experts + 1, dtype=torch.int32, device=dev)
         to = torch.empty(num_experts + 1, dtype=torch.int32, device=dev)
-        ext().moe_sort(topk_w, topk_e, int(num_experts), GG_BM, pt, pw, eo, to)
-        return MoERouting(topk_w, topk_e, pt, pw, eo, to, num_experts)
+        ext().moe_sort(topk_w, topk_e, int(num_experts), GG_BM, pt, pw, eo, to, inv)
+        return MoERouting(topk_w, topk_e, pt, pw, eo, to, num_experts, inv)
     flat = topk_e.reshape(-1).long()
     perm = torch.argsort(flat, stable=True)
     counts = torch.bincount(flat, minlength=num_experts)
@@ -657,8 +662,10 @@ def moe_sort(topk_w: torch.Tensor, topk_e: torch.Tensor, num_experts: int) -> Mo
     eo[1:] = torch.cumsum(counts, 0)
     to = torch.zeros(num_experts + 1, dtype=torch.int32)
     to[1:] = torch.cumsum((counts + GG_BM - 1) // GG_BM, 0)
+    if inverse:
+        inv.view(-1)[perm] = torch.arange(T * k, dtype=torch.int32)
     return MoERouting(topk_w, topk_e, (perm // k).to(torch.int32), topk_w.reshape(-1)[perm].float(), eo, to,
-                      num_experts)
+                      num_experts, inv)
 
 
 def grouped_gemm(x: torch.Tensor, w: torch.Tensor, r: MoERouting, gather: bool, e_lo: int = 0,

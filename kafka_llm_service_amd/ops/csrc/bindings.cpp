@@ -84,7 +84,7 @@ hipError_t kafka_launch_moe_route(const bf16* logits, int64_t ld, int T, int E, 
                                   hipStream_t st);
 int kafka_moe_sort_max_e();
 hipError_t kafka_launch_moe_sort(const float* topk_w, const int* topk_e, int n, int k, int E, int bm, int* perm_tok,
-                                 float* perm_w, int* expert_off, int* tile_off, hipStream_t st);
+                                 float* perm_w, int* expert_off, int* tile_off, int* inv, hipStream_t st);
 hipError_t kafka_launch_grouped_wide(const bf16* X, int64_t ldx, const bf16* Wt, int E, int N, int K,
                                      const int* perm_tok, const float* perm_w, const int* expert_off, int n_ent,
                                      int gather, int epi, bf16* Y, int64_t ldy, float* out, int64_t ldo,
@@ -753,7 +753,8 @@ static void wstream_grouped(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at
 }
 
 // The same products for long steps (128 x 256 tiles; every expert of the routing resident). epi: 0 gate_up with silu * up
-// or its clamped form into y [n_ent, N/2], 1 relu squared into y [n_ent, N], 2 the weighted combine into out f32 [T, N].
+// or its clamped form into y [n_ent, N/2], 1 relu squared into y [n_ent, N], 2 the weighted combine into out f32 [T, N],
+// 3 the weighted rows into y [n_ent, N].
 // Expert ids were in [0, E) when the entries were sorted, so perm_tok / expert_off stay inside x and wt.
 static void grouped_wide(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at::Tensor perm_w, at::Tensor expert_off,
                          bool gather, int64_t epi, c10::optional<at::Tensor> y, c10::optional<at::Tensor> out,
@@ -769,7 +770,7 @@ static void grouped_wide(at::Tensor x, at::Tensor wt, at::Tensor perm_tok, at::T
   TORCH_CHECK(perm_w.numel() == n_ent && perm_tok.is_contiguous() && perm_w.is_contiguous() &&
                   expert_off.is_contiguous() && expert_off.numel() == E + 1, "grouped_wide: routing of these experts");
   TORCH_CHECK(gather || x.size(0) >= n_ent, "grouped_wide: one x row per entry");
-  TORCH_CHECK(epi >= 0 && epi <= 2 && (epi == 2) == out.has_value() && (epi != 2) == y.has_value(), "grouped_wide: epilogue");
+  TORCH_CHECK(epi >= 0 && epi <= 3 && (epi == 2) == out.has_value() && (epi != 2) == y.has_value(), "grouped_wide: epilogue");
   bf16* yp = nullptr; int64_t ldy = 0; float* op = nullptr; int64_t ldo = 0;
   if (epi == 2) {
     CHECK_DT(out.value(), at::kFloat); CHECK_LASTDIM(out.value());
@@ -848,9 +849,10 @@ static void moe_route(at::Tensor logits, int64_t k, int64_t bm, at::Tensor topk_
                                    expert_off.data_ptr<int>(), tile_off.data_ptr<int>(), cur_stream()));
 }
 
-// the sort of moe_route alone, for entries routed elsewhere (topk_w / topk_e [T, k] are inputs; expert ids in [0, E))
+// the sort of moe_route alone, for entries routed elsewhere (topk_w / topk_e [T, k] are inputs; expert ids in [0, E));
+// inv [T, k]: every entry's place in the sorted order
 static void moe_sort(at::Tensor topk_w, at::Tensor topk_e, int64_t E, int64_t bm, at::Tensor perm_tok,
-                     at::Tensor perm_w, at::Tensor expert_off, at::Tensor tile_off) {
+                     at::Tensor perm_w, at::Tensor expert_off, at::Tensor tile_off, c10::optional<at::Tensor> inv) {
   CHECK_CUDA(topk_w); CHECK_DT(topk_w, at::kFloat); CHECK_DT(perm_w, at::kFloat);
   CHECK_DT(topk_e, at::kInt); CHECK_DT(perm_tok, at::kInt); CHECK_DT(expert_off, at::kInt); CHECK_DT(tile_off, at::kInt);
   TORCH_CHECK(topk_w.dim() == 2 && topk_e.sizes() == topk_w.sizes() && topk_w.is_contiguous() && topk_e.is_contiguous(),
@@ -860,10 +862,17 @@ static void moe_sort(at::Tensor topk_w, at::Tensor topk_e, int64_t E, int64_t bm
   TORCH_CHECK(perm_tok.numel() == T * k && perm_w.numel() == T * k && expert_off.numel() == E + 1 &&
                   tile_off.numel() == E + 1 && perm_tok.is_contiguous() && perm_w.is_contiguous(),
               "moe_sort: output sizes");
+  int* ip = nullptr;
+  if (inv.has_value()) {
+    CHECK_DT(inv.value(), at::kInt);
+    TORCH_CHECK(inv->is_cuda() && inv->is_contiguous() && inv->numel() == T * k && E <= kafka_moe_sort_max_e(),
+                "moe_sort: inv [T, k], up to ", kafka_moe_sort_max_e(), " experts");
+    ip = inv->data_ptr<int>();
+  }
   if (E <= kafka_moe_sort_max_e() && T * k < (int64_t)1 << 30) {
     CHECK_HIP(kafka_launch_moe_sort(topk_w.data_ptr<float>(), topk_e.data_ptr<int>(), (int)(T * k), (int)k, (int)E,
                                     (int)bm, perm_tok.data_ptr<int>(), perm_w.data_ptr<float>(),
-                                    expert_off.data_ptr<int>(), tile_off.data_ptr<int>(), cur_stream()));
+                                    expert_off.data_ptr<int>(), tile_off.data_ptr<int>(), ip, cur_stream()));
     return;
   }
   CHECK_HIP(kafka_launch_moe_route(nullptr, 0, (int)T, (int)E, (int)k, (int)bm, topk_w.data_ptr<float>(),
@@ -1129,7 +1138,8 @@ PYBIND11_MODULE(_kafka_ops, m) {
   m.def("wstream_grouped", &wstream_grouped, py::arg("x"), py::arg("wt"), py::arg("perm_tok"), py::arg("perm_w"),
         py::arg("expert_off"), py::arg("e_lo"), py::arg("max_rows"), py::arg("gather"), py::arg("y"), py::arg("out"),
         py::arg("pin") = true, py::arg("glu_limit") = 0.0, py::arg("glu_alpha") = 1.0, py::arg("relu2") = false);
-  m.def("moe_sort", &moe_sort);
+  m.def("moe_sort", &moe_sort, py::arg("topk_w"), py::arg("topk_e"), py::arg("E"), py::arg("bm"), py::arg("perm_tok"),
+        py::arg("perm_w"), py::arg("expert_off"), py::arg("tile_off"), py::arg("inv") = py::none());
   m.def("moe_route", &moe_route);
   m.def("cu_mask_stream", &cu_mask_stream);
   m.def("stream_cu_mask", &stream_cu_mask);

@@ -176,9 +176,10 @@ hipError_t kafka_hy_lin_scan(int f32, const void* qk, int64_t qk_s, int q_off, i
                              int R, int min_n, int max_n, float* S, float* out, int64_t os, hipStream_t st);
 int kafka_hy_add_tanh_norm_max_slabs();
 hipError_t kafka_hy_add_tanh_norm(int f32, float* x, int64_t xs, const void* y1, int64_t y1s, int y1_f32, int S,
-                                  int64_t slab, const float* y2, int64_t y2s, int assign, int n_norms,
-                                  const float* alpha, const float* const* w, const float* const* b, void* const* out,
-                                  const int64_t* os, void* copy, int64_t cs, int64_t T, int d, hipStream_t st);
+                                  int64_t slab, const float* y2, int64_t y2s, const void* er, int64_t ers,
+                                  const int* inv, int ek, int assign, int n_norms, const float* alpha,
+                                  const float* const* w, const float* const* b, void* const* out, const int64_t* os,
+                                  void* copy, int64_t cs, int64_t T, int d, hipStream_t st);
 int64_t kafka_hy_lin_chunk_scratch(int D, int Dv, int delta);
 hipError_t kafka_hy_lin_chunked(int f32, const void* qk, int64_t qk_s, int q_off, int k_off, const void* v, int64_t v_s,
                                 const void* z, int64_t z_s, const float* z_bias, const float* rate, const void* beta,
@@ -1167,13 +1168,14 @@ void norm_add(at::Tensor x, at::Tensor y1, OptT y2, at::Tensor w, double eps, Op
 
 // x (+)= y1 + y2, then up to two tanh norms of the new x and a copy of it in the activation dtype
 void add_tanh_norm(at::Tensor x, OptT y1, OptT y2, bool assign, std::vector<double> alpha, std::vector<at::Tensor> w,
-                   std::vector<at::Tensor> b, std::vector<at::Tensor> outs, OptT copy) {
+                   std::vector<at::Tensor> b, std::vector<at::Tensor> outs, OptT copy, OptT rows, OptT inv) {
   rows2d(x, "x"); f32t(x, "x");
   const int64_t T = x.size(0), d = x.size(1);
   TORCH_CHECK(x.stride(0) >= d, "add_tanh_norm: rows of x must not overlap");
   const size_t n = outs.size();
   TORCH_CHECK(n <= 2 && alpha.size() == n && w.size() == n && b.size() == n, "add_tanh_norm: up to two norms");
-  TORCH_CHECK(y1.has_value() || (!assign && !y2.has_value()), "add_tanh_norm: y2 and assign need y1");
+  TORCH_CHECK(y1.has_value() || (!assign && !y2.has_value() && !rows.has_value()),
+              "add_tanh_norm: y2 and assign need y1");
   int f32 = -1;   // the activation dtype: that of the outputs, else of y1
   float al[2]; const float *wp[2], *bp[2]; void* op[2]; int64_t os[2];
   auto dest = [&](const at::Tensor& o) {
@@ -1212,8 +1214,18 @@ void add_tanh_norm(at::Tensor x, OptT y1, OptT y2, bool assign, std::vector<doub
     TORCH_CHECK(y2->size(0) == T && y2->size(1) == d, "add_tanh_norm: y2 fp32 [T, d]");
     p2 = y2->data_ptr<float>(); s2 = y2->stride(0);
   }
+  const void* er = nullptr; int64_t ers = 0; const int* ip = nullptr; int ek = 0;
+  if (rows.has_value()) {   // row numbers come from the expert sort, which keeps them below T k
+    TORCH_CHECK(inv.has_value() && inv->is_cuda() && inv->scalar_type() == at::kInt && inv->is_contiguous() &&
+                    inv->dim() == 2 && inv->size(0) == T && inv->size(1) >= 1, "add_tanh_norm: inv int32 [T, k]");
+    rows2d(*rows, "rows");
+    if (f32 < 0) f32 = act_f32(*rows);
+    same_act(f32, {&*rows});
+    TORCH_CHECK(rows->size(0) >= inv->numel() && rows->size(1) == d, "add_tanh_norm: expert rows [T k, d]");
+    er = rows->data_ptr(); ers = rows->stride(0); ip = inv->data_ptr<int>(); ek = (int)inv->size(1);
+  }
   if (f32 < 0) return;   // nothing to do
-  HY_HIP(kafka_hy_add_tanh_norm(f32, x.data_ptr<float>(), x.stride(0), p1, s1, y1f, (int)S, slab, p2, s2,
+  HY_HIP(kafka_hy_add_tanh_norm(f32, x.data_ptr<float>(), x.stride(0), p1, s1, y1f, (int)S, slab, p2, s2, er, ers, ip, ek,
                                 assign ? 1 : 0, (int)n, al, wp, bp, op, os,
                                 copy.has_value() ? copy->data_ptr() : nullptr, copy.has_value() ? copy->stride(0) : 0,
                                 T, (int)d, stream()));
@@ -1353,7 +1365,8 @@ void kafka_bind_hybrid(pybind11::module_& m) {
   m.def("hy_norm_add", &norm_add);
   m.def("hy_ff_act", &ff_act);
   m.def("hy_add_tanh_norm", &add_tanh_norm, py::arg("x"), py::arg("y1"), py::arg("y2"), py::arg("assign"),
-        py::arg("alpha"), py::arg("w"), py::arg("b"), py::arg("outs"), py::arg("copy") = py::none());
+        py::arg("alpha"), py::arg("w"), py::arg("b"), py::arg("outs"), py::arg("copy") = py::none(),
+        py::arg("rows") = py::none(), py::arg("inv") = py::none());
   m.def("hy_lin_scan", &lin_scan);
   m.def("hy_lin_chunk", []() { return kafka_hy_lin_chunk(); });
   m.def("hy_sigmoid_attn_mfma_ok",

@@ -2,7 +2,8 @@
 //
 //   add_tanh_norm   x += y1 + y2 (or x = y1 + y2) on the fp32 stream and, from the new x, up to two outputs
 //                   tanh(alpha x) * w + b and a copy, in the activation dtype. y1 may be the split-K slabs of a projection
-//                   (summed while loading); every part is optional.
+//                   (summed while loading), y2 a token's routed expert rows (gathered while loading); every part is
+//                   optional.
 //
 // Built for bf16 and fp32 activations; the stream, the sums and the norms are fp32 in both. Sizes are run-time values
 // with no alignment assumptions (four columns per thread where sizes and strides allow).
@@ -42,7 +43,9 @@ struct TanhNorms {
 template <typename AT, int VEC, int S>
 __global__ __launch_bounds__(NT) void add_tanh_norm_kernel(float* __restrict__ x, int64_t xs,
                                                            const void* __restrict__ y1, int64_t y1s, int64_t slab,
-                                                           const float* __restrict__ y2, int64_t y2s, bool assign,
+                                                           const float* __restrict__ y2, int64_t y2s,
+                                                           const AT* __restrict__ er, int64_t ers,
+                                                           const int* __restrict__ inv, int ek, bool assign,
                                                            TanhNorms nm, AT* __restrict__ copy, int64_t cs, int64_t T,
                                                            int d, int rows) {
   const int i = ((int)blockIdx.x * NT + (int)threadIdx.x) * VEC;
@@ -80,6 +83,23 @@ __global__ __launch_bounds__(NT) void add_tanh_norm_kernel(float* __restrict__ x
 #pragma unroll
         for (int e = 0; e < VEC; ++e) y[e] += y2[t * y2s + i + e];
       }
+      if (er != nullptr) {   // in the order of the token's choices
+        constexpr int PF = 4;
+        for (int j0 = 0; j0 < ek; j0 += PF) {
+          AT z[PF][VEC];
+#pragma unroll
+          for (int j = 0; j < PF; ++j) {
+            const AT* p = er + (int64_t)inv[t * ek + min(j0 + j, ek - 1)] * ers + i;
+#pragma unroll
+            for (int e = 0; e < VEC; ++e) z[j][e] = p[e];
+          }
+#pragma unroll
+          for (int j = 0; j < PF; ++j)
+            if (j0 + j < ek)
+#pragma unroll
+              for (int e = 0; e < VEC; ++e) y[e] += (float)z[j][e];
+        }
+      }
 #pragma unroll
       for (int e = 0; e < VEC; ++e) v[e] += y[e];
 #pragma unroll
@@ -110,9 +130,10 @@ int kafka_hy_add_tanh_norm_max_slabs() { return TN_MAXS; }
 
 // y1_f32: y1 is fp32 with S slabs (S >= 1), else of the activation dtype
 hipError_t kafka_hy_add_tanh_norm(int f32, float* x, int64_t xs, const void* y1, int64_t y1s, int y1_f32, int S,
-                                  int64_t slab, const float* y2, int64_t y2s, int assign, int n_norms,
-                                  const float* alpha, const float* const* w, const float* const* b, void* const* out,
-                                  const int64_t* os, void* copy, int64_t cs, int64_t T, int d, hipStream_t st) {
+                                  int64_t slab, const float* y2, int64_t y2s, const void* er, int64_t ers,
+                                  const int* inv, int ek, int assign, int n_norms, const float* alpha,
+                                  const float* const* w, const float* const* b, void* const* out, const int64_t* os,
+                                  void* copy, int64_t cs, int64_t T, int d, hipStream_t st) {
   if (T <= 0 || d <= 0) return hipSuccess;
   if (n_norms < 0 || n_norms > 2 || S < 1 || S > TN_MAXS) return hipErrorInvalidValue;
   TanhNorms nm{};
@@ -123,7 +144,7 @@ hipError_t kafka_hy_add_tanh_norm(int f32, float* x, int64_t xs, const void* y1,
   };
   const size_t ab = f32 ? 16 : 8;
   bool v4 = d % 4 == 0 && al(x, xs, 16) && al(y1, y1s, y1_f32 ? 16 : ab) && slab % 4 == 0 && al(y2, y2s, 16) &&
-            al(copy, cs, ab);
+            al(copy, cs, ab) && al(er, ers, ab);
   for (int k = 0; k < n_norms; ++k) {
     nm.alpha[k] = alpha[k]; nm.w[k] = w[k]; nm.b[k] = b[k]; nm.out[k] = out[k]; nm.os[k] = os[k];
     v4 = v4 && al(w[k], 0, 16) && al(b[k], 0, 16) && al(out[k], os[k], ab);
@@ -135,7 +156,7 @@ hipError_t kafka_hy_add_tanh_norm(int f32, float* x, int64_t xs, const void* y1,
   const dim3 grid(gx, (unsigned)((T + rows - 1) / rows));
   auto a = [&](auto k, auto* tag) {
     using AT = std::remove_pointer_t<decltype(tag)>;
-    k<<<grid, NT, 0, st>>>(x, xs, y1, y1s, slab, y2, y2s, assign != 0, nm, (AT*)copy, cs, T, d, rows);
+    k<<<grid, NT, 0, st>>>(x, xs, y1, y1s, slab, y2, y2s, (const AT*)er, ers, inv, ek, assign != 0, nm, (AT*)copy, cs, T, d, rows);
   };
 #define TN_S(AT, V)                                                                 \
   do {                                                                              \

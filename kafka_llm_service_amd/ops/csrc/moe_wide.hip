@@ -8,7 +8,8 @@
 //                  column tile, then expert, and every XCD takes one contiguous stretch of them: the row tiles of a
 //                  column tile run side by side on one L2 and its weights leave memory once.
 //                  Epilogues: silu(gate) * up or its clamped form on GLU-interleaved tiles (a wave holds both tiles of a
-//                  pair), relu squared, or the weighted combine into fp32 rows.
+//                  pair), relu squared, the weighted combine into fp32 rows, or the weighted rows as they are (in entry
+//                  order; their consumer gathers a token's rows through the sort's inverse, no atomics).
 //   moe_sort       stable sort of (token, choice) entries by expert, one workgroup: every wave counts and then places
 //                  its stretch of the entries 64 at a time, equal experts found by ballots over the bits of their ids
 //   narrow         fp32 products of bf16 rows with up to 64 bf16 weight rows (router logits, gate projections): 16 rows a
@@ -25,7 +26,7 @@ constexpr int KS = BK / 16;        // matrix steps per staged block
 constexpr int MT = BM / 32;        // row tiles
 constexpr int XL = BM * (BK / 8) / 256;
 
-enum { EPI_GLU = 0, EPI_RELU2 = 1, EPI_COMBINE = 2 };
+enum { EPI_GLU = 0, EPI_RELU2 = 1, EPI_COMBINE = 2, EPI_ROWS = 3 };
 
 // 16-byte piece c (0 .. 7) of LDS row r
 __device__ __forceinline__ int xoff(int r, int c) { return r * BK + 8 * (c ^ (r & 7)); }
@@ -165,6 +166,11 @@ __global__ __launch_bounds__(256, 2) void grouped_wide_kernel(const bf16* __rest
         const float pw = perm_w[ent];
         atomicAdd(o, pw * acc[mt][0][i]);
         atomicAdd(o + 32, pw * acc[mt][1][i]);
+      } else if constexpr (EPI == EPI_ROWS) {
+        bf16* y = Y + (int64_t)ent * ldy + nb * 32 + r;
+        const float pw = perm_w[ent];
+        y[0] = (bf16)(pw * acc[mt][0][i]);
+        y[32] = (bf16)(pw * acc[mt][1][i]);
       } else if constexpr (EPI == EPI_RELU2) {
         bf16* y = Y + (int64_t)ent * ldy + nb * 32 + r;
         const float a = fmaxf(acc[mt][0][i], 0.f), b = fmaxf(acc[mt][1][i], 0.f);
@@ -200,7 +206,7 @@ __global__ __launch_bounds__(SORT_NT) void moe_sort_kernel(const float* __restri
                                                            const int* __restrict__ topk_e, int n, int k, int E, int bits,
                                                            int bm, int* __restrict__ perm_tok,
                                                            float* __restrict__ perm_w, int* __restrict__ expert_off,
-                                                           int* __restrict__ tile_off) {
+                                                           int* __restrict__ tile_off, int* __restrict__ inv) {
   __shared__ int cnt[SORT_W][SORT_MAXE];
   __shared__ int sum[2][SORT_W];
   const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
@@ -279,6 +285,7 @@ __global__ __launch_bounds__(SORT_NT) void moe_sort_kernel(const float* __restri
         const int pos = at + __builtin_popcountll(m & ((1ull << lane) - 1));
         perm_tok[pos] = i / k;
         perm_w[pos] = wv[p];
+        if (inv != nullptr) inv[i] = pos;
         if (__builtin_ctzll(m) == lane) cnt[w][ev[p]] = at + __builtin_popcountll(m);
       }
       __builtin_amdgcn_wave_barrier();
@@ -416,23 +423,24 @@ extern "C" {
 int kafka_moe_sort_max_e() { return SORT_MAXE; }
 
 hipError_t kafka_launch_moe_sort(const float* topk_w, const int* topk_e, int n, int k, int E, int bm, int* perm_tok,
-                                 float* perm_w, int* expert_off, int* tile_off, hipStream_t st) {
+                                 float* perm_w, int* expert_off, int* tile_off, int* inv, hipStream_t st) {
   if (n < 1) return hipSuccess;
   if (E < 1 || E > SORT_MAXE || k < 1 || bm < 1) return hipErrorInvalidValue;
   int bits = 0;
   while ((1 << bits) < E) ++bits;
-  moe_sort_kernel<<<1, SORT_NT, 0, st>>>(topk_w, topk_e, n, k, E, bits, bm, perm_tok, perm_w, expert_off, tile_off);
+  moe_sort_kernel<<<1, SORT_NT, 0, st>>>(topk_w, topk_e, n, k, E, bits, bm, perm_tok, perm_w, expert_off, tile_off,
+                                        inv);
   return hipGetLastError();
 }
 
 // epi: 0 gate_up -> silu(gate) * up (or clamped) into Y [n_ent][N / 2], 1 relu squared into Y [n_ent][N], 2 combine into
-// out [T][N]
+// out [T][N], 3 weighted rows into Y [n_ent][N]
 hipError_t kafka_launch_grouped_wide(const bf16* X, int64_t ldx, const bf16* Wt, int E, int N, int K,
                                      const int* perm_tok, const float* perm_w, const int* expert_off, int n_ent,
                                      int gather, int epi, bf16* Y, int64_t ldy, float* out, int64_t ldo,
                                      float glu_limit, float glu_alpha, hipStream_t st) {
   if (n_ent < 1 || E < 1) return hipSuccess;
-  if (N % 64 || K % (2 * BK) || N < 64 || K < 2 * BK || epi < 0 || epi > 2 || (epi == EPI_COMBINE) != (out != nullptr) ||
+  if (N % 64 || K % (2 * BK) || N < 64 || K < 2 * BK || epi < 0 || epi > 3 || (epi == EPI_COMBINE) != (out != nullptr) ||
       (epi != EPI_COMBINE) != (Y != nullptr))
     return hipErrorInvalidValue;
   const int64_t items = ((int64_t)n_ent / BM + E) * ((N + BN - 1) / BN);   // an upper bound over all routings
@@ -444,6 +452,7 @@ hipError_t kafka_launch_grouped_wide(const bf16* X, int64_t ldx, const bf16* Wt,
   };
   if (epi == EPI_GLU) { if (gather) a(grouped_wide_kernel<true, EPI_GLU>); else a(grouped_wide_kernel<false, EPI_GLU>); }
   else if (epi == EPI_RELU2) { if (gather) a(grouped_wide_kernel<true, EPI_RELU2>); else a(grouped_wide_kernel<false, EPI_RELU2>); }
+  else if (epi == EPI_ROWS) { if (gather) a(grouped_wide_kernel<true, EPI_ROWS>); else a(grouped_wide_kernel<false, EPI_ROWS>); }
   else { if (gather) a(grouped_wide_kernel<true, EPI_COMBINE>); else a(grouped_wide_kernel<false, EPI_COMBINE>); }
   return hipGetLastError();
 }

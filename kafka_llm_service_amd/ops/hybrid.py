@@ -455,6 +455,35 @@ def moe_grouped_ok(h, w_gu, w_down, glu: bool = True) -> bool:
                 (F2 // 2 if glu else F2) % 64 == 0 and h.stride(0) % 8 == 0)
 
 
+class ExpertRows:
+    """The routed experts' weighted outputs as rows in entry order (activation dtype [T k, d]) with every entry's row
+    number ``inv`` int32 [T, k]: a token's sum is still to be taken (``add_tanh_norm`` does)."""
+    __slots__ = ("rows", "inv")
+
+    def __init__(self, rows: torch.Tensor, inv: torch.Tensor):
+        self.rows, self.inv = rows, inv
+
+    def sum(self) -> torch.Tensor:
+        return self.rows[self.inv.long()].float().sum(1)
+
+
+def moe_expert_rows(h, w_up_t, w_down_t, topk_w, topk_e, n_experts: int, act: str = "relu2", limit: float = 0.0,
+                    alpha: float = 1.0) -> ExpertRows:
+    """The experts of a long step on tiled weights (``moe_experts``' wide form) without the sum over a token's experts."""
+    from kafka_llm_service_amd import ops
+
+    glu = act != "relu2"
+    lim, al = _glu_act(act, limit, alpha) if glu else (0.0, 1.0)
+    r = ops.moe_sort(topk_w, topk_e, n_experts, inverse=True)
+    a = ops.grouped_wide(h, w_up_t, r, "glu" if glu else "relu2", True, limit=lim, alpha=al)
+    return ExpertRows(ops.grouped_wide(a, w_down_t, r, "rows", False), r.inv)
+
+
+def moe_wide(T: int, k: int, n_experts: int) -> bool:
+    """Whether a step of T rows runs tiled expert weights on the wide kernels."""
+    return T > MOE_STREAM_MAX_T or T * k >= MOE_WIDE_ROWS * n_experts
+
+
 def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None, act: str = "silu",
                 limit: float = 0.0, alpha: float = 1.0) -> None:
     """out (fp32 [T, d]) = the routed experts' weighted sum for every row. Sizes the framework's expert-sorted
@@ -473,7 +502,7 @@ def moe_experts(h, w_gu, w_down, topk_w, topk_e, out, w_gu_t=None, w_down_t=None
         out.zero_()
         if w_gu_t is not None and w_down_t is not None:
             lim, al = _glu_act(act, limit, alpha) if glu else (0.0, 1.0)
-            if T > MOE_STREAM_MAX_T or T * topk_e.shape[1] >= MOE_WIDE_ROWS * w_gu.shape[0]:
+            if moe_wide(T, topk_e.shape[1], w_gu.shape[0]):
                 a = ops.grouped_wide(h, w_gu_t, r, "glu" if glu else "relu2", True, limit=lim, alpha=al)
                 ops.grouped_wide(a, w_down_t, r, "combine", False, out)
             else:
@@ -831,16 +860,21 @@ class TanhNorm:
 def add_tanh_norm(x, y1=None, y2=None, norms=(), outs=(), copy=None, assign: bool = False) -> None:
     """One element-wise pass over the fp32 stream x [T, d], every part optional:
       x += y1 + y2, or with ``assign`` x = y1 + y2 (y1 [T, d] in the activation dtype or fp32, or the fp32 split-K slabs
-      [S, T, d] of a projection, summed here; y2 fp32);
+      [S, T, d] of a projection, summed here; y2 fp32 [T, d], or ``ExpertRows`` whose rows are gathered here);
       outs[k] = norms[k](new x), up to two ``TanhNorm``; copy = new x in its dtype (both may be column slices)."""
     if len(norms) != len(outs) or len(norms) > 2:
         raise ValueError("add_tanh_norm: up to two norms, an output each")
     if y1 is None and (y2 is not None or assign):
         raise ValueError("add_tanh_norm: y2 and assign need y1")
     if _gpu(x):
+        rows = inv = None
+        if isinstance(y2, ExpertRows):
+            y2, rows, inv = None, y2.rows, y2.inv
         ext().hy_add_tanh_norm(x, y1, y2, bool(assign), [n.alpha for n in norms], [n.w for n in norms],
-                               [n.b for n in norms], list(outs), copy)
+                               [n.b for n in norms], list(outs), copy, rows, inv)
     else:
+        if isinstance(y2, ExpertRows):
+            y2 = y2.sum()
         ref.add_tanh_norm(x, y1, y2, norms, outs, copy, assign)
 
 

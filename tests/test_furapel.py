@@ -203,6 +203,16 @@ def test_add_tanh_norm(device, d, T):
     assert ((out.cpu().double() - want).abs() <= 1e-6 * want.abs() + 1e-12).all()
     with pytest.raises((ValueError, RuntimeError)):
         hops.add_tanh_norm(x, assign=True)
+    # a token's expert rows, gathered
+    for dt, k in ((torch.float32, 3), (torch.bfloat16, 6)):
+        inv = torch.randperm(T * k, generator=g).int().view(T, k)
+        rows = torch.randn(T * k, d, generator=g).to(dt)
+        x, out = dv(x0.clone()), torch.empty(T, d, dtype=dt, device=device)
+        hops.add_tanh_norm(x, dv(y1.to(dt)), hops.ExpertRows(dv(rows), dv(inv)), norms[:1], [out])
+        want = x0.double() + y1.to(dt).double() + rows.double()[inv.long()].sum(1)
+        assert (x.cpu().double() - want).abs().max() < 1e-5 * max(1.0, float(want.abs().max()))
+        e = (out.cpu().double() - plain.tanh_norm(x.cpu().double(), W64, "n0")).abs().max()
+        assert e < (1e-6 if dt == torch.float32 else 2e-2)
 
 
 @pytest.mark.parametrize("rot", [YARN, {"base": 10000.0, "dims": 24}, dict(YARN, dims=24),
@@ -604,8 +614,8 @@ def test_sort_by_expert(n_exp, k, T):
         te[:, 0] = torch.where(te[:, 0] == 5, (te[:, 1] + 1) % n_exp, te[:, 0])
         te[T // 2:, 1] = 7
     tw = torch.rand(T, k, generator=g)
-    a, b = ops.moe_sort(tw.cuda(), te.cuda(), n_exp), ops.moe_sort(tw, te, n_exp)
-    for n in ("perm_tok", "perm_w", "expert_off", "tile_off"):
+    a, b = ops.moe_sort(tw.cuda(), te.cuda(), n_exp, inverse=True), ops.moe_sort(tw, te, n_exp, inverse=True)
+    for n in ("perm_tok", "perm_w", "expert_off", "tile_off", "inv"):
         assert torch.equal(getattr(a, n).cpu(), getattr(b, n)), n
 
 
@@ -638,6 +648,9 @@ def test_wide_expert_products(E, k, T, d, ff):
         ops.grouped_wide(a, ops.tile_experts(dd), r, "combine", False, out)
         ops.grouped_wide(a.cpu(), ops.tile_experts(down), rc, "combine", False, oc)
         assert close(out, oc, 1e-2)
+        rows = ops.grouped_wide(a, ops.tile_experts(dd), r, "rows", False)
+        r2 = ops.moe_sort(tw.cuda(), te.cuda(), E, inverse=True)
+        assert close(hops.ExpertRows(rows, r2.inv).sum(), oc, 1e-2)
 
 
 @pytest.mark.parametrize("device", DEVICES)
