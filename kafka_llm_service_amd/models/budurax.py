@@ -220,6 +220,22 @@ class SegMeta:
     max_keys: int = 0         # longest context of the step (first position + rows over the runs)
     cache: dict = field(default_factory=dict)   # per-step device tables derived from seg_host (chunk plans)
 
+    def tile_kinds(self, tokens: int) -> tuple[bool, bool]:
+        """(whether attention tiles of up to ``tokens`` tokens include single decoded tokens, whether they include prompt
+        portions), as ``hops.window_attn`` takes it. Tiles that hold one token anyway count as decoded ones as soon as
+        one sequence has a single row."""
+        key = ("tile kinds", tokens)
+        if key not in self.cache:
+            kinds = (True, False)
+            if self.seg_host is not None and len(self.seg_host):
+                rows = self.seg_host[:, 1]
+                if tokens > 1:
+                    kinds = (bool((rows % tokens == 1).any()), bool((rows > 1).any()))
+                elif (rows > 1).all():
+                    kinds = (False, True)
+            self.cache[key] = kinds
+        return self.cache[key]
+
     def chunks(self, chunk: int, min_rows: int):
         """(device tensors of ``hops.chunk_tables`` or None, (fewest, most rows) of the segments that are too short for
         chunks or None), built once per step. On the CPU nothing runs in chunks."""

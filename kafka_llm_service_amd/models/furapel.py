@@ -494,7 +494,7 @@ class FurapelLM:
         ao = torch.empty(T, H * Dv, dtype=dt, device=dev)
         hops.window_attn(q, k_cache, v_cache_t, m.block_tables, m.tok_seg, inp.positions, H, G, lw.scale, lw.window,
                          None, ao, m.tiles.get(hops.sig_tile_tokens(H, G)), m.max_keys, gate=proj,
-                         gate_off=H * D + G * D + G * Dv)
+                         gate_off=H * D + G * D + G * Dv, kinds=m.tile_kinds(hops.sig_tile_tokens(H, G)))
         return self._lin(ao, lw.o, getattr(lw, "o_t", None), slabs=True)
 
     def _latent_attention(self, r: int, lw, h, inp, m: SegMeta, pages: list) -> torch.Tensor:

@@ -567,7 +567,8 @@ class MagedraLM:
                            v_cache_t, inp.slot_mapping, q)
         ao = torch.empty(T, H * Dv, dtype=dt, device=dev)
         hops.window_attn(q, k_cache, v_cache_t, m.block_tables, m.tok_seg, inp.positions, H, G, lw.scale, 0, None, ao,
-                         m.tiles.get(hops.sig_tile_tokens(H, G)), m.max_keys, shared_keys=True)
+                         m.tiles.get(hops.sig_tile_tokens(H, G)), m.max_keys, shared_keys=True,
+                         kinds=m.tile_kinds(hops.sig_tile_tokens(H, G)))
         both = torch.empty(T, H * Dv + Hr * Dvr, dtype=dt, device=dev)            # [left heads | right heads]
         hops.gate_mul(ao, proj, lw.g_off, lw.left_scale, both[:, :H * Dv])
         o = torch.empty(T, Hr * Dvr, dtype=torch.float32, device=dev)

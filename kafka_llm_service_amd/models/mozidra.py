@@ -493,7 +493,8 @@ class MozidraLM:
             step[i] = (qkv, H * D + G * D)
         ao = torch.empty(T, H * Dv, dtype=dt, device=dev)
         hops.window_attn(q, k_cache, v_cache_t, m.block_tables, m.tok_seg, inp.positions, H, G, lw.scale, lw.window,
-                         lw.sink, ao, m.tiles.get(hops.sig_tile_tokens(H, G)), m.max_keys)
+                         lw.sink, ao, m.tiles.get(hops.sig_tile_tokens(H, G)), m.max_keys,
+                         kinds=m.tile_kinds(hops.sig_tile_tokens(H, G)))
         return self._lin(ao, lw.o, getattr(lw, "o_t", None))
 
     def _latent_attention(self, i: int, lw, h, inp, m: SegMeta, pages: list) -> torch.Tensor:

@@ -522,7 +522,7 @@ class RogosunLM:
                            inp.slot_mapping, q, lw.q_norm, lw.k_norm, eps, v_off=H * D)
         hops.window_attn(q, k_cache, v_cache_t, m.block_tables, m.tok_seg, inp.positions, H, G, lw.scale, 0, lw.sink,
                          both[:, :H * D], m.tiles.get(hops.sig_tile_tokens(H, G)), m.max_keys,
-                         out_scale=lw.left_scale)
+                         out_scale=lw.left_scale, kinds=m.tile_kinds(hops.sig_tile_tokens(H, G)))
         qkv = torch.empty(T, lw.conv.shape[0], dtype=dt, device=dev)
         hops.short_conv(proj, off["conv"], lw.conv, None, m.tok_seg, m.seg, st["conv"], qkv, act="silu")
         low = F.linear(proj[:, off["low"]:off["low"] + lw.low.shape[1]], lw.low)  # raw decays | output gate

@@ -128,7 +128,7 @@ hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, 
                                      int bt_stride, const int* items, int n_items, const int64_t* positions, int H,
                                      int G, int D, int Dv, float scale, int window, const float* sink, const void* gate, int64_t gs, void* out,
                                      int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
-                                     float out_scale, hipStream_t st);
+                                     float out_scale, int max_tok, int min_rows_tok, hipStream_t st);
 int kafka_hy_grouped_router_max_e();
 int kafka_hy_grouped_router_max_k();
 int kafka_hy_grouped_router_max_g();
@@ -949,7 +949,7 @@ void window_attn(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::
 void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt, at::Tensor items, int64_t tile_tokens,
                       at::Tensor positions, int64_t H, int64_t G, double scale, int64_t window, OptT sink,
                       at::Tensor out, int64_t nsplit, OptT po, OptT pml, bool shared_keys, double out_scale,
-                      OptT gate, int64_t gate_off) {
+                      OptT gate, int64_t gate_off, int64_t max_tok, int64_t min_rows_tok) {
   for (const at::Tensor* t : {&q, &kc, &vt, &out})
     TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16, "window_attn_mfma: bf16 GPU tensors");
   rows2d(q, "q"); rows2d(out, "out");
@@ -969,7 +969,9 @@ void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt,
                   positions.is_cuda() && positions.scalar_type() == at::kLong && positions.is_contiguous() &&
                   positions.numel() == T, "window_attn_mfma: block tables / items / positions");
   float *pop = nullptr, *pmlp = nullptr;
-  TORCH_CHECK(nsplit >= 1 && nsplit <= 64, "window_attn_mfma: 1..64 key-range splits");
+  TORCH_CHECK(nsplit >= 1 && nsplit <= 64 && (nsplit == 1 || min_rows_tok == 0), "window_attn_mfma: 1..64 key-range splits");
+  TORCH_CHECK(max_tok >= 0 && max_tok <= 32 && min_rows_tok >= 0 && (min_rows_tok == 0 || min_rows_tok == max_tok + 1),
+              "window_attn_mfma: every item belongs to one of the two kernels");
   if (nsplit > 1) {
     TORCH_CHECK(po.has_value() && pml.has_value() && po->is_cuda() && po->scalar_type() == at::kFloat &&
                     po->is_contiguous() && po->numel() >= nsplit * T * H * Dv && pml->is_cuda() &&
@@ -983,7 +985,8 @@ void window_attn_mfma(at::Tensor q, at::Tensor kc, at::Tensor vt, at::Tensor bt,
                                    positions.data_ptr<int64_t>(), (int)H, (int)G, (int)D, (int)Dv, (float)scale,
                                    (int)window, sink_ptr(sink, H), head_gate_ptr(gate, gate_off, 0, T, H),
                                    gate.has_value() ? gate->stride(0) : 0, out.data_ptr(), out.stride(0), (int)nsplit,
-                                   pop, pmlp, T, shared_keys ? 1 : 0, (float)out_scale, stream()));
+                                   pop, pmlp, T, shared_keys ? 1 : 0, (float)out_scale, (int)max_tok,
+                                   (int)min_rows_tok, stream()));
 }
 
 void moe_topk_grouped(at::Tensor logits, int64_t E, OptT corr, int64_t groups, int64_t keep, double eps,
@@ -1352,7 +1355,7 @@ void kafka_bind_hybrid(pybind11::module_& m) {
         py::arg("items"), py::arg("tile_tokens"), py::arg("positions"), py::arg("H"), py::arg("G"), py::arg("scale"),
         py::arg("window"), py::arg("sink"), py::arg("out"), py::arg("nsplit") = 1, py::arg("po") = py::none(),
         py::arg("pml") = py::none(), py::arg("shared_keys") = false, py::arg("out_scale") = 1.0,
-        py::arg("gate") = py::none(), py::arg("gate_off") = 0);
+        py::arg("gate") = py::none(), py::arg("gate_off") = 0, py::arg("max_tok") = 32, py::arg("min_rows_tok") = 0);
   m.def("hy_moe_topk_grouped", &moe_topk_grouped);
   m.def("hy_act_norm", &act_norm);
   m.def("hy_gate_mul", &gate_mul);

@@ -19,6 +19,9 @@
 //                       row's keys are visited in order, whatever the batch
 //   window_attn_mfma    the same attention on the matrix cores (bf16): 32 (token, head) rows of one key/value head per
 //                       workgroup, 128-key blocks, online softmax, key-range splits with a merge pass
+//   window_attn_rows    the same attention for prompt portions (bf16): a wave per 32 (token, head) rows of one key/value
+//                       head, scores transposed so that rows are lanes - maxima, sums and weights stay in a lane's
+//                       registers, no LDS and no barriers
 //   moe_topk_grouped    softmax or sigmoid scores, choice among the best groups (by their largest score or the sum of
 //                       their two largest) by corrected score, weights normalised or as they are, times a scale
 #include "common.h"
@@ -387,7 +390,8 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
     const bf16* __restrict__ q, int64_t qs, const bf16* __restrict__ kc, const bf16* __restrict__ vt,
     const int* __restrict__ bt, int bt_stride, const int* __restrict__ items, const int64_t* __restrict__ positions,
     int H, int G, int D, int Dv, int Ck, int kstep, float scale_log2e, int window, const float* __restrict__ sink,
-    const bf16* __restrict__ gate, int64_t gs, bf16* __restrict__ out, int64_t os, float* __restrict__ po, float* __restrict__ pml, int64_t T, float out_scale) {
+    const bf16* __restrict__ gate, int64_t gs, bf16* __restrict__ out, int64_t os, float* __restrict__ po,
+    float* __restrict__ pml, int64_t T, float out_scale, int max_tok) {
   // (D, Ck, kstep as in window_attn_kernel: kstep = 0 and D = Ck when every query row meets the whole key row)
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   const int nks = D >> 4, qstride = D + 8;
@@ -397,6 +401,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
   int* prow_s = reinterpret_cast<int*>(mloc + 4 * WM_ROWS);       // [32]
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, lr = lane & 31, lh = lane >> 5;
   const int t0 = items[4 * blockIdx.x], ntok = items[4 * blockIdx.x + 1], sg = items[4 * blockIdx.x + 2];
+  if (ntok > max_tok) return;   // (uniform) an item of window_attn_rows
   const int g = blockIdx.y, rep = H / G;
   const int nrows = ntok * rep;
   for (int i = threadIdx.x; i < WM_ROWS * (D >> 3); i += 256) {
@@ -551,6 +556,140 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(
       }
     }
   }
+}
+
+// ---- the same for prompt portions: a wave per item ------------------------------------------------------------------
+// A wave takes one item's 32 (token, head) rows of one key/value head and walks their keys 32 at a time:
+//   scores   S^T = K Q^T: lane = row, a lane's 16 registers = its half of the block's keys. The key rows are loaded with
+//            bits 2 and 3 of their numbers swapped, which leaves lane half lh with keys 8 lh .. + 7 of each page;
+//   softmax  a row's maximum, sum and weights live in its two lanes; the accumulators are rescaled only when a row's
+//            maximum has moved;
+//   values   O^T += V^T P^T: the weights are the right operand as they lie in the registers, the left one is a channel's
+//            8 consecutive tokens of a transposed page (16 bytes).
+// No LDS and no barriers; the four waves of a workgroup are neighbouring items (the same keys, from the cache), a key/value
+// head's workgroups go to one XCD where there are eight of them, the items with the most keys first. NKS, NVT: steps of
+// 16 key channels and tiles of 32 value channels held in registers (queries past D are zero).
+template <int NKS, int NVT>
+__global__ __launch_bounds__(256, NKS * 4 + NVT * 16 <= 96 ? 2 : 1) void window_attn_rows_kernel(
+    const bf16* __restrict__ q, int64_t qs, const bf16* __restrict__ kc, const bf16* __restrict__ vt,
+    const int* __restrict__ bt, int bt_stride, const int* __restrict__ items, int n_items,
+    const int64_t* __restrict__ positions, int H, int G, int D, int Dv, int Ck, int kstep, float scale_log2e, int window,
+    const float* __restrict__ sink, const bf16* __restrict__ gate, int64_t gs, bf16* __restrict__ out, int64_t os,
+    float out_scale, int min_tok, bool vec4) {
+  const int lane = threadIdx.x & 63, lr = lane & 31, lh = lane >> 5;
+  const int item = n_items - 1 - ((int)blockIdx.y * (int)(blockDim.x >> 6) + (int)(threadIdx.x >> 6));
+  if (item < 0) return;   // whole waves leave; nothing below synchronises across waves
+  const int t0 = items[4 * item], ntok = items[4 * item + 1], sg = items[4 * item + 2];
+  if (ntok < min_tok) return;
+  const int g = blockIdx.x, rep = H / G, nks = D >> 4, nrows = ntok * rep;
+  const bool live = lr < nrows;
+  const int row = min(lr, nrows - 1), h = g * rep + row % rep;
+  const int64_t t = t0 + row / rep;
+  const int p = (int)positions[t], minpos = (int)positions[t0], maxpos = (int)positions[t0 + ntok - 1];
+  const int* btr = bt + (int64_t)sg * bt_stride;
+  const int Cv = G * Dv;
+  bf16x8 qf[NKS], kf[NKS];
+#pragma unroll
+  for (int ks = 0; ks < NKS; ++ks) {
+    qf[ks] = load_bf16x8(q + t * qs + (int64_t)h * D + 16 * min(ks, nks - 1) + 8 * lh);
+    if (ks >= nks) qf[ks] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+  }
+  const int krow = (lr & 19) | ((lr & 4) << 1) | ((lr & 8) >> 1);   // bits 2 and 3 swapped
+  auto fetch_keys = [&](int kb) {
+    const int key = min(32 * kb + krow, maxpos);   // past the item's last position: a valid row, masked below
+    const bf16* kp = kc + ((int64_t)btr[key >> 4] * PAGE + (key & 15)) * Ck + (int64_t)g * kstep + 8 * lh;
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) kf[ks] = load_bf16x8(kp + 16 * min(ks, nks - 1));
+  };
+  float m = -INFINITY, l = 0.f;
+  f32x16 O[NVT];
+#pragma unroll
+  for (int v = 0; v < NVT; ++v)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) O[v][i] = 0.f;
+  const int kb0 = window > 0 ? max(0, minpos - window + 1) >> 5 : 0, kb1 = (maxpos >> 5) + 1;
+  fetch_keys(kb0);
+  for (int kb = kb0; kb < kb1; ++kb) {
+    bf16x8 vf[2][NVT];
+#pragma unroll
+    for (int pg = 0; pg < 2; ++pg) {
+      // a page past the last position: the last valid one, its weights are zero
+      const bf16* vp = vt + ((int64_t)btr[min(2 * kb + pg, maxpos >> 4)] * Cv + (int64_t)g * Dv) * PAGE + 8 * lh;
+#pragma unroll
+      for (int v = 0; v < NVT; ++v) vf[pg][v] = load_bf16x8(vp + (int64_t)min(32 * v + lr, Dv - 1) * PAGE);
+    }
+    f32x16 S;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) S[i] = 0.f;
+#pragma unroll
+    for (int ks = 0; ks < NKS; ++ks) S = mfma32(kf[ks], qf[ks], S);
+    if (kb + 1 < kb1) fetch_keys(kb + 1);
+    float s[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) s[i] = S[i] * scale_log2e;
+    // (uniform) a block that every row sees whole needs no mask
+    if (32 * kb + 31 > minpos || (window > 0 && 32 * kb <= maxpos - window)) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int key = 32 * kb + 16 * (i >> 3) + 8 * lh + (i & 7);
+        if (key > p || (window > 0 && key <= p - window)) s[i] = -INFINITY;
+      }
+    }
+    float mx = s[0];
+#pragma unroll
+    for (int i = 1; i < 16; ++i) mx = fmaxf(mx, s[i]);
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float mn = fmaxf(m, mx);
+    const float base = mn == -INFINITY ? 0.f : mn;   // nothing visible yet: every weight is 2^-inf = 0
+    if (__any(mx > m)) {
+      const float corr = m == -INFINITY ? 0.f : fast_exp2(m - base);
+      l *= corr;
+#pragma unroll
+      for (int v = 0; v < NVT; ++v)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) O[v][i] *= corr;
+    }
+    m = mn;
+    bf16x8 pf[2];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float e = fast_exp2(s[i] - base);
+      l += e;
+      pf[i >> 3][i & 7] = (bf16)e;
+    }
+#pragma unroll
+    for (int pg = 0; pg < 2; ++pg)
+#pragma unroll
+      for (int v = 0; v < NVT; ++v) O[v] = mfma32(vf[pg][v], pf[pg], O[v]);
+  }
+  // the last products' results are complete before anything reads them behind a branch
+  __builtin_amdgcn_sched_barrier(0);
+  asm volatile("s_nop 15");
+  __builtin_amdgcn_sched_barrier(0);
+  l += __shfl_xor(l, 32, 64);
+  if (!live) return;
+  if (sink != nullptr) l += fast_exp2(sink[h] * LOG2E - m);
+  float inv = out_scale / l;
+  if (gate != nullptr) inv *= head_gate(gate + t * gs + h);
+  bf16* op = out + t * os + (int64_t)h * Dv;
+#pragma unroll
+  for (int v = 0; v < NVT; ++v)
+#pragma unroll
+    for (int i4 = 0; i4 < 4; ++i4) {
+      const int c = 32 * v + 8 * i4 + 4 * lh;
+      if (vec4) {
+        typedef bf16 bf16x4 __attribute__((ext_vector_type(4)));
+        if (c < Dv) {
+          const bf16x4 o = {(bf16)(O[v][4 * i4] * inv), (bf16)(O[v][4 * i4 + 1] * inv), (bf16)(O[v][4 * i4 + 2] * inv),
+                            (bf16)(O[v][4 * i4 + 3] * inv)};
+          *reinterpret_cast<bf16x4*>(op + c) = o;
+        }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (c + e < Dv) op[c + e] = (bf16)(O[v][4 * i4 + e] * inv);
+      }
+    }
 }
 
 // out[t][h] = sum_z 2^(m_z - m) O_z / (sum_z 2^(m_z - m) l_z + 2^(sink_h - m)) over the key-range splits
@@ -831,18 +970,46 @@ int kafka_hy_window_attn_mfma_ok(int page, int D, int Dv, int rep) {
 hipError_t kafka_hy_window_attn_mfma(const void* q, int64_t qs, const void* kc, const void* vt, const int* bt,
                                      int bt_stride, const int* items, int n_items, const int64_t* positions, int H,
                                      int G, int D, int Dv, float scale, int window, const float* sink,
-                                     const void* gate, int64_t gs, void* out, int64_t os, int nsplit, float* po, float* pml, int64_t T, int shared_keys,
-                                     float out_scale, hipStream_t st) {
+                                     const void* gate, int64_t gs, void* out, int64_t os, int nsplit, float* po,
+                                     float* pml, int64_t T, int shared_keys, float out_scale, int max_tok, int min_rows_tok, hipStream_t st) {
+  // items of up to max_tok tokens here (0: none), those of at least min_rows_tok tokens a wave each (0: none)
   if (n_items <= 0) return hipSuccess;
   const int Ck = shared_keys ? D : G * D, kstep = shared_keys ? 0 : D;
   if (G < 1 || H % G || window < 0 || !kafka_hy_window_attn_mfma_ok(PAGE, D, Dv, H / G)) return hipErrorInvalidValue;
   if (nsplit < 1 || nsplit > 64 || (nsplit > 1 && (po == nullptr || pml == nullptr))) return hipErrorInvalidValue;
+  if (min_rows_tok > 0) {
+    const bool vec4 = Dv % 4 == 0 && os % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0;
+    const int waves = (int64_t)n_items * G >= 2048 ? 4 : (int64_t)n_items * G >= 1024 ? 2 : 1;
+    const int64_t gy = (n_items + waves - 1) / waves;
+    if (gy > 65535) return hipErrorInvalidValue;
+    const dim3 gr((unsigned)G, (unsigned)gy);
+    auto b = [&](auto k) {
+      k<<<gr, 64 * waves, 0, st>>>((const bf16*)q, qs, (const bf16*)kc, (const bf16*)vt, bt, bt_stride, items, n_items,
+                                   positions, H, G, D, Dv, Ck, kstep, scale * LOG2E, window, sink, (const bf16*)gate, gs,
+                                   (bf16*)out, os, out_scale, min_rows_tok, vec4);
+    };
+    if (D <= 64) {
+      if (Dv <= 64) b(window_attn_rows_kernel<4, 2>);
+      else if (Dv <= 128) b(window_attn_rows_kernel<4, 4>);
+      else b(window_attn_rows_kernel<4, 8>);
+    } else if (D <= 128) {
+      if (Dv <= 64) b(window_attn_rows_kernel<8, 2>);
+      else if (Dv <= 128) b(window_attn_rows_kernel<8, 4>);
+      else b(window_attn_rows_kernel<8, 8>);
+    } else {
+      if (Dv <= 64) b(window_attn_rows_kernel<16, 2>);
+      else if (Dv <= 128) b(window_attn_rows_kernel<16, 4>);
+      else b(window_attn_rows_kernel<16, 8>);
+    }
+  }
+  if (max_tok <= 0) return hipGetLastError();
+  if (nsplit > 1 && min_rows_tok > 0) return hipErrorInvalidValue;   // (the merge pass takes every row)
   const size_t lds = (size_t)WM_ROWS * (D + 8) * 2 + WM_ROWS * 136 * 2 + 5 * WM_ROWS * 4;
   const dim3 grid((unsigned)n_items, (unsigned)G, (unsigned)nsplit);
   auto a = [&](auto k) {
     k<<<grid, 256, lds, st>>>((const bf16*)q, qs, (const bf16*)kc, (const bf16*)vt, bt, bt_stride, items, positions, H,
                               G, D, Dv, Ck, kstep, scale * LOG2E, window, sink, (const bf16*)gate, gs, (bf16*)out, os, po, pml,
-                              T, out_scale);
+                              T, out_scale, max_tok);
   };
   const int nks = D / 16, tw = ((Dv + 31) / 32 + 3) / 4;
   if (tw == 1 && nks <= 4) a(window_attn_mfma_kernel<1, 4>);

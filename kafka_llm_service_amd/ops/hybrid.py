@@ -614,7 +614,7 @@ def window_attn_mfma_ok(q, k_cache, v_cache_t, H: int, G: int, shared_keys: bool
 
 def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int, G: int, scale: float, window: int,
                 sink, out, tiles=None, max_keys: int = 0, shared_keys: bool = False, out_scale: float = 1.0, gate=None,
-                gate_off: int = 0) -> None:
+                gate_off: int = 0, kinds=(True, False)) -> None:
     """Causal softmax attention over paged keys [pages, page, G D] and page-wise transposed values [pages, G Dv, page]:
     row t at position p, head h (key/value head h // (H / G)) sees the keys p - window < j <= p (window 0: all j <= p);
         out = sum_j e^(s_j) v_j / (sum_j e^(s_j) + e^(sink[h])),  s_j = (q . k_j) scale
@@ -627,7 +627,9 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
     product with ALL G key heads of a token (queries that hold a mix over the heads, see ``rope_kv_store``); values
     stay per key/value head. The result is multiplied by ``out_scale``; ``out`` may be a column slice.
     ``gate``: rows whose columns [gate_off, gate_off + H) hold one raw gate per head - head h's output is multiplied by
-    sigmoid(gate[t, gate_off + h])."""
+    sigmoid(gate[t, gate_off + h]).
+    ``kinds``: (whether ``tiles`` has decoded-token tiles, whether it has prompt tiles) as ``SegMeta.tile_kinds`` tells:
+    prompt tiles then run a wave each (window_attn_rows), without key-range splits."""
     if window < 0:
         raise ValueError("window_attn: window must be positive (0 = every earlier position)")
     if _gpu(q):
@@ -637,14 +639,16 @@ def window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, H: int,
                 max_keys = min(max_keys, window + tt)
             # (shared keys: few key/value heads, every workgroup walks the whole key row - more, shorter ranges)
             ns = sig_splits(tiles.shape[0] * G, max_keys, SHARED_SPLIT_WGS if shared_keys else WINDOW_SPLIT_WGS) \
-                if max_keys else 1
+                if max_keys and not kinds[1] else 1
+            # tiles of up to mt tokens here, the others a wave each
+            mt = 32 if not kinds[1] else 1 if kinds[0] and tt > 1 else 0
             po = pml = None
             if ns > 1:
                 po = torch.empty(ns, q.shape[0], out.shape[1], dtype=torch.float32, device=q.device)
                 pml = torch.empty(ns, q.shape[0], H, 2, dtype=torch.float32, device=q.device)
             ext().hy_window_attn_mfma(q, k_cache, v_cache_t, block_tables, tiles, tt, positions, int(H), int(G),
                                       float(scale), int(window), sink, out, ns, po, pml, bool(shared_keys),
-                                      float(out_scale), gate, int(gate_off))
+                                      float(out_scale), gate, int(gate_off), mt, mt + 1 if kinds[1] else 0)
         else:
             ext().hy_window_attn(q, k_cache, v_cache_t, block_tables, tok_seg, positions, int(H), int(G), float(scale),
                                  int(window), sink, out, bool(shared_keys), float(out_scale), gate, int(gate_off))

@@ -352,10 +352,12 @@ def test_head_gated_attention_matrix_cores(H, G, D, Dv, rot, n):
         tiles = torch.tensor([(a, min(tt, rows - a), 0, 0) for a in range(0, rows, tt)], dtype=torch.int32, device=dev)
         assert hops.window_attn_mfma_ok(q, kc, vt, H, G)
         outs = []
-        for t, max_keys in ((None, 0), (tiles, 0), (tiles, at + rows)):   # vector kernel; unsplit; split key ranges
+        # vector kernel; unsplit; split key ranges; a wave per tile
+        for t, max_keys, kinds in ((None, 0, (True, False)), (tiles, 0, (True, False)), (tiles, at + rows, (True, False)),
+                                   (tiles, at + rows, (rows % tt == 1, True))):
             out = torch.zeros(rows, H * Dv, dtype=torch.bfloat16, device=dev)
             hops.window_attn(q, kc, vt, bt, ts, pos, H, G, m["scale"], 0, None, out, t, max_keys, gate=src,
-                             gate_off=H * D + G * D + G * Dv)
+                             gate_off=H * D + G * D + G * Dv, kinds=kinds)
             outs.append(out.float().cpu())
         for o in outs[1:]:
             assert (o - outs[0]).abs().max() < 0.03 * want.abs().max()
@@ -363,6 +365,88 @@ def test_head_gated_attention_matrix_cores(H, G, D, Dv, rot, n):
         at += rows
     assert at == n
     assert (got.double() - want).abs().max() < 0.05 * want.abs().max()
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("H,G,D,Dv,window,shared,lengths", [
+    (8, 2, 32, 48, 0, False, (300, 70)), (4, 4, 64, 20, 129, False, (700, 5)), (32, 1, 48, 96, 0, False, (90, 33)),
+    (16, 2, 128, 128, 0, False, (900, 41)), (6, 3, 96, 96, 1, False, (150, 150)), (8, 2, 128, 256, 200, False, (500, 65)),
+    (2, 1, 256, 256, 0, False, (300, 1)), (12, 4, 80, 130, 33, False, (260, 97)), (6, 3, 48, 40, 0, True, (200, 47)),
+    (20, 1, 64, 64, 50, False, (120, 1))])
+def test_attention_of_prompt_portions(H, G, D, Dv, window, shared, lengths):
+    """The wave-per-item attention (bf16) against the vector kernel and a direct softmax: two sequences side by side in
+    unequal portions and single tokens, whole tiles and ends of tiles, windows whose edges fall inside blocks, a sink,
+    head gates, an output scale, whole key rows, loud keys on the windows' edges and one outside."""
+    from kafka_llm_service_amd.models.budurax import SegMeta
+
+    dev = "cuda:0"
+    g = torch.Generator().manual_seed(H * D + Dv)
+    Dq = G * D if shared else D
+    tt, w = hops.sig_tile_tokens(H, G), window or 10 ** 6
+    data = []
+    for n in lengths:
+        q, k = 0.5 * torch.randn(n, H, Dq, generator=g), torch.randn(n, G, D, generator=g)
+        v, gate = torch.randn(n, G, Dv, generator=g), torch.randn(n, H + 3, generator=g)
+        for i, (at, key) in enumerate([(n - 1, 0), (n - 1, n - 1), (n - 1, max(0, n - w)), (n - 1, max(0, n - 1 - w)),
+                                       (n // 2, max(0, n // 2 - w + 1)), (n // 2 + 1, max(0, n // 2 + 1 - w)),
+                                       (n // 2, n // 3), (min(33, n - 1), min(32, n - 1))]):
+            h, at = i % H, min(at, n - 1)
+            if shared:
+                q[at, h] = 1.5 * k[min(key, at)].reshape(-1) / G ** 0.5
+            else:
+                q[at, h] = 1.5 * k[min(key, at), h // (H // G)]
+        data.append([x.to(torch.bfloat16) for x in (q, k, v, gate)])
+    sink, scale = torch.randn(H, generator=g), 1.5 * Dq ** -0.5
+    want = []
+    for q, k, v, gate in data:
+        n = q.shape[0]
+        kk = k.double().reshape(n, 1, -1).expand(n, H, -1) if shared else k.double().repeat_interleave(H // G, 1)
+        s = torch.einsum("ihd,jhd->hij", q.double(), kk) * scale
+        ok = plain.visible(n, window or None)
+        s = torch.cat([s.masked_fill(~ok, float("-inf")), sink.double().view(H, 1, 1).expand(H, n, 1)], 2)
+        o = torch.einsum("hij,jhv->ihv", torch.softmax(s, -1)[:, :, :n], v.double().repeat_interleave(H // G, 1))
+        want.append((0.6 * o * torch.sigmoid(gate[:, 2:2 + H].double())[:, :, None]).reshape(n, -1))
+    pg = Paged(dev, lengths, seed=3)
+    kc = torch.zeros(pg.n_pages, 16, G * D, dtype=torch.bfloat16, device=dev)
+    vt = torch.zeros(pg.n_pages, G * Dv, 16, dtype=torch.bfloat16, device=dev)
+    at, got, seen = [0, 0], [[], []], set()
+    cuts = ((1, 2), (tt + 1, 3), (10 ** 6, 1), (0, 10 ** 6))
+    for step, (a, b) in enumerate(cuts):
+        left = [lengths[0] - at[0], lengths[1] - at[1]]
+        take = [min(a, max(0, left[0] - (0 if step >= 2 else 2))), min(b, left[1])]
+        runs = [(s, at[s], take[s]) for s in (0, 1) if take[s]]
+        if not runs:
+            continue
+        bt, ts, pos, sl = pg.step(runs)
+        rows = [torch.cat([data[s][x][p:p + m] for s, p, m in runs]).to(dev) for x in range(4)]
+        T = rows[0].shape[0]
+        hops.kv_store(torch.cat([rows[1].reshape(T, -1), rows[2].reshape(T, -1)], 1), 0, G * D, kc, vt, sl)
+        q0, segs, tiles = 0, [], []
+        for j, (s, p, m) in enumerate(runs):
+            segs.append((q0, m, p, 0))
+            tiles += [(q0 + x, min(tt, m - x), j, 0) for x in range(0, m, tt)]
+            q0 += m
+        seg = torch.tensor(segs, dtype=torch.int32, device=dev)
+        kinds = SegMeta(T, len(runs), seg, ts, bt, seg_host=np.asarray(segs)).tile_kinds(tt)
+        seen.add(kinds)
+        qq = rows[0].reshape(T, -1).contiguous()
+        assert hops.window_attn_mfma_ok(qq, kc, vt, H, G, shared)
+        tl, outs = torch.tensor(tiles, dtype=torch.int32, device=dev), []
+        for t, kd in ((None, (True, False)), (tl, kinds)):
+            wide = torch.zeros(T, H * Dv + 6, dtype=torch.bfloat16, device=dev)
+            hops.window_attn(qq, kc, vt, bt, ts, pos, H, G, scale, window, sink.to(dev), wide[:, :H * Dv], t,
+                             max(p + m for _, p, m in runs), shared, 0.6, rows[3], 2, kd)
+            assert float(wide[:, H * Dv:].abs().max()) == 0.0
+            outs.append(wide[:, :H * Dv].float().cpu())
+        assert (outs[0] - outs[1]).abs().max() < 0.02 * max(x.abs().max() for x in want), kinds
+        q0 = 0
+        for s, p, m in runs:
+            got[s].append(outs[1][q0:q0 + m])
+            at[s] += m
+            q0 += m
+    assert tuple(at) == tuple(lengths) and any(k[1] for k in seen)
+    for s in (0, 1):
+        assert (torch.cat(got[s]).double() - want[s]).abs().max() < 0.03 * want[s].abs().max(), s
 
 
 def _latent_case(g, n, H, D, Dv, R, spots):
