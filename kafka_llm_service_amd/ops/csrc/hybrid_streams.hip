@@ -577,9 +577,10 @@ __global__ __launch_bounds__(256, NKS * 4 + NVT * 16 <= 96 ? 2 : 1) void window_
     const float* __restrict__ sink, const bf16* __restrict__ gate, int64_t gs, bf16* __restrict__ out, int64_t os,
     float out_scale, int min_tok, bool vec4) {
   const int lane = threadIdx.x & 63, lr = lane & 31, lh = lane >> 5;
-  const int item = n_items - 1 - ((int)blockIdx.y * (int)(blockDim.x >> 6) + (int)(threadIdx.x >> 6));
+  const int item = __builtin_amdgcn_readfirstlane(
+      n_items - 1 - ((int)blockIdx.y * (int)(blockDim.x >> 6) + (int)(threadIdx.x >> 6)));
   if (item < 0) return;   // whole waves leave; nothing below synchronises across waves
-  const int t0 = items[4 * item], ntok = items[4 * item + 1], sg = items[4 * item + 2];
+  const int t0 = items[4 * item], ntok = items[4 * item + 1], sg = items[4 * item + 2];   // (uniform)
   if (ntok < min_tok) return;
   const int g = blockIdx.x, rep = H / G, nks = D >> 4, nrows = ntok * rep;
   const bool live = lr < nrows;
@@ -595,9 +596,11 @@ __global__ __launch_bounds__(256, NKS * 4 + NVT * 16 <= 96 ? 2 : 1) void window_
     if (ks >= nks) qf[ks] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
   }
   const int krow = (lr & 19) | ((lr & 4) << 1) | ((lr & 8) >> 1);   // bits 2 and 3 swapped
-  auto fetch_keys = [&](int kb) {
-    const int key = min(32 * kb + krow, maxpos);   // past the item's last position: a valid row, masked below
-    const bf16* kp = kc + ((int64_t)btr[key >> 4] * PAGE + (key & 15)) * Ck + (int64_t)g * kstep + 8 * lh;
+  // the two pages of a block (past the item's last position: the last valid one, masked below)
+  const int lastpg = maxpos >> 4;
+  auto page_of = [&](int kb, int pg) { return btr[min(2 * kb + pg, lastpg)]; };
+  auto fetch_keys = [&](int pa, int pb) {
+    const bf16* kp = kc + ((int64_t)(krow & 16 ? pb : pa) * PAGE + (krow & 15)) * Ck + (int64_t)g * kstep + 8 * lh;
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks) kf[ks] = load_bf16x8(kp + 16 * min(ks, nks - 1));
   };
@@ -608,13 +611,14 @@ __global__ __launch_bounds__(256, NKS * 4 + NVT * 16 <= 96 ? 2 : 1) void window_
 #pragma unroll
     for (int i = 0; i < 16; ++i) O[v][i] = 0.f;
   const int kb0 = window > 0 ? max(0, minpos - window + 1) >> 5 : 0, kb1 = (maxpos >> 5) + 1;
-  fetch_keys(kb0);
+  int pa = page_of(kb0, 0), pb = page_of(kb0, 1), na = page_of(kb0 + 1, 0), nb = page_of(kb0 + 1, 1);
+  fetch_keys(pa, pb);
   for (int kb = kb0; kb < kb1; ++kb) {
+    const int fa = page_of(kb + 2, 0), fb = page_of(kb + 2, 1);   // (two blocks ahead)
     bf16x8 vf[2][NVT];
 #pragma unroll
     for (int pg = 0; pg < 2; ++pg) {
-      // a page past the last position: the last valid one, its weights are zero
-      const bf16* vp = vt + ((int64_t)btr[min(2 * kb + pg, maxpos >> 4)] * Cv + (int64_t)g * Dv) * PAGE + 8 * lh;
+      const bf16* vp = vt + ((int64_t)(pg ? pb : pa) * Cv + (int64_t)g * Dv) * PAGE + 8 * lh;
 #pragma unroll
       for (int v = 0; v < NVT; ++v) vf[pg][v] = load_bf16x8(vp + (int64_t)min(32 * v + lr, Dv - 1) * PAGE);
     }
@@ -623,7 +627,11 @@ __global__ __launch_bounds__(256, NKS * 4 + NVT * 16 <= 96 ? 2 : 1) void window_
     for (int i = 0; i < 16; ++i) S[i] = 0.f;
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks) S = mfma32(kf[ks], qf[ks], S);
-    if (kb + 1 < kb1) fetch_keys(kb + 1);
+    fetch_keys(na, nb);
+    pa = na;
+    pb = nb;
+    na = fa;
+    nb = fb;
     float s[16];
 #pragma unroll
     for (int i = 0; i < 16; ++i) s[i] = S[i] * scale_log2e;
