@@ -66,6 +66,11 @@ class MoEBlock:
             out = torch.zeros(T, d, dtype=torch.float32, device=x.device)
             ops.grouped_stream_combine(a, lw.w2_t, r, T, out, e_lo=self.e0)
             return self._finish(out, x.dtype)
+        if self.model.stream and lw.w13_t is not None and self.ep == 1 and d % 128 == 0 and self.F % 128 == 0:
+            # long steps on the same tiled weights: 128-row tiles (csrc/moe_wide.hip)
+            a = ops.grouped_wide(x, lw.w13_t, r, "glu", True)
+            out = torch.zeros(T, d, dtype=torch.float32, device=x.device)
+            return self._finish(ops.grouped_wide(a, lw.w2_t, r, "combine", False, out), x.dtype)
         # gate_up for every (token, expert) entry routed to a local expert, rows gathered from x by the kernel
         h = ops.grouped_gemm(x, lw.w13, r, gather=True, e_lo=self.e0)
         a = ops.silu_mul(h)
