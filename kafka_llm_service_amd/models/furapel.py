@@ -23,8 +23,9 @@ Experts           router logits in fp32, softmax over all of them, the ``top`` l
 
 How the engine runs it. A layer's projections of norm1(x) are one GEMM. The add to the residual, both norms of the next
 layer and, in front of a pass, the residual's copy into the loop product's input are one element-wise kernel, which also
-sums a split-K projection's slabs and, in long steps, gathers every token's expert rows. The head gates are applied by the attention kernels as they write their output. The
-squared relu is part of the expert products. Long portions run the matrix memory in chunks of matrix products.
+sums a split-K projection's slabs and, in long steps, gathers every token's expert rows. The head gates are applied by the
+attention kernels as they write their output. The squared relu is part of the expert products. Long portions run the
+matrix memory in chunks of matrix products.
 
 Per sequence the engine keeps, for every layer RUN (a looped layer counts once per pass), pages (keys and page-wise
 transposed values, or latent rows; page ids shared by all runs) or a slot of matrix-memory state (S, n, m). The residual,

@@ -450,10 +450,17 @@ hipError_t kafka_launch_grouped_wide(const bf16* X, int64_t ldx, const bf16* Wt,
   auto a = [&](auto kern) {
     kern<<<grid, 256, 0, st>>>(X, ldx, wt, E, N, K, perm_tok, perm_w, expert_off, Y, ldy, out, ldo, glu_limit, glu_alpha);
   };
-  if (epi == EPI_GLU) { if (gather) a(grouped_wide_kernel<true, EPI_GLU>); else a(grouped_wide_kernel<false, EPI_GLU>); }
-  else if (epi == EPI_RELU2) { if (gather) a(grouped_wide_kernel<true, EPI_RELU2>); else a(grouped_wide_kernel<false, EPI_RELU2>); }
-  else if (epi == EPI_ROWS) { if (gather) a(grouped_wide_kernel<true, EPI_ROWS>); else a(grouped_wide_kernel<false, EPI_ROWS>); }
-  else { if (gather) a(grouped_wide_kernel<true, EPI_COMBINE>); else a(grouped_wide_kernel<false, EPI_COMBINE>); }
+  if (gather) {
+    if (epi == EPI_GLU) a(grouped_wide_kernel<true, EPI_GLU>);
+    else if (epi == EPI_RELU2) a(grouped_wide_kernel<true, EPI_RELU2>);
+    else if (epi == EPI_ROWS) a(grouped_wide_kernel<true, EPI_ROWS>);
+    else a(grouped_wide_kernel<true, EPI_COMBINE>);
+  } else {
+    if (epi == EPI_GLU) a(grouped_wide_kernel<false, EPI_GLU>);
+    else if (epi == EPI_RELU2) a(grouped_wide_kernel<false, EPI_RELU2>);
+    else if (epi == EPI_ROWS) a(grouped_wide_kernel<false, EPI_ROWS>);
+    else a(grouped_wide_kernel<false, EPI_COMBINE>);
+  }
   return hipGetLastError();
 }
 
